@@ -894,3 +894,308 @@ class NatatarConfig:
         if self.streams:
             raw["streams"] = self.streams
         return raw
+
+
+# ---- Teberax ------------------------------------------------------------------------------------------
+
+
+@dataclass(frozen=True)
+class TeberaxRotation:
+    """Neighbouring pairs of a head's first `dims` coordinates turn; `factor` divides every frequency."""
+
+    dims: int
+    base: float
+    factor: float = 1.0
+
+    @classmethod
+    def from_dict(cls, raw, where: str):
+        if not raw or not raw.get("dims"):
+            return None
+        scaling = raw.get("scaling")
+        factor = float(_need(scaling, "factor", where + "scaling.")) if scaling else 1.0
+        return cls(int(raw["dims"]), float(_need(raw, "base", where)), factor)
+
+    def to_dict(self) -> dict:
+        raw = {"dims": self.dims, "base": self.base}
+        if self.factor != 1.0:
+            raw["scaling"] = {"factor": self.factor}
+        return raw
+
+
+@dataclass(frozen=True)
+class TeberaxMask:
+    """The keys a position sees: the last `size` (0: all), and with a window those of the first `keep_first` tokens."""
+
+    size: int = 0
+    keep_first: int = 0
+
+    @classmethod
+    def from_dict(cls, raw) -> "TeberaxMask":
+        raw = raw or {}
+        return cls(int(raw.get("size") or 0), int(raw.get("keep_first") or 0))
+
+    def to_dict(self) -> dict:
+        return {"size": self.size, "keep_first": self.keep_first} if self.keep_first else {"size": self.size}
+
+
+@dataclass(frozen=True)
+class TeberaxAttention:
+    """A differential attention's sizes and constants (a layer's mixer "attention"): two maps of `dim` over values of
+    `vdim`.  kv_from >= 0: the layer has no keys and values of its own and reads that layer's."""
+
+    heads: int
+    kv_heads: int
+    dim: int
+    vdim: int
+    scale: float
+    diff: float
+    mask: TeberaxMask
+    kv_from: int = -1
+
+    @classmethod
+    def from_dict(cls, raw: dict, where: str) -> "TeberaxAttention":
+        return cls(*(int(_need(raw, k, where)) for k in ("heads", "kv_heads", "dim", "vdim")),
+                   scale=float(_need(raw, "scale", where)), diff=float(_need(raw, "diff", where)),
+                   mask=TeberaxMask.from_dict(raw.get("mask")),
+                   kv_from=int(raw["kv_from"]) if raw.get("kv_from") is not None else -1)  # fmt: skip
+
+    def to_dict(self) -> dict:
+        raw = {"heads": self.heads, "kv_heads": self.kv_heads, "dim": self.dim, "vdim": self.vdim, "scale": self.scale,
+               "diff": self.diff}  # fmt: skip
+        if self.mask.size:
+            raw["mask"] = self.mask.to_dict()
+        if self.kv_from >= 0:
+            raw["kv_from"] = self.kv_from
+        return raw
+
+
+@dataclass(frozen=True)
+class TeberaxSinkAttention:
+    """The left half of a "parallel" mixer: a biased, rotary attention with capped scores and a sink."""
+
+    heads: int
+    kv_heads: int
+    dim: int
+    vdim: int
+    scale: float
+    softcap: float  # 0: scores are not capped
+    rot: object  # TeberaxRotation or None
+    mask: TeberaxMask
+
+    @classmethod
+    def from_dict(cls, raw: dict, where: str) -> "TeberaxSinkAttention":
+        return cls(*(int(_need(raw, k, where)) for k in ("heads", "kv_heads", "dim", "vdim")),
+                   scale=float(_need(raw, "scale", where)), softcap=float(raw.get("softcap") or 0.0),
+                   rot=TeberaxRotation.from_dict(raw.get("rot"), where + "rot."), mask=TeberaxMask.from_dict(raw.get("mask")))  # fmt: skip
+
+    def to_dict(self) -> dict:
+        raw = {"heads": self.heads, "kv_heads": self.kv_heads, "dim": self.dim, "vdim": self.vdim, "scale": self.scale}
+        if self.softcap:
+            raw["softcap"] = self.softcap
+        if self.rot:
+            raw["rot"] = self.rot.to_dict()
+        if self.mask.size:
+            raw["mask"] = self.mask.to_dict()
+        return raw
+
+
+@dataclass(frozen=True)
+class TeberaxLinear:
+    """The right half of a "parallel" mixer: a gated linear attention with a decay per key channel.  The rank of the
+    decays' two-step projection is a size that only the checkpoint's shapes tell: a configuration read from a model
+    folder is completed from them, one written by this package names it itself."""
+
+    heads: int
+    dim: int
+    vdim: int
+    tau: float
+    rank: int = 0
+
+    @classmethod
+    def from_dict(cls, raw: dict, where: str) -> "TeberaxLinear":
+        return cls(*(int(_need(raw, k, where)) for k in ("heads", "dim", "vdim")), tau=float(_need(raw, "tau", where)),
+                   rank=int(raw.get("rank", 0)))  # fmt: skip
+
+    def to_dict(self) -> dict:
+        return {"heads": self.heads, "dim": self.dim, "vdim": self.vdim, "tau": self.tau, "rank": self.rank}
+
+
+@dataclass(frozen=True)
+class TeberaxParallel:
+    left: TeberaxSinkAttention
+    right: TeberaxLinear
+
+    @classmethod
+    def from_dict(cls, raw: dict, where: str) -> "TeberaxParallel":
+        return cls(TeberaxSinkAttention.from_dict(_need(raw, "left", where), where + "left."),
+                   TeberaxLinear.from_dict(_need(raw, "right", where), where + "right."))  # fmt: skip
+
+    def to_dict(self) -> dict:
+        return {"left": self.left.to_dict(), "right": self.right.to_dict()}
+
+
+@dataclass(frozen=True)
+class TeberaxLatent:
+    """An attention through a cached latent whose queries are a plain projection."""
+
+    heads: int
+    dim: int  # coordinates of a query/key head that do not turn
+    rot_dim: int  # and those that do
+    vdim: int
+    kv_rank: int
+    scale: float
+    rot: object  # TeberaxRotation or None (rot_dim 0)
+    mask: TeberaxMask
+
+    @classmethod
+    def from_dict(cls, raw: dict, where: str) -> "TeberaxLatent":
+        rot_dim = int(raw.get("rot_dim") or 0)
+        rot = TeberaxRotation.from_dict(raw.get("rot"), where + "rot.") if rot_dim else None
+        if rot_dim and (rot is None or rot.dims != rot_dim):
+            raise ConfigError(f"{where}rot.dims must equal rot_dim")
+        return cls(int(_need(raw, "heads", where)), int(_need(raw, "dim", where)), rot_dim, int(_need(raw, "vdim", where)),
+                   int(_need(raw, "kv_rank", where)), float(_need(raw, "scale", where)), rot, TeberaxMask.from_dict(raw.get("mask")))  # fmt: skip
+
+    def to_dict(self) -> dict:
+        raw = {"heads": self.heads, "dim": self.dim, "rot_dim": self.rot_dim, "vdim": self.vdim, "kv_rank": self.kv_rank,
+               "scale": self.scale}  # fmt: skip
+        if self.rot:
+            raw["rot"] = self.rot.to_dict()
+        if self.mask.size:
+            raw["mask"] = self.mask.to_dict()
+        return raw
+
+
+@dataclass(frozen=True)
+class TeberaxFeedForward:
+    kind: str  # "dense" (without a gate) or "moe" (gated experts)
+    ff: int  # width inside the feed-forward (of one expert for "moe")
+    experts: int = 0
+    top: int = 0
+    identity: int = 0  # router outputs behind the experts' whose output is the input itself
+
+    @classmethod
+    def from_dict(cls, raw: dict, where: str) -> "TeberaxFeedForward":
+        kind = _need(raw, "kind", where)
+        if kind == "dense":
+            return cls("dense", int(_need(raw, "ff", where)))
+        if kind == "moe":
+            router = _need(raw, "router", where)
+            return cls("moe", int(_need(_need(raw, "expert", where), "ff", where + "expert.")),
+                       int(_need(router, "experts", where + "router.")), int(_need(router, "top", where + "router.")),
+                       int(router.get("identity") or 0))  # fmt: skip
+        raise ConfigError(f"{where}kind={kind!r} is not supported ('dense' or 'moe')")
+
+    def to_dict(self) -> dict:
+        if self.kind == "dense":
+            return {"kind": "dense", "ff": self.ff}
+        router = {"experts": self.experts, "top": self.top}
+        if self.identity:
+            router["identity"] = self.identity
+        return {"kind": "moe", "expert": {"ff": self.ff}, "router": router}
+
+
+@dataclass(frozen=True)
+class TeberaxLayer:
+    type: str  # "attention", "parallel" or "latent_attention"
+    mixer: object
+    mlp: object  # TeberaxFeedForward or None
+
+
+@dataclass(frozen=True)
+class TeberaxConfig:
+    """A Teberax decoder: layers with a norm before and after each sublayer (every norm has one number as its gain); mixers
+    of three kinds (a differential attention that may read an earlier layer's keys and values, a rotary attention with
+    capped scores and a sink beside a gated linear attention, an attention through a latent over a window); feed-forwards
+    without a gate whose activation is a polynomial of normed powers, or gated experts chosen by corrected softmax scores,
+    some of which are the input itself; a normed embedding, a head of its own, capped logits."""
+
+    vocab_size: int
+    hidden_size: int
+    norm_eps: float
+    layers: tuple  # of TeberaxLayer
+    logit_softcap: float = 0.0  # 0: logits are not capped
+
+    architecture = "Teberax"
+    MIXERS = {"attention": TeberaxAttention, "parallel": TeberaxParallel, "latent_attention": TeberaxLatent}
+
+    @classmethod
+    def from_dict(cls, raw: dict) -> "TeberaxConfig":
+        _require(raw, ["vocab", "width", "layers", "norm"])
+        layers = []
+        for i, entry in enumerate(raw["layers"]):
+            where = f"layers[{i}]."
+            kind = _need(entry, "type", where)
+            if kind not in cls.MIXERS:
+                raise ConfigError(f"{where}type={kind!r} is not supported (one of {', '.join(cls.MIXERS)})")
+            mixer = cls.MIXERS[kind].from_dict(_need(entry, "mixer", where), where + "mixer.")
+            mlp = entry.get("mlp")
+            layers.append(TeberaxLayer(kind, mixer, None if mlp is None else TeberaxFeedForward.from_dict(mlp, where + "mlp.")))
+        cfg = cls(
+            vocab_size=int(raw["vocab"]),
+            hidden_size=int(raw["width"]),
+            norm_eps=float(_need(raw["norm"], "eps", "norm.")),
+            layers=tuple(layers),
+            logit_softcap=float(raw.get("logit_softcap") or 0.0),
+        )
+        cfg.validate()
+        return cfg
+
+    def validate(self) -> None:
+        if self.vocab_size < 1 or self.hidden_size < 1 or not self.layers:
+            raise ConfigError("vocab, width and the number of layers must be positive")
+        if not self.norm_eps > 0:
+            raise ConfigError("norm.eps must be positive")
+        if self.logit_softcap < 0:
+            raise ConfigError("logit_softcap is not negative")
+        for i, layer in enumerate(self.layers):
+            m, at = layer.mixer, f"layers[{i}]"
+            attention = m.left if layer.type == "parallel" else m
+            if min(attention.mask.size, attention.mask.keep_first) < 0:
+                raise ConfigError(f"{at}: mask.size and mask.keep_first are not negative")
+            if layer.type == "latent_attention":
+                if min(m.heads, m.dim, m.vdim, m.kv_rank) < 1 or m.rot_dim < 0 or m.rot_dim % 2:
+                    raise ConfigError(f"{at}: sizes must be positive and rot_dim even")
+            elif min(attention.heads, attention.kv_heads, attention.dim, attention.vdim) < 1 or attention.heads % attention.kv_heads:
+                raise ConfigError(f"{at}: head counts and sizes must be positive, heads a multiple of kv_heads")
+            rot = getattr(attention, "rot", None)
+            if rot is not None:
+                most = m.rot_dim if layer.type == "latent_attention" else attention.dim
+                if rot.dims < 2 or rot.dims % 2 or rot.dims > most or not rot.base > 1 or not rot.factor > 0:
+                    raise ConfigError(f"{at}: rot.dims is even and at most the head's, rot.base exceeds 1, scaling.factor is positive")
+            if layer.type == "parallel":
+                if attention.softcap < 0:
+                    raise ConfigError(f"{at}: softcap is not negative")
+                if min(m.right.heads, m.right.dim, m.right.vdim) < 1 or not m.right.tau > 0:
+                    raise ConfigError(f"{at}: the linear attention's head count, sizes and tau must be positive")
+            if layer.type == "attention" and m.kv_from >= 0:
+                src = self.layers[m.kv_from] if m.kv_from < i else None
+                if src is None or src.type != "attention" or src.mixer.kv_from >= 0:
+                    raise ConfigError(f"{at}: kv_from names an earlier attention layer with keys and values of its own")
+                s = src.mixer
+                if (s.heads, s.kv_heads, s.dim, s.vdim) != (m.heads, m.kv_heads, m.dim, m.vdim):
+                    raise ConfigError(f"{at}: head counts and sizes must equal those of layer {m.kv_from}, whose keys it reads (kv_from)")
+            f = layer.mlp
+            if f is not None and (f.ff < 1 or (f.kind == "moe" and (f.experts < 1 or f.identity < 0 or not 1 <= f.top <= f.experts + f.identity))):
+                raise ConfigError(f"{at}.mlp: sizes must be positive and top at most the number of experts")
+
+    def completed(self, shape_of) -> "TeberaxConfig":
+        """This configuration with the sizes that only tensors tell: shape_of(checkpoint name) -> shape or None."""
+        layers = []
+        for i, layer in enumerate(self.layers):
+            m = layer.mixer
+            if layer.type == "parallel":
+                first = shape_of(f"l{i}.mix.right.a1")
+                m = replace(m, right=replace(m.right, rank=int(first[0]) if first else m.right.rank))
+            layers.append(replace(layer, mixer=m))
+        return replace(self, layers=tuple(layers))
+
+    def to_dict(self) -> dict:
+        """The config.json that `from_dict` reads back to this object."""
+        layers = [{"type": layer.type, "mixer": layer.mixer.to_dict(), "mlp": None if layer.mlp is None else layer.mlp.to_dict()}
+                  for layer in self.layers]  # fmt: skip
+        raw = {"architecture": self.architecture, "vocab": self.vocab_size, "width": self.hidden_size,
+               "norm": {"eps": self.norm_eps}, "layers": layers}  # fmt: skip
+        if self.logit_softcap:
+            raw["logit_softcap"] = self.logit_softcap
+        return raw

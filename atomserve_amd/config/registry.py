@@ -91,3 +91,4 @@ def _load_builtin() -> None:
     import atomserve_amd.models.mumizen  # noqa: F401
     import atomserve_amd.models.natatar  # noqa: F401
     import atomserve_amd.models.qwen3  # noqa: F401
+    import atomserve_amd.models.teberax  # noqa: F401

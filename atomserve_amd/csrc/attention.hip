@@ -3,8 +3,8 @@
 // Cache pages of one layer: k_pages [num_pages, KV, block_size, D] and v_pages
 // [num_pages, KV, D, block_size] (values transposed within a page); a token at position p
 // of a request lives in page table[p / block_size] at offset p % block_size.  A query at position p sees the keys at positions lo..p, with
-// lo = max(0, p - window + 1) if window > 0, else 0.  Query head h reads kv head
-// h / (H / KV).  Scores, softmax and the weighted sum are fp32.
+// lo = max(0, p - window + 1) if window > 0, else 0, and beside a window the first `keep` of the sequence (`Sight`).
+// Query head h reads kv head h / (H / KV).  Scores, softmax and the weighted sum are fp32.
 //
 // attn_single_query: one work item per query token.  A workgroup (4 waves) takes one
 // token, one kv head, up to GT query heads of its group, and one partition of
@@ -23,6 +23,26 @@
 template <typename T> __device__ __forceinline__ float fexp(float x);
 template <> __device__ __forceinline__ float fexp<float>(float x) { return expf(x); }
 template <> __device__ __forceinline__ float fexp<bf16>(float x) { return __expf(x); }
+
+// What a query at position p sees, and how scores become weights.
+struct Sight {
+  int window;  // > 0: keys p - window + 1 .. p; 0: every key up to p
+  int keep;    // with a window: the sequence's first `keep` keys stay visible behind it
+  float cap;   // > 0: a score s counts as cap tanh(s / cap)
+  int sink;    // 1: the denominator has one more score, of 0, which has no value
+};
+__device__ __forceinline__ int first_in_window(const Sight& sight, int ctx) {
+  return sight.window > 0 ? max(0, ctx - sight.window) : 0;
+}
+static inline bool sight_ok(const Sight& s) {
+  return s.window >= 0 && s.keep >= 0 && (s.keep == 0 || s.window > 0) && s.cap >= 0.f && (s.sink == 0 || s.sink == 1);
+}
+
+// tanh through the hardware's exponential and reciprocal: an absolute error of 1e-7, which is what a capped score
+// (times the cap) of the bf16 kernels may carry.
+__device__ __forceinline__ float quick_tanh(float x) {
+  return 1.f - 2.f * __builtin_amdgcn_rcpf(1.f + __builtin_amdgcn_exp2f(2.8853900817779268f * x));
+}
 
 template <typename T> struct Chunk;  // 16 bytes of a head
 template <> struct Chunk<float> {
@@ -51,7 +71,7 @@ __global__ __launch_bounds__(256) void attn_single_query_kernel(
     const int* __restrict__ items, const int* __restrict__ positions, const int* __restrict__ tok_row,
     const int* __restrict__ block_tables, int table_width, T* __restrict__ out,
     float* __restrict__ part_m, float* __restrict__ part_l, float* __restrict__ part_acc, int H, int KV,
-    int D, int bs, float scale, int window, int part_size, int P, int lpk) {
+    int D, int bs, float scale, Sight sight, int part_size, int P, int lpk) {
   constexpr int CH = Chunk<T>::N;
   extern __shared__ float smem[];  // [4][GT] m, [4][GT] l, [4][GT][D] acc
   const int G = H / KV;
@@ -60,8 +80,9 @@ __global__ __launch_bounds__(256) void attn_single_query_kernel(
   const int t = items ? items[item] : item;  // null: every token, in order
   const int pos = positions[t];
   const int ctx = pos + 1;
-  const int lo = window > 0 ? max(0, ctx - window) : 0;
-  const int k0 = max(lo, part * part_size), k1 = min(ctx, (part + 1) * part_size);
+  // the visible keys in order, the kept first ones and then the window's: partitions cut this list
+  const int lo = first_in_window(sight, ctx), kept = min(sight.keep, lo);
+  const int k0 = part * part_size, k1 = min(kept + ctx - lo, (part + 1) * part_size);
   const int h0 = kvh * G + hc * GT;       // first query head of this workgroup
   const int ng = min(GT, G - hc * GT);    // valid heads among the GT
   const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
@@ -107,8 +128,9 @@ __global__ __launch_bounds__(256) void attn_single_query_kernel(
   const int stride = 4 * nsub;
   const int iters = (k1 - k0 + stride - 1) / stride;  // uniform over the workgroup
   for (int it = 0; it < iters; ++it) {
-    const int key = k0 + it * stride + wave * nsub + sub;
-    const bool valid = key < k1;
+    const int place = k0 + it * stride + wave * nsub + sub;
+    const bool valid = place < k1;
+    const int key = place < kept ? place : place - kept + lo;
     float kv[CH], vv[CH];
     if (valid && active) {
       const int page = table[key / bs];
@@ -128,7 +150,7 @@ __global__ __launch_bounds__(256) void attn_single_query_kernel(
 #pragma unroll
       for (int c = 0; c < CH; ++c) d += qr[g][c] * kv[c];
       for (int off = 1; off < lpk; off <<= 1) d += __shfl_xor(d, off, WAVE);
-      s[g] = d;
+      s[g] = sight.cap > 0.f ? sight.cap * tanhf(d / sight.cap) : d;
     }
     if (valid) {
 #pragma unroll
@@ -192,6 +214,11 @@ __global__ __launch_bounds__(256) void attn_single_query_kernel(
     }
     const int h = h0 + g;
     if (P == 1) {
+      if (sight.sink) {
+        const float top = fmaxf(mx, 0.f), e = fexp<T>(mx - top);
+        num *= e;
+        den = den * e + fexp<T>(-top);
+      }
       out[((size_t)t * H + h) * D + d] = from_f32<T>(num / den);
     } else {
       const size_t o = ((size_t)item * H + h) * P + part;
@@ -211,12 +238,13 @@ __global__ __launch_bounds__(256) void attn_reduce_kernel(const int* __restrict_
                                                           const float* __restrict__ part_m,
                                                           const float* __restrict__ part_l,
                                                           const float* __restrict__ part_acc, T* __restrict__ out,
-                                                          int H, int D, int P) {
+                                                          int H, int D, int P, int sink) {
   const int item = blockIdx.x, h = blockIdx.y;
   const size_t base = ((size_t)item * H + h) * P;
   float mx = NEG_INF;
   for (int p = 0; p < P; ++p) mx = fmaxf(mx, part_m[base + p]);
-  float den = 0.f;
+  if (sink) mx = fmaxf(mx, 0.f);
+  float den = sink ? fexp<T>(-mx) : 0.f;
   for (int p = 0; p < P; ++p) {
     const float mp = part_m[base + p];
     den += (mp == NEG_INF) ? 0.f : part_l[base + p] * fexp<T>(mp - mx);
@@ -360,12 +388,12 @@ __device__ __forceinline__ void load_gains8(const bf16* w, float* g) {
   for (int j = 0; j < 8; ++j) g[j] = (float)v[j];
 }
 
-template <int DC, int FRESH>  // D / 32; FRESH 0: finished queries, 1: qkv with bf16 gains, 2: with fp32 gains
+template <int DC, int FRESH, bool CAP>  // D / 32; FRESH 0: finished queries, 1: qkv with bf16 gains, 2: with fp32 gains
 __global__ __launch_bounds__(256) void attn_decode_mfma_kernel(
     const bf16* __restrict__ q, const bf16* __restrict__ k_pages, const bf16* __restrict__ v_pages,
     const int* __restrict__ items, const int* __restrict__ positions, const int* __restrict__ tok_row,
     const int* __restrict__ block_tables, int table_width, bf16* __restrict__ out, float* __restrict__ part_m,
-    float* __restrict__ part_l, float* __restrict__ part_acc, int H, int KV, int bs, float scale, int window,
+    float* __restrict__ part_l, float* __restrict__ part_acc, int H, int KV, int bs, float scale, Sight sight,
     int part_size, int P, int cus, int share, FreshQKV fresh) {
   // share > 1: every `share` consecutive kv heads named here are one head of the pages (a group of more query heads
   // than a workgroup takes, cut into several); the pages then hold KV / share heads.
@@ -392,14 +420,20 @@ __global__ __launch_bounds__(256) void attn_decode_mfma_kernel(
   const int t = items ? items[item] : item;  // null: every token, in order
   const int pos = positions[t];
   const int ctx = pos + 1;
-  const int lo = window > 0 ? max(0, ctx - window) : 0;
-  const int k0 = max(lo, part * part_size), k1 = min(ctx, (part + 1) * part_size);
+  // The keys are walked in steps of 32: first those that hold kept tokens (`kept_steps` from the sequence's start), then
+  // those of the window (from step `base` on); where the two meet it is one run from the start.  Partitions cut this list.
+  const int lo = first_in_window(sight, ctx), kept = min(sight.keep, lo);
+  int kept_steps = (kept + 31) / 32, base = lo / 32;
+  if (kept_steps > 0 && kept_steps >= base) kept_steps = base = 0;
+  const int steps = kept_steps + (ctx - 1) / 32 - base + 1;
+  const int s0 = part * (part_size / 32), s1 = min(steps, (part + 1) * (part_size / 32));
+  auto first_key = [&](int step) { return 32 * (step < kept_steps ? step : step - kept_steps + base); };
   const int h0 = kvh * G;
   const int page_heads = KV / share, page_head = kvh / share;
   const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
   const int col = lane & 15, grp = lane >> 4;  // col: head within the group (and key row of A)
 
-  if (k0 >= k1) {  // an empty partition (P > 1 only): mark it so for the reduce
+  if (s0 >= s1) {  // an empty partition (P > 1 only): mark it so for the reduce
     if (tid < G) {
       const size_t o = ((size_t)item * H + h0 + tid) * P + part;
       part_m[o] = NEG_INF;
@@ -442,7 +476,7 @@ __global__ __launch_bounds__(256) void attn_decode_mfma_kernel(
 #pragma unroll
       for (int j = 0; j < 4; ++j) angle[c * 4 + j] = cs4[j];
     }
-    fresh_here = fresh.store && pos >= k0 && pos < k1;  // the same for the whole workgroup
+    fresh_here = fresh.store && s1 == steps;  // the same for the whole workgroup
     if (fresh_here && wave == 0) {
       slot = fresh.slots[t];
       const bf16* src = fresh.qkv + (row + H + kvh) * D;
@@ -462,10 +496,8 @@ __global__ __launch_bounds__(256) void attn_decode_mfma_kernel(
       for (int p = 0; p < 2 * PAIRS; ++p) vv[p] = src[min(lane + p * WAVE, D - 1)];
     }
   }
-  const int first = (k0 / 32) * 32;
   KVStep<DC> cur, nxt;
-  int kb = first + 32 * wave;
-  if (kb < k1) load_kv_step<DC>(cur, k_pages, v_pages, table, kb, k1, page_heads, page_head, bs, col, grp);
+  if (s0 + wave < s1) load_kv_step<DC>(cur, k_pages, v_pages, table, first_key(s0 + wave), ctx, page_heads, page_head, bs, col, grp);
 
   if constexpr (FRESH != 0) {
     // the queries of this lane's head: norm over the head (its D values lie in four lanes), rotation
@@ -534,9 +566,10 @@ __global__ __launch_bounds__(256) void attn_decode_mfma_kernel(
   for (int dt = 0; dt < DT; ++dt) o[dt] = f32x4_t{0.f, 0.f, 0.f, 0.f};
   float m = NEG_INF, l = 0.f;
 
-  for (; kb < k1; kb += 128) {
-    const bool more = kb + 128 < k1;
-    if (more) load_kv_step<DC>(nxt, k_pages, v_pages, table, kb + 128, k1, page_heads, page_head, bs, col, grp);
+  for (int step = s0 + wave; step < s1; step += 4) {
+    const int kb = first_key(step);
+    const bool more = step + 4 < s1;
+    if (more) load_kv_step<DC>(nxt, k_pages, v_pages, table, first_key(step + 4), ctx, page_heads, page_head, bs, col, grp);
     if constexpr (FRESH != 0) {
       if (fresh_here && pos >= kb && pos < kb + 32) {  // this wave's step holds the token itself: take it from LDS
         const int at = pos - kb;  // = KEY_OF_ROW(tile, row) for
@@ -573,8 +606,10 @@ __global__ __launch_bounds__(256) void attn_decode_mfma_kernel(
 #pragma unroll
       for (int r = 0; r < 4; ++r) {
         const int key = kb + KEY_OF_ROW(tt, 4 * grp + r);
-        const bool seen = key >= k0 && key < k1;
-        s[tt][r] = seen ? s[tt][r] * scale : NEG_INF;
+        const bool seen = key < ctx && (key >= lo || key < kept);
+        float sc = s[tt][r] * scale;
+        if (CAP) sc = sight.cap * quick_tanh(sc / sight.cap);
+        s[tt][r] = seen ? sc : NEG_INF;
         mx = fmaxf(mx, s[tt][r]);
       }
     mx = quad_rows_max(mx);
@@ -633,6 +668,11 @@ __global__ __launch_bounds__(256) void attn_decode_mfma_kernel(
     }
     const int h = h0 + g;
     if (P == 1) {
+      if (sight.sink) {
+        const float top = fmaxf(mxw, 0.f), e = __expf(mxw - top);
+        num *= e;
+        den = den * e + __expf(-top);
+      }
       out[((size_t)t * H + h) * D + d] = (bf16)(num / den);
     } else {
       const size_t ob = ((size_t)item * H + h) * P + part;
@@ -692,11 +732,13 @@ struct PrefillSplit {
 };
 constexpr int PREFILL_MIN_PIECE_ROUNDS = 2;  // an item's last two rounds hold its own tokens: one piece
 
-template <int DC, int QT>  // D / 32; column tiles of 16 queries that a wave owns: 2, or 1 (see the launcher)
+// With kept first tokens behind a window the rounds of 64 keys are first those from the sequence's start that hold kept
+// tokens, then those of the window (`first_key`); pieces cut this list.
+template <int DC, int QT, bool CAP>  // D / 32; column tiles of 16 queries that a wave owns: 2, or 1 (see the launcher)
 __global__ __launch_bounds__(256, 2) void attn_prefill_mfma_kernel(
     const bf16* __restrict__ q, const bf16* __restrict__ k_pages, const bf16* __restrict__ v_pages,
     const int* __restrict__ tiles, const int* __restrict__ block_tables, int table_width,
-    bf16* __restrict__ out, int H, int KV, int bs, float scale, int window, int units_z, int pass, PrefillSplit split) {
+    bf16* __restrict__ out, int H, int KV, int bs, float scale, Sight sight, int units_z, int pass, PrefillSplit split) {
   constexpr int D = DC * 32, DT = DC * 2;
   constexpr int PIECE = 64 * DC;  // 16-byte slots of a 16-key piece: 16 * D / 8
   typedef unsigned int u32x4_t __attribute__((ext_vector_type(4)));
@@ -730,6 +772,7 @@ __global__ __launch_bounds__(256, 2) void attn_prefill_mfma_kernel(
   const int tok0 = tiles[4 * tile], count = tiles[4 * tile + 1], row = tiles[4 * tile + 2];
   const int pos0 = tiles[4 * tile + 3];
   const int* table = block_tables + (size_t)row * table_width;
+  const int window = sight.window;
 
   // the keys this workgroup walks: from the first key any of its waves sees to the last
   int wg_lo = 0x7fffffff, wg_last = -1;
@@ -744,17 +787,21 @@ __global__ __launch_bounds__(256, 2) void attn_prefill_mfma_kernel(
     if (split.pieces > 1 && piece == 0 && threadIdx.x == 0) split.cut[item] = 1;
     return;
   }
+  const int kept = min(sight.keep, wg_lo);  // kept tokens that lie before every query's window
+  int kept_rounds = (kept + 63) / 64, kb0 = (wg_lo / 32) * 32;
+  if (kept_rounds > 0 && 64 * kept_rounds >= kb0) kept_rounds = kb0 = 0;  // one run from the start
+  int rd_first = 0, rd_end = kept_rounds + ((wg_last - kb0) / 32 + 2) / 2;
+  auto first_key = [&](int rd) { return rd < kept_rounds ? 64 * rd : kb0 + 64 * (rd - kept_rounds); };
   bool partial = false;  // this workgroup leaves its share of a cut item for the merge
   if (split.pieces > 1) {
-    const int kb_first = (wg_lo / 32) * 32, all_rounds = ((wg_last - kb_first) / 32 + 2) / 2;
+    const int all_rounds = rd_end;
     const int mine = min(split.pieces, (all_rounds + split.piece_rounds - 1) / split.piece_rounds);  // pieces of this item
     if (piece == 0 && threadIdx.x == 0) split.cut[item] = mine;
     if (piece >= mine) return;
     if (mine > 1) {
       partial = true;
-      const int from = kb_first + 64 * split.piece_rounds * piece;  // the piece's first key
-      if (piece + 1 < mine) wg_last = from + 64 * split.piece_rounds - 1;
-      if (piece > 0) wg_lo = from;
+      rd_first = split.piece_rounds * piece;
+      if (piece + 1 < mine) rd_end = rd_first + split.piece_rounds;
     }
   }
 
@@ -766,7 +813,7 @@ __global__ __launch_bounds__(256, 2) void attn_prefill_mfma_kernel(
   const int nq = working ? min(WQ, count - q0) : 1;
   const int my_last = working ? pos0 + q0 + nq - 1 : -1;
   const int my_first_q = pos0 + q0;                  // position of this wave's first query
-  const float scale2 = scale * 1.4426950408889634f;  // scores are kept in base 2
+  const float scale2 = CAP ? 1.f : scale * 1.4426950408889634f;  // scores are kept in base 2
   const int my_lo = working ? (window > 0 ? max(0, pos0 + q0 - window + 1) : 0) : 0x7fffffff;
 
   bf16x8_t qop[QT][DC];
@@ -800,8 +847,6 @@ __global__ __launch_bounds__(256, 2) void attn_prefill_mfma_kernel(
   // ---- this wave's share of the copies: of every 32-key step, waves 0 and 1 bring the keys
   // (half of the 16-byte chunks of all 32 rows each), waves 2 and 3 the values of keys 0-15 and
   // 16-31.
-  const int kb0 = (wg_lo / 32) * 32;
-  const int nsteps = (wg_last - kb0) / 32 + 1;
   const int last_piece = (wg_last / 16) * 16;
   // Where the 16-key pieces lie in memory is worked out 64 pieces at a time, one piece per lane
   // (its page from the block table, asked for one batch of 64 ahead), and a step reads the two
@@ -810,10 +855,11 @@ __global__ __launch_bounds__(256, 2) void attn_prefill_mfma_kernel(
   // shared by all waves of the compute unit.  A piece that would start beyond the last key
   // repeats the last one (finite numbers; its scores are masked).
   unsigned long long k_at = 0, v_at = 0;  // byte offsets of this lane's piece in k_pages and v_pages
-  auto entry_of = [&](int piece) { return min(kb0 + 16 * piece, last_piece) / bs; };
+  auto key_of = [&](int piece) { return min(first_key(rd_first + (piece >> 2)) + 16 * (piece & 3), last_piece); };
+  auto entry_of = [&](int piece) { return key_of(piece) / bs; };
   int page_ahead = table[entry_of(lane)];
   auto locate = [&](int batch) {  // pieces 64 batch .. 64 batch + 63
-    const int piece = 64 * batch + lane, key = min(kb0 + 16 * piece, last_piece);
+    const int piece = 64 * batch + lane, key = key_of(piece);
     const unsigned long long row = (unsigned long long)((unsigned)page_ahead * KV + kvh) * bs;
     k_at = (row + key % bs) * (D * 2);
     v_at = (row * D + key % bs) * 2;
@@ -881,15 +927,15 @@ __global__ __launch_bounds__(256, 2) void attn_prefill_mfma_kernel(
     if (wave >= 2) __builtin_amdgcn_global_load_lds((global_ptr_t)(from[j] + lane_at[i]), (lds_ptr_t)(to[j] + i * 64), 16, 0, 0);
     else __builtin_amdgcn_global_load_lds((global_ptr_t)(from[j] + i * 32), (lds_ptr_t)(to[j] + i * 64), 16, 0, 0);
   };
-  const int nrounds = (nsteps + 1) / 2;
+  const int nrounds = rd_end - rd_first;
   issue(0);
   issue(1);  // beyond the last key it repeats the last piece
   for (int rd = 0; rd < nrounds; ++rd) {
     PF_WAIT_VM(0);    // this wave's copies for the round have landed
     __syncthreads();  // ... and everyone's; and everyone is done with the round before
     const bool more = rd + 1 < nrounds;  // copies into the two stages the round before used
-    const int kb = kb0 + 64 * rd;
-    const bool active = working && kb <= my_last && kb + 63 >= my_lo;
+    const int kb = first_key(rd_first + rd);
+    const bool active = working && kb <= my_last && (kb + 63 >= my_lo || kb < sight.keep);
     if (more) {
       aim(2 * rd + 2);
       if (!active) {
@@ -936,6 +982,15 @@ __global__ __launch_bounds__(256, 2) void attn_prefill_mfma_kernel(
       bf16x8_t pop[QT][2];
       float alpha[QT];
       bool rescale = false;
+      if (CAP) {  // the capped scores, in base 2 already
+        const float inner = scale / sight.cap, outer = sight.cap * 1.4426950408889634f;
+#pragma unroll
+        for (int qt = 0; qt < QT; ++qt)
+#pragma unroll
+          for (int tt = 0; tt < 4; ++tt)
+#pragma unroll
+            for (int r = 0; r < 4; ++r) sc[qt][tt][r] = outer * quick_tanh(sc[qt][tt][r] * inner);
+      }
 #pragma unroll
       for (int qt = 0; qt < QT; ++qt) {
         if (masked) {
@@ -944,7 +999,7 @@ __global__ __launch_bounds__(256, 2) void attn_prefill_mfma_kernel(
 #pragma unroll
             for (int r = 0; r < 4; ++r) {
               const int key = kb + 32 * (tt >> 1) + KEY_OF_ROW(tt & 1, 4 * grp + r);
-              const bool seen = key <= qpos[qt] && (window <= 0 || key > qpos[qt] - window);
+              const bool seen = key <= qpos[qt] && (window <= 0 || key > qpos[qt] - window || key < sight.keep);
               sc[qt][tt][r] = seen ? sc[qt][tt][r] : NEG_INF;
             }
         }
@@ -1019,7 +1074,11 @@ __global__ __launch_bounds__(256, 2) void attn_prefill_mfma_kernel(
 #pragma unroll
   for (int qt = 0; qt < QT; ++qt) {
     if (!qok[qt]) continue;
-    const float inv = 1.0f / l[qt];
+    float inv = 1.0f / l[qt];
+    if (sight.sink) {
+      const float top = fmaxf(m[qt], 0.f), e = __builtin_amdgcn_exp2f(m[qt] - top);
+      inv = e / (l[qt] * e + __builtin_amdgcn_exp2f(-top));
+    }
     bf16* orow = out + ((size_t)(tok0 + q0 + qt * 16 + col) * H + head) * D + 4 * grp;
 #pragma unroll
     for (int dt = 0; dt < DT; ++dt) {
@@ -1035,7 +1094,7 @@ __global__ __launch_bounds__(256, 2) void attn_prefill_mfma_kernel(
 // largest maximum; a piece that saw no key has m = -inf and l = 0.
 template <int DC, int QT>
 __global__ __launch_bounds__(256) void attn_prefill_merge_kernel(const int* __restrict__ tiles, bf16* __restrict__ out,
-                                                                  int H, int KV, int units_z, PrefillSplit split) {
+                                                                  int H, int KV, int units_z, PrefillSplit split, int sink) {
   constexpr int D = DC * 32, DT = DC * 2, WQ = 16 * QT, PARTS = 64 / WQ;
   const int item = blockIdx.x;
   const int n = split.cut[item];
@@ -1054,10 +1113,11 @@ __global__ __launch_bounds__(256) void attn_prefill_merge_kernel(const int* __re
     const float2* ml = reinterpret_cast<const float2*>(split.ml) + at;  // (m, l) of the pieces
     float m = NEG_INF;
     for (int j = 0; j < n; ++j) m = fmaxf(m, ml[j].x);
+    if (sink) m = fmaxf(m, 0.f);
     f32x4_t sum[DT];
 #pragma unroll
     for (int dt = 0; dt < DT; ++dt) sum[dt] = f32x4_t{0.f, 0.f, 0.f, 0.f};
-    float den = 0.f;
+    float den = sink ? __builtin_amdgcn_exp2f(-m) : 0.f;
     for (int j = 0; j < n; ++j) {
       const float2 p = ml[j];
       const float w = p.x == NEG_INF ? 0.f : __builtin_amdgcn_exp2f(p.x - m);
@@ -1089,10 +1149,12 @@ __global__ __launch_bounds__(256) void attn_prefill_merge_kernel(const int* __re
 // piece_rounds * pieces covers the longest item.  pieces <= 1: none is cut, the three may be null.
 extern "C" int as_attn_prefill_mfma(const void* q, const void* k_pages, const void* v_pages, const int* tiles,
                                     int num_tiles, const int* block_tables, int table_width, void* out, int H,
-                                    int KV, int D, int bs, float scale, int window, int query_tiles,
-                                    int pieces, int piece_rounds, int* cut, float* part_ml, float* part_acc,
-                                    hipStream_t stream) {
+                                    int KV, int D, int bs, float scale, int window, int keep, float cap, int sink,
+                                    int query_tiles, int pieces, int piece_rounds, int* cut, float* part_ml,
+                                    float* part_acc, hipStream_t stream) {
   if (num_tiles <= 0) return AS_OK;
+  const Sight sight{window, keep, cap, sink};
+  if (!sight_ok(sight)) return AS_BAD_SHAPE;
   if (H <= 0 || KV <= 0 || H % KV || bs <= 0 || table_width <= 0) return AS_BAD_SHAPE;
   const int G = H / KV;
   if (D % 32 || D <= 0 || D > 256 || bs % 16) return AS_BAD_SHAPE;
@@ -1105,19 +1167,20 @@ extern "C" int as_attn_prefill_mfma(const void* q, const void* k_pages, const vo
   if (blocks > 0x7fffffffL) return AS_BAD_SHAPE;
   const int pass = compute_units();
   const PrefillSplit split{pieces, piece_rounds, cut, part_ml, part_acc};
-#define LAUNCH(DCV)                                                                                   \
-  if (query_tiles == 1) {                                                                             \
-    attn_prefill_mfma_kernel<DCV, 1><<<(int)blocks, 256, 0, stream>>>(                                \
-        (const bf16*)q, (const bf16*)k_pages, (const bf16*)v_pages, tiles, block_tables, table_width, \
-        (bf16*)out, H, KV, bs, scale, window, units_z, pass, split);                                  \
-    if (pieces > 1)                                                                                   \
-      attn_prefill_merge_kernel<DCV, 1><<<(int)items, 256, 0, stream>>>(tiles, (bf16*)out, H, KV, units_z, split); \
-  } else {                                                                                            \
-    attn_prefill_mfma_kernel<DCV, 2><<<(int)blocks, 256, 0, stream>>>(                                \
-        (const bf16*)q, (const bf16*)k_pages, (const bf16*)v_pages, tiles, block_tables, table_width, \
-        (bf16*)out, H, KV, bs, scale, window, units_z, pass, split);                                  \
-    if (pieces > 1)                                                                                   \
-      attn_prefill_merge_kernel<DCV, 2><<<(int)items, 256, 0, stream>>>(tiles, (bf16*)out, H, KV, units_z, split); \
+#define LAUNCH2(DCV, QTV, CAPV)                                                                       \
+  attn_prefill_mfma_kernel<DCV, QTV, CAPV><<<(int)blocks, 256, 0, stream>>>(                          \
+      (const bf16*)q, (const bf16*)k_pages, (const bf16*)v_pages, tiles, block_tables, table_width,   \
+      (bf16*)out, H, KV, bs, scale, sight, units_z, pass, split)
+#define LAUNCH1(DCV, QTV)                                                                             \
+  if (cap > 0.f) LAUNCH2(DCV, QTV, true);                                                             \
+  else LAUNCH2(DCV, QTV, false);                                                                      \
+  if (pieces > 1)                                                                                     \
+    attn_prefill_merge_kernel<DCV, QTV><<<(int)items, 256, 0, stream>>>(tiles, (bf16*)out, H, KV, units_z, split, sink);
+#define LAUNCH(DCV)              \
+  if (query_tiles == 1) {        \
+    LAUNCH1(DCV, 1)              \
+  } else {                       \
+    LAUNCH1(DCV, 2)              \
   }
   switch (D / 32) {
     case 1: LAUNCH(1); break;
@@ -1130,14 +1193,17 @@ extern "C" int as_attn_prefill_mfma(const void* q, const void* k_pages, const vo
     default: LAUNCH(8); break;
   }
 #undef LAUNCH
+#undef LAUNCH1
+#undef LAUNCH2
   return launch_status();
 }
 
 static int launch_decode_mfma(const void* q, const void* k_pages, const void* v_pages, const int* items,
                               int num_items, const int* positions, const int* tok_row, const int* block_tables,
                               int table_width, void* out, float* part_m, float* part_l, float* part_acc, int H,
-                              int KV, int D, int bs, float scale, int window, int part_size, int P,
+                              int KV, int D, int bs, float scale, const Sight& sight, int part_size, int P,
                               const FreshQKV* fresh, int gains_dtype, hipStream_t stream, int share = 1) {
+  if (!sight_ok(sight) || (fresh && sight.cap > 0.f)) return AS_BAD_SHAPE;
   const int G = H / KV;
   if (D % 32 || D > 256 || G > 16 || bs % 16 || part_size % 32) return AS_BAD_SHAPE;
   if (fresh && D % 64) return AS_BAD_SHAPE;
@@ -1146,11 +1212,15 @@ static int launch_decode_mfma(const void* q, const void* k_pages, const void* v_
   const size_t shmem = sizeof(float) * (size_t)(128 + 4 * D * G);
   if (shmem + 1024 > (64u << 10)) return AS_BAD_SHAPE;  // wide heads in large groups: the general kernel's
   const FreshQKV none = {};
-#define LAUNCH(DCV, FRESHV)                                                                               \
-  attn_decode_mfma_kernel<DCV, FRESHV><<<grid, 256, shmem, stream>>>(                                     \
+#define LAUNCH3(DCV, FRESHV, CAPV)                                                                        \
+  attn_decode_mfma_kernel<DCV, FRESHV, CAPV><<<grid, 256, shmem, stream>>>(                               \
       (const bf16*)q, (const bf16*)k_pages, (const bf16*)v_pages, items, positions, tok_row, block_tables, \
-      table_width, (bf16*)out, part_m, part_l, part_acc, H, KV, bs, scale, window, part_size, P,          \
+      table_width, (bf16*)out, part_m, part_l, part_acc, H, KV, bs, scale, sight, part_size, P,           \
       compute_units(), share, FRESHV ? *fresh : none)
+#define LAUNCH(DCV, FRESHV) LAUNCH3(DCV, FRESHV, false)
+#define LAUNCH_PLAIN(DCV)                          \
+  if (sight.cap > 0.f) LAUNCH3(DCV, 0, true);      \
+  else LAUNCH3(DCV, 0, false)
 #define LAUNCH_FRESH(FRESHV)            \
   switch (D / 64) {                     \
     case 1: LAUNCH(2, FRESHV); break;   \
@@ -1164,22 +1234,24 @@ static int launch_decode_mfma(const void* q, const void* k_pages, const void* v_
     LAUNCH_FRESH(1)
   } else {
     switch (D / 32) {
-      case 1: LAUNCH(1, 0); break;
-      case 2: LAUNCH(2, 0); break;
-      case 3: LAUNCH(3, 0); break;
-      case 4: LAUNCH(4, 0); break;
-      case 5: LAUNCH(5, 0); break;
-      case 6: LAUNCH(6, 0); break;
-      case 7: LAUNCH(7, 0); break;
-      default: LAUNCH(8, 0); break;
+      case 1: LAUNCH_PLAIN(1); break;
+      case 2: LAUNCH_PLAIN(2); break;
+      case 3: LAUNCH_PLAIN(3); break;
+      case 4: LAUNCH_PLAIN(4); break;
+      case 5: LAUNCH_PLAIN(5); break;
+      case 6: LAUNCH_PLAIN(6); break;
+      case 7: LAUNCH_PLAIN(7); break;
+      default: LAUNCH_PLAIN(8); break;
     }
   }
 #undef LAUNCH_FRESH
+#undef LAUNCH_PLAIN
 #undef LAUNCH
+#undef LAUNCH3
   if (hipGetLastError() != hipSuccess) return AS_LAUNCH_FAILED;
   if (P > 1) {
     attn_reduce_kernel<bf16><<<dim3(num_items, H), D <= 64 ? 64 : (D <= 128 ? 128 : 256), 0, stream>>>(
-        items, part_m, part_l, part_acc, (bf16*)out, H, D, P);
+        items, part_m, part_l, part_acc, (bf16*)out, H, D, P, sight.sink);
   }
   return launch_status();
 }
@@ -1189,14 +1261,15 @@ extern "C" int as_attn_decode_mfma(const void* q, const void* k_pages, const voi
                                    int num_items, const int* positions, const int* tok_row,
                                    const int* block_tables, int table_width, void* out, float* part_m,
                                    float* part_l, float* part_acc, int H, int KV, int D, int bs, float scale,
-                                   int window, int part_size, int P, hipStream_t stream) {
+                                   int window, int keep, float cap, int sink, int part_size, int P,
+                                   hipStream_t stream) {
   if (num_items <= 0) return AS_OK;
   if (H <= 0 || KV <= 0 || H % KV || D <= 0 || bs <= 0 || part_size <= 0 || P <= 0 || table_width <= 0)
     return AS_BAD_SHAPE;
   if (P > 1 && (!part_m || !part_l || !part_acc)) return AS_BAD_SHAPE;
   return launch_decode_mfma(q, k_pages, v_pages, items, num_items, positions, tok_row, block_tables, table_width,
-                            out, part_m, part_l, part_acc, H, KV, D, bs, scale, window, part_size, P, nullptr,
-                            DT_BF16, stream);
+                            out, part_m, part_l, part_acc, H, KV, D, bs, scale, Sight{window, keep, cap, sink},
+                            part_size, P, nullptr, DT_BF16, stream);
 }
 
 // The same where the pages hold KV / share heads and every `share` consecutive groups of H / KV query heads read
@@ -1205,14 +1278,15 @@ extern "C" int as_attn_decode_mfma_shared(const void* q, const void* k_pages, co
                                           int num_items, const int* positions, const int* tok_row,
                                           const int* block_tables, int table_width, void* out, float* part_m,
                                           float* part_l, float* part_acc, int H, int KV, int D, int bs, float scale,
-                                          int window, int part_size, int P, int share, hipStream_t stream) {
+                                          int window, int keep, float cap, int sink, int part_size, int P,
+                                          int share, hipStream_t stream) {
   if (num_items <= 0) return AS_OK;
   if (H <= 0 || KV <= 0 || H % KV || D <= 0 || bs <= 0 || part_size <= 0 || P <= 0 || table_width <= 0)
     return AS_BAD_SHAPE;
   if (P > 1 && (!part_m || !part_l || !part_acc)) return AS_BAD_SHAPE;
   return launch_decode_mfma(q, k_pages, v_pages, items, num_items, positions, tok_row, block_tables, table_width,
-                            out, part_m, part_l, part_acc, H, KV, D, bs, scale, window, part_size, P, nullptr,
-                            DT_BF16, stream, share);
+                            out, part_m, part_l, part_acc, H, KV, D, bs, scale, Sight{window, keep, cap, sink},
+                            part_size, P, nullptr, DT_BF16, stream, share);
 }
 
 // A decode step (token t is row t of the block tables) from the projection's output: per-head norm,
@@ -1235,8 +1309,8 @@ extern "C" int as_attn_decode_fresh(const void* qkv, const void* qw, const void*
   const FreshQKV fresh = {(const bf16*)qkv, qw, kw, (const float2*)cs, slots, (bf16*)k_pages, (bf16*)v_pages,
                           eps, store};
   return launch_decode_mfma(nullptr, k_pages, v_pages, items, num_tokens, positions, nullptr, block_tables,
-                            table_width, out, part_m, part_l, part_acc, H, KV, D, bs, scale, window, part_size,
-                            P, &fresh, gains_dtype, stream);
+                            table_width, out, part_m, part_l, part_acc, H, KV, D, bs, scale, Sight{window, 0, 0.f, 0},
+                            part_size, P, &fresh, gains_dtype, stream);
 }
 
 static int pow2ceil(int v) { int p = 1; while (p < v) p <<= 1; return p; }
@@ -1246,7 +1320,8 @@ static int launch_single_query(const void* q, const void* k_pages, const void* v
                                int num_items, const int* positions, const int* tok_row,
                                const int* block_tables, int table_width, void* out, float* part_m,
                                float* part_l, float* part_acc, int H, int KV, int D, int bs, float scale,
-                               int window, int part_size, int P, hipStream_t stream) {
+                               const Sight& sight, int part_size, int P, hipStream_t stream) {
+  if (!sight_ok(sight)) return AS_BAD_SHAPE;
   constexpr int CH = Chunk<T>::N;
   if (D % CH != 0 || D > 64 * CH || D > 256) return AS_BAD_SHAPE;
   const int G = H / KV;
@@ -1258,7 +1333,7 @@ static int launch_single_query(const void* q, const void* k_pages, const void* v
 #define LAUNCH(GTV)                                                                                      \
   attn_single_query_kernel<T, GTV><<<grid, 256, shmem, stream>>>(                                        \
       (const T*)q, (const T*)k_pages, (const T*)v_pages, items, positions, tok_row, block_tables,       \
-      table_width, (T*)out, part_m, part_l, part_acc, H, KV, D, bs, scale, window, part_size, P, lpk)
+      table_width, (T*)out, part_m, part_l, part_acc, H, KV, D, bs, scale, sight, part_size, P, lpk)
   switch (GT) {
     case 1: LAUNCH(1); break;
     case 2: LAUNCH(2); break;
@@ -1269,19 +1344,19 @@ static int launch_single_query(const void* q, const void* k_pages, const void* v
   if (hipGetLastError() != hipSuccess) return AS_LAUNCH_FAILED;
   if (P > 1) {
     attn_reduce_kernel<T><<<dim3(num_items, H), D <= 64 ? 64 : (D <= 128 ? 128 : 256), 0, stream>>>(
-        items, part_m, part_l, part_acc, (T*)out, H, D, P);
+        items, part_m, part_l, part_acc, (T*)out, H, D, P, sight.sink);
   }
   return launch_status();
 }
 
 // part_m, part_l: [num_items, H, P] fp32; part_acc: [num_items, H, P, D] fp32 (unused when P == 1).
-// P must be >= ceil(max context of the items / part_size).
+// P must be >= ceil(n / part_size), n the most keys that an item sees (its context; with a window at most window + keep).
 extern "C" int as_attn_single_query(const void* q, const void* k_pages, const void* v_pages, int dtype,
                                     const int* items, int num_items, const int* positions,
                                     const int* tok_row, const int* block_tables, int table_width, void* out,
                                     float* part_m, float* part_l, float* part_acc, int H, int KV, int D,
-                                    int bs, float scale, int window, int part_size, int P,
-                                    hipStream_t stream) {
+                                    int bs, float scale, int window, int keep, float cap, int sink,
+                                    int part_size, int P, hipStream_t stream) {
   if (num_items <= 0) return AS_OK;
   if (H <= 0 || KV <= 0 || H % KV || D <= 0 || bs <= 0 || part_size <= 0 || P <= 0 || table_width <= 0)
     return AS_BAD_SHAPE;
@@ -1289,11 +1364,11 @@ extern "C" int as_attn_single_query(const void* q, const void* k_pages, const vo
   if (dtype == DT_F32)
     return launch_single_query<float>(q, k_pages, v_pages, items, num_items, positions, tok_row, block_tables,
                                       table_width, out, part_m, part_l, part_acc, H, KV, D, bs, scale,
-                                      window, part_size, P, stream);
+                                      Sight{window, keep, cap, sink}, part_size, P, stream);
   if (dtype == DT_BF16)
     return launch_single_query<bf16>(q, k_pages, v_pages, items, num_items, positions, tok_row, block_tables,
-                                     table_width, out, part_m, part_l, part_acc, H, KV, D, bs, scale, window,
-                                     part_size, P, stream);
+                                     table_width, out, part_m, part_l, part_acc, H, KV, D, bs, scale,
+                                     Sight{window, keep, cap, sink}, part_size, P, stream);
   return AS_BAD_DTYPE;
 }
 
@@ -1338,6 +1413,6 @@ extern "C" int as_attn_single_query_static(const void* q, const void* k_pages, c
     part_l = part_m + rows;
   }
   return as_attn_single_query(q, k_pages, v_pages, dtype, items, num_items, positions, tok_row, block_tables,
-                              table_width, out, part_m, part_l, part_acc, H, KV, D, bs, scale, window,
+                              table_width, out, part_m, part_l, part_acc, H, KV, D, bs, scale, window, 0, 0.f, 0,
                               part_size, P, stream);
 }

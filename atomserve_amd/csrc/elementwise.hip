@@ -688,13 +688,17 @@ extern "C" int as_head_norm_store(const void* proj, int dtype, int ld, int q_off
 // values may be mixed with those that an earlier layer kept for the same tokens: v_mode 1 writes this layer's values
 // (bias added) into v_keep fp32 [T, KV vdim]; v_mode 2 stores (1 - lam) v + lam v_keep[t] instead of v.  The rotation
 // (after the norm) and the layout of q_out and of the pages are head_norm_store's.  A workgroup per token.
+// maps > 1: a head has that many queries and keys side by side that share its values.  A key head of the pages is all of
+// a head's keys (dim = maps times the width of one), and every query is a query head of its own (H counts them; they are
+// dim / maps wide in `proj`) laid out at its map's place of those dim coordinates, zero elsewhere: its product with the
+// head's keys is its product with its own map's.  Neither a norm nor a rotation goes with it.
 template <typename T>
 __global__ __launch_bounds__(256) void whole_norm_store_kernel(
     const T* __restrict__ proj, int ld, int q_off, int k_off, int v_off, int H, int KV, int dim, int vdim, int Dp,
     const float* __restrict__ q_bias, const float* __restrict__ k_bias, const float* __restrict__ v_bias,
     const float* __restrict__ qw, const float* __restrict__ kw, float eps, const float2* __restrict__ cs, int R,
     float* __restrict__ v_keep, int v_mode, float lam, const int* __restrict__ slots, T* __restrict__ q_out,
-    T* __restrict__ k_pages, T* __restrict__ v_pages, int bs, int store) {
+    T* __restrict__ k_pages, T* __restrict__ v_pages, int bs, int store, int maps) {
   // blockIdx.y: one of gridDim.y workgroups that share a token's heads (query, key and value heads in one list, dealt
   // out in turn); every one of them takes the root mean squares over the whole projections for itself.
   __shared__ float red[17];
@@ -727,14 +731,15 @@ __global__ __launch_bounds__(256) void whole_norm_store_kernel(
       const float* w = is_k ? kw : qw;
       const float inv = is_k ? inv_k : inv_q;
       if (is_k && slot < 0) continue;
+      const int wide = is_k ? dim : dim / maps, at = is_k ? 0 : (hh % maps) * wide;  // the head's coordinates at .. at + wide
       T* dst = is_k ? k_pages + (((size_t)(slot / bs) * KV + hh) * bs + slot % bs) * Dp : q_out + ((size_t)t * H + hh) * Dp;
       auto value = [&](int dd) {
-        const int c = hh * dim + dd;
+        const int c = hh * wide + dd - at;
         float v = to_f32(row[off + c]) + (bias ? bias[c] : 0.f);
         if (w) v = v * inv * w[c];
         return v;
       };
-      float v = d < dim ? value(d) : 0.f;
+      float v = d >= at && d < at + wide ? value(d) : 0.f;
       if (d < 2 * half) {
         const int i = d < half ? d : d - half, o = d < half ? d + half : d - half;
         const float u = value(o);
@@ -744,6 +749,7 @@ __global__ __launch_bounds__(256) void whole_norm_store_kernel(
       dst[d] = from_f32<T>(finite_or_zero(v));
     } else {  // a value head
       const int g = head - H - KV;
+      if (slot < 0 && v_mode != 1) continue;  // nobody takes it (and `proj` may hold no values at all)
       float v = 0.f;
       if (d < vdim) {
         const int c = g * vdim + d;
@@ -760,13 +766,14 @@ extern "C" int as_whole_norm_store(const void* proj, int dtype, int ld, int q_of
                                    int dim, int vdim, int Dp, const float* q_bias, const float* k_bias,
                                    const float* v_bias, const float* qw, const float* kw, float eps, const float* cs,
                                    int R, float* v_keep, int v_mode, float lam, const int* slots, void* q_out,
-                                   void* k_pages, void* v_pages, int bs, int store, int num_tokens,
+                                   void* k_pages, void* v_pages, int bs, int store, int maps, int num_tokens,
                                    hipStream_t stream) {
   if (num_tokens <= 0) return AS_OK;
   if (cs && (R <= 0 || (R & 1) || R > dim)) return AS_BAD_SHAPE;
   if (H <= 0 || KV <= 0 || dim <= 0 || vdim <= 0 || Dp < dim || Dp < vdim || bs <= 0 || ld <= 0 || (!qw) != (!kw))
     return AS_BAD_SHAPE;
   if (v_mode < 0 || v_mode > 2 || (v_mode && !v_keep)) return AS_BAD_SHAPE;
+  if (maps < 1 || (maps > 1 && (cs || qw || dim % maps || H % maps))) return AS_BAD_SHAPE;
   // few tokens (a decode step): a token's heads are dealt out over several workgroups; many: one takes them all
   int across = num_tokens >= 256 ? 1 : (H + 2 * KV < 32 ? H + 2 * KV : 32);
   const int threads = across > 1 && Dp <= 128 ? (Dp > 64 ? 128 : 64) : 256;
@@ -774,11 +781,11 @@ extern "C" int as_whole_norm_store(const void* proj, int dtype, int ld, int q_of
   if (dtype == DT_F32)
     whole_norm_store_kernel<float><<<grid, threads, 0, stream>>>(
         (const float*)proj, ld, q_off, k_off, v_off, H, KV, dim, vdim, Dp, q_bias, k_bias, v_bias, qw, kw, eps,
-        (const float2*)cs, R, v_keep, v_mode, lam, slots, (float*)q_out, (float*)k_pages, (float*)v_pages, bs, store);
+        (const float2*)cs, R, v_keep, v_mode, lam, slots, (float*)q_out, (float*)k_pages, (float*)v_pages, bs, store, maps);
   else if (dtype == DT_BF16)
     whole_norm_store_kernel<bf16><<<grid, threads, 0, stream>>>(
         (const bf16*)proj, ld, q_off, k_off, v_off, H, KV, dim, vdim, Dp, q_bias, k_bias, v_bias, qw, kw, eps,
-        (const float2*)cs, R, v_keep, v_mode, lam, slots, (bf16*)q_out, (bf16*)k_pages, (bf16*)v_pages, bs, store);
+        (const float2*)cs, R, v_keep, v_mode, lam, slots, (bf16*)q_out, (bf16*)k_pages, (bf16*)v_pages, bs, store, maps);
   else return AS_BAD_DTYPE;
   return launch_status();
 }

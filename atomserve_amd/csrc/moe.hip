@@ -25,9 +25,10 @@ typedef unsigned int u32x4 __attribute__((ext_vector_type(4)));  // 16 bytes as 
 // tiles [max_tiles, 3]: (expert, first place in `order`, count <= 64); counts[0] = number of tiles.
 // One workgroup; the order of pairs within an expert is whatever the atomics make it, which no
 // result depends on.
-// With token_ids null, `table` is [P]: the expert of every pair as a router's kernel left it.
+// With token_ids null, `table` is [P]: the expert of every pair as a router's kernel left it.  identity > 0: the numbers
+// experts .. experts + identity - 1 are experts without matrices; their pairs (-1 here) stand in no tile and nowhere in `order`.
 __device__ __forceinline__ int expert_of_pair(const int* token_ids, const int* table, int vocab, int top, int experts,
-                                              int p) {
+                                              int identity, int p) {
   int e;
   if (token_ids) {
     int id = token_ids[p / top];
@@ -36,6 +37,7 @@ __device__ __forceinline__ int expert_of_pair(const int* token_ids, const int* t
   } else {
     e = table[p];
   }
+  if (identity > 0 && e >= experts) return -1;
   return e < 0 ? 0 : (e >= experts ? experts - 1 : e);
 }
 
@@ -43,15 +45,15 @@ __global__ __launch_bounds__(1024) void moe_route_table_kernel(const int* __rest
                                                                const int* __restrict__ table, int vocab, int top,
                                                                int experts, int num_tokens, int* __restrict__ order,
                                                                int* __restrict__ tiles, int* __restrict__ counts,
-                                                               int max_tiles) {
+                                                               int max_tiles, int identity) {
   __shared__ int hist[MOE_MAX_EXPERTS];
   __shared__ int cursor[MOE_MAX_EXPERTS];
   const int P = num_tokens * top;
   for (int e = threadIdx.x; e < experts; e += blockDim.x) hist[e] = 0;
   __syncthreads();
   for (int p = threadIdx.x; p < P; p += blockDim.x) {
-    const int e = expert_of_pair(token_ids, table, vocab, top, experts, p);
-    atomicAdd(&hist[e], 1);
+    const int e = expert_of_pair(token_ids, table, vocab, top, experts, identity, p);
+    if (e >= 0) atomicAdd(&hist[e], 1);
   }
   __syncthreads();
   if (threadIdx.x == 0) {
@@ -69,8 +71,8 @@ __global__ __launch_bounds__(1024) void moe_route_table_kernel(const int* __rest
   }
   __syncthreads();
   for (int p = threadIdx.x; p < P; p += blockDim.x) {
-    const int e = expert_of_pair(token_ids, table, vocab, top, experts, p);
-    order[atomicAdd(&cursor[e], 1)] = p;
+    const int e = expert_of_pair(token_ids, table, vocab, top, experts, identity, p);
+    if (e >= 0) order[atomicAdd(&cursor[e], 1)] = p;
   }
 }
 
@@ -80,7 +82,8 @@ __global__ __launch_bounds__(1024) void moe_route_table_kernel(const int* __rest
 // s / (sum of the chosen + 1e-20).  mode 1: the experts with the largest z, weighing the softmax over the chosen z alone.
 // mode 2: s = softmax(z) over all experts; the experts form `groups` equal groups of neighbours, a group scores its
 // largest s, and only experts of the `keep` best groups (of equal ones the lower number first) can be chosen; the `top`
-// largest s among them weigh s * scale, not renormalised.
+// largest s among them weigh s * scale, not renormalised.  correction [experts] (mode 2 with one group; null: none) is
+// added to s for the choice alone: the `top` largest s + correction are chosen and weigh s * scale.
 // pair_expert, pair_weight [T * top].  A workgroup per token: its waves take the experts four at a time, a lane 16 bytes
 // of the token's row and of the four router rows at a time (the rows stream once, coalesced), the sums meet by lane swaps
 // and the scores in LDS, where the first wave makes the choice.
@@ -104,11 +107,12 @@ template <> struct RoutePiece<bf16> {
 template <typename T>
 __global__ __launch_bounds__(256) void moe_route_scores_kernel(const T* __restrict__ h, const T* __restrict__ router,
                                                                 const float* __restrict__ bias, int mode,
-                                                                int groups, int keep, float scale,
+                                                                const float* __restrict__ correction, int groups,
+                                                                int keep, float scale,
                                                                 int K, int experts, int top, int num_tokens,
                                                                 int* __restrict__ pair_expert,
                                                                 float* __restrict__ pair_weight) {
-  extern __shared__ float scores[];  // [experts], then [groups] group scores and [groups] marks of the kept ones
+  extern __shared__ float scores[];  // [experts], then [groups] group scores and [groups] marks of the kept ones, or [experts] weights
   constexpr int N = RoutePiece<T>::N;
   const int lane = threadIdx.x & (WAVE - 1), wave = threadIdx.x / WAVE;
   const int t = blockIdx.x;
@@ -156,7 +160,13 @@ __global__ __launch_bounds__(256) void moe_route_scores_kernel(const T* __restri
     sum = wave_sum(sum);
     for (int e = lane; e < experts; e += WAVE) mine[e] = expf(mine[e] - mx) / sum;
     __builtin_amdgcn_wave_barrier();
-    if (groups > 1 && keep < groups) {
+    if (correction) {  // what is chosen by, and beside it what a chosen one weighs
+      for (int e = lane; e < experts; e += WAVE) {
+        scores[experts + e] = mine[e];
+        mine[e] += correction[e];
+      }
+      __builtin_amdgcn_wave_barrier();
+    } else if (groups > 1 && keep < groups) {
       float* gscore = scores + experts;
       float* gkept = gscore + groups;
       const int per = experts / groups;
@@ -204,6 +214,7 @@ __global__ __launch_bounds__(256) void moe_route_scores_kernel(const T* __restri
       if (ob > best || (ob == best && oa < at)) { best = ob; at = oa; }
     }
     if (at >= experts) { at = 0; best = 0.f; }  // nothing left to choose (scores that are not numbers)
+    else if (correction) best = scores[experts + at];
     if (mode == 1) {  // the first found is the largest: weights are exponentials of the distance to it
       if (j == 0) largest = best;
       best = expf(best - largest);
@@ -226,33 +237,34 @@ __global__ __launch_bounds__(256) void moe_route_scores_kernel(const T* __restri
     for (int j = WAVE; j < top; ++j) pair_weight[(size_t)t * top + j] *= inv;
 }
 
-extern "C" int as_moe_route_scores(const void* h, const void* router, const float* bias, int mode, int groups, int keep,
-                                   float scale, int dtype, int K,
+extern "C" int as_moe_route_scores(const void* h, const void* router, const float* bias, int mode,
+                                   const float* correction, int groups, int keep, float scale, int dtype, int K,
                                    int experts, int top, int num_tokens, int* pair_expert, float* pair_weight,
                                    hipStream_t stream) {
   if (num_tokens <= 0) return AS_OK;
   if (K <= 0 || experts <= 0 || experts > MOE_MAX_EXPERTS || top <= 0 || top > experts || mode < 0 || mode > 2) return AS_BAD_SHAPE;
   if (mode == 2 && (groups < 1 || experts % groups || keep < 1 || keep > groups || keep * (experts / groups) < top)) return AS_BAD_SHAPE;
+  if (correction && (mode != 2 || groups > 1)) return AS_BAD_SHAPE;
   const int blocks = num_tokens;
-  const size_t lds = (size_t)(experts + 2 * (groups > 0 ? groups : 0)) * sizeof(float);
+  const size_t lds = (size_t)(correction ? 2 * experts : experts + 2 * (groups > 0 ? groups : 0)) * sizeof(float);
   if (dtype == DT_F32)
-    moe_route_scores_kernel<float><<<blocks, 256, lds, stream>>>((const float*)h, (const float*)router, bias, mode, groups, keep, scale, K, experts, top,
+    moe_route_scores_kernel<float><<<blocks, 256, lds, stream>>>((const float*)h, (const float*)router, bias, mode, correction, groups, keep, scale, K, experts, top,
                                                                   num_tokens, pair_expert, pair_weight);
   else if (dtype == DT_BF16)
-    moe_route_scores_kernel<bf16><<<blocks, 256, lds, stream>>>((const bf16*)h, (const bf16*)router, bias, mode, groups, keep, scale, K, experts, top,
+    moe_route_scores_kernel<bf16><<<blocks, 256, lds, stream>>>((const bf16*)h, (const bf16*)router, bias, mode, correction, groups, keep, scale, K, experts, top,
                                                                  num_tokens, pair_expert, pair_weight);
   else return AS_BAD_DTYPE;
   return launch_status();
 }
 
 extern "C" int as_moe_route_table(const int* token_ids, const int* table, int vocab, int top, int experts,
-                                  int num_tokens, int* order, int* tiles, int* counts, int max_tiles,
+                                  int num_tokens, int* order, int* tiles, int* counts, int max_tiles, int identity,
                                   hipStream_t stream) {
   if (num_tokens <= 0) return AS_OK;
   if (top <= 0 || experts <= 0 || experts > MOE_MAX_EXPERTS || (token_ids && vocab <= 0)) return AS_BAD_SHAPE;
   if (max_tiles < (num_tokens * top + MOE_TILE - 1) / MOE_TILE + experts) return AS_BAD_SHAPE;
   moe_route_table_kernel<<<1, 1024, 0, stream>>>(token_ids, table, vocab, top, experts, num_tokens, order, tiles,
-                                                 counts, max_tiles);
+                                                 counts, max_tiles, identity);
   return launch_status();
 }
 
@@ -491,30 +503,35 @@ extern "C" int as_moe_gemm(const void* a, int dtype, int a_div, const void* w, i
 
 // out[t, n] = sum over a token's `top` pairs of weight * pair_weight[t * top + j] * pair_out[t * top + j, n]
 // (+ add[t, n]); fp32 in, T out.  pair_weight null: every pair weighs `weight`; add (T) null: nothing is added.
+// same [T, N] (null: none) with pair_expert: a pair whose expert is numbered `experts` or more has same[t] as its output.
 template <typename T>
 __global__ void moe_combine_kernel(const float* __restrict__ pair_out, int top, float weight, int N,
                                    T* __restrict__ out, size_t total, const float* __restrict__ pair_weight,
-                                   const T* __restrict__ add) {
+                                   const T* __restrict__ add, const T* __restrict__ same,
+                                   const int* __restrict__ pair_expert, int experts) {
   const size_t stride = (size_t)gridDim.x * blockDim.x;
   for (size_t idx = (size_t)blockIdx.x * blockDim.x + threadIdx.x; idx < total; idx += stride) {
     const size_t t = idx / N;
     const int n = (int)(idx % N);
     float s = 0.f;
-    for (int j = 0; j < top; ++j)
-      s += weight * (pair_weight ? pair_weight[t * top + j] : 1.f) * pair_out[(t * top + j) * N + n];
+    for (int j = 0; j < top; ++j) {
+      const bool is_same = same && pair_expert[t * top + j] >= experts;
+      s += weight * (pair_weight ? pair_weight[t * top + j] : 1.f) * (is_same ? to_f32(same[idx]) : pair_out[(t * top + j) * N + n]);
+    }
     if (add) s += to_f32(add[idx]);
     out[idx] = from_f32<T>(s);
   }
 }
 
 extern "C" int as_moe_combine(const float* pair_out, int top, float weight, int N, void* out, int out_dtype,
-                              int num_tokens, const float* pair_weight, const void* add, hipStream_t stream) {
+                              int num_tokens, const float* pair_weight, const void* add, const void* same,
+                              const int* pair_expert, int experts, hipStream_t stream) {
   if (num_tokens <= 0) return AS_OK;
-  if (top <= 0 || N <= 0) return AS_BAD_SHAPE;
+  if (top <= 0 || N <= 0 || (same && !pair_expert)) return AS_BAD_SHAPE;
   const size_t total = (size_t)num_tokens * N, want = (total + 255) / 256;
   const int blocks = (int)(want > 8192 ? 8192 : want);
-  if (out_dtype == DT_F32) moe_combine_kernel<float><<<blocks, 256, 0, stream>>>(pair_out, top, weight, N, (float*)out, total, pair_weight, (const float*)add);
-  else if (out_dtype == DT_BF16) moe_combine_kernel<bf16><<<blocks, 256, 0, stream>>>(pair_out, top, weight, N, (bf16*)out, total, pair_weight, (const bf16*)add);
+  if (out_dtype == DT_F32) moe_combine_kernel<float><<<blocks, 256, 0, stream>>>(pair_out, top, weight, N, (float*)out, total, pair_weight, (const float*)add, (const float*)same, pair_expert, experts);
+  else if (out_dtype == DT_BF16) moe_combine_kernel<bf16><<<blocks, 256, 0, stream>>>(pair_out, top, weight, N, (bf16*)out, total, pair_weight, (const bf16*)add, (const bf16*)same, pair_expert, experts);
   else return AS_BAD_DTYPE;
   return launch_status();
 }

@@ -208,8 +208,15 @@ def silu_mul(gate_up, out) -> None:
 SINGLE_QUERY_MAX_HEAD_DIM = 256
 
 
+def _sight(window, keep_first, softcap, sink) -> tuple:
+    """(window, keep, cap, sink) as the attention kernels take them: what a query sees and how scores become weights."""
+    if window < 0 or keep_first < 0 or softcap < 0:
+        raise KernelError("attention: a window, a number of kept tokens and a cap of the scores are not negative")
+    return int(window), int(keep_first) if window > 0 else 0, float(softcap), int(bool(sink))
+
+
 def attn_single_query(q, k_pages, v_pages, items, positions, tok_row, block_tables, out, scale, window,
-                      max_context, part_size=None, force_generic=False) -> None:  # fmt: skip
+                      max_context, part_size=None, force_generic=False, keep_first=0, softcap=0.0, sink=False) -> None:  # fmt: skip
     """Attention of single query tokens over the paged cache.  bfloat16 with head widths in steps
     of 32 and pages of a multiple of 16 tokens runs on the matrix cores (a group of more than 16 query
     heads, or of wide heads that overfill a workgroup's LDS, as several equal groups that read the same kv
@@ -217,9 +224,12 @@ def attn_single_query(q, k_pages, v_pages, items, positions, tok_row, block_tabl
 
     q, out [T, H, D]; items [N] int32: the tokens (rows of q) to process, None for all of them in
     order; positions, tok_row [T] int32 (tok_row None: token t belongs to row t, a decode step);
-    block_tables [R, W] int32; max_context: host bound on positions[items] + 1."""
+    block_tables [R, W] int32; max_context: host bound on positions[items] + 1.
+    window > 0: a query at p sees the keys p - window + 1 .. p and those of the first `keep_first` positions.
+    softcap > 0: a score s counts as softcap tanh(s / softcap).  sink: the softmax's denominator has one more score of 0."""
     _check(q, "q", (F32, BF16), (None, None, None))
     T, H, D = q.shape
+    sight = _sight(window, keep_first, softcap, sink)
     _check(out, "out", q.dtype, (T, H, D))
     _check(k_pages, "k_pages", q.dtype, (None, None, None, D))
     _, KV, bs, _ = k_pages.shape
@@ -246,20 +256,20 @@ def attn_single_query(q, k_pages, v_pages, items, positions, tok_row, block_tabl
     share = next((G // g for g in range(min(G, 16), 0, -1) if G % g == 0 and _decode_mfma_fits(D, g)), 0)
     mfma = q.dtype == BF16 and D % 32 == 0 and bs % 16 == 0 and share > 0 and not force_generic
     if mfma and share > 1:
-        part_size, P, part_m, part_l, part_acc = _partitions(N, H, KV * share, D, max_context, window, True, part_size, q.device)
+        part_size, P, part_m, part_l, part_acc = _partitions(N, H, KV * share, D, max_context, window, True, part_size, q.device, sight[1])
         call("as_attn_decode_mfma_shared", _ptr(q), _ptr(k_pages), _ptr(v_pages), _ptr(items), N, _ptr(positions),
              _ptr(tok_row), _ptr(block_tables), block_tables.shape[1], _ptr(out), _ptr(part_m), _ptr(part_l),
-             _ptr(part_acc), H, KV * share, D, bs, float(scale), int(window), part_size, P, share, _stream())  # fmt: skip
+             _ptr(part_acc), H, KV * share, D, bs, float(scale), *sight, part_size, P, share, _stream())  # fmt: skip
         return
-    part_size, P, part_m, part_l, part_acc = _partitions(N, H, KV, D, max_context, window, mfma, part_size, q.device)
+    part_size, P, part_m, part_l, part_acc = _partitions(N, H, KV, D, max_context, window, mfma, part_size, q.device, sight[1])
     if mfma:
         call("as_attn_decode_mfma", _ptr(q), _ptr(k_pages), _ptr(v_pages), _ptr(items), N, _ptr(positions),
              _ptr(tok_row), _ptr(block_tables), block_tables.shape[1], _ptr(out), _ptr(part_m), _ptr(part_l),
-             _ptr(part_acc), H, KV, D, bs, float(scale), int(window), part_size, P, _stream())  # fmt: skip
+             _ptr(part_acc), H, KV, D, bs, float(scale), *sight, part_size, P, _stream())  # fmt: skip
         return
     call("as_attn_single_query", _ptr(q), _ptr(k_pages), _ptr(v_pages), _DT[q.dtype], _ptr(items), N,
          _ptr(positions), _ptr(tok_row), _ptr(block_tables), block_tables.shape[1], _ptr(out), _ptr(part_m),
-         _ptr(part_l), _ptr(part_acc), H, KV, D, bs, float(scale), int(window), part_size, P, _stream())  # fmt: skip
+         _ptr(part_l), _ptr(part_acc), H, KV, D, bs, float(scale), *sight, part_size, P, _stream())  # fmt: skip
 
 
 DECODE_MFMA_MAX_LDS = 64 << 10  # what a workgroup may ask for without raising the kernel's limit
@@ -302,14 +312,29 @@ def _partition_cost(groups: int, span: int, part: int) -> float:
     return (4.0 + 0.025 * min(part, span)) * max(1.0, groups * parts / (2 * compute_units())) + 0.6 * parts
 
 
-def _partitions(N, H, KV, D, max_context, window, mfma, part_size, device):
+def _up32(n: int) -> int:
+    return -(-n // 32) * 32
+
+
+def _seen_keys(max_context: int, window: int, keep_first: int, mfma: bool) -> int:
+    """The most keys that a query of these contexts walks: with a window those of the window and the kept first ones
+    (the matrix-core kernel in whole steps of 32, and a window that starts within a step takes it whole)."""
+    if window <= 0:
+        return max_context
+    if mfma:
+        return min(_up32(max_context), _up32(window + 31) + _up32(keep_first))
+    return min(max_context, window + keep_first)
+
+
+def _partitions(N, H, KV, D, max_context, window, mfma, part_size, device, keep_first=0):
     """How the keys of N single queries are cut for the split-KV kernels, and the buffers of the
-    partial results: (part_size, P, part_m, part_l, part_acc), the buffers None when P == 1."""
-    span = min(max_context, window) if window > 0 else max_context
+    partial results: (part_size, P, part_m, part_l, part_acc), the buffers None when P == 1.  What is cut is the
+    list of the keys a query sees, in order: whole contexts, or the kept first keys and then the window's."""
+    span = _seen_keys(max_context, window, keep_first, mfma)
     G = H // KV
     if part_size is None:
         # Enough partitions to occupy the GPU when few tokens are in the batch, few enough that
-        # the merge stays small; boundaries are multiples of part_size in absolute position.
+        # the merge stays small; boundaries are multiples of part_size in the list of visible keys.
         if mfma:
             groups = N * KV
             if groups >= attn_fill_groups():
@@ -322,7 +347,7 @@ def _partitions(N, H, KV, D, max_context, window, mfma, part_size, device):
                 part_size *= 2
     if mfma and part_size % 32:
         raise KernelError("attention: partitions of the matrix-core kernel are multiples of 32 keys")
-    P = max(1, math.ceil(max_context / part_size))
+    P = max(1, math.ceil(span / part_size))
     part_m = part_l = part_acc = None
     if P > 1:
         part_m = torch.empty((N, H, P), dtype=F32, device=device)
@@ -453,18 +478,18 @@ def _prefill_cost(num_tiles: int, H: int, KV: int, D: int, rounds: int, mean_rou
 
 
 def _prefill_plan(num_tiles: int, H: int, KV: int, D: int, max_context: int, window: int = 0, query_tiles=None,
-                  tile_keys: int = 0) -> tuple:  # fmt: skip
+                  tile_keys: int = 0, keep_first: int = 0) -> tuple:  # fmt: skip
     """(query tiles of a wave, pieces, rounds of a piece) for a prompt step; pieces 1 (and 0 rounds): nothing is cut.
     tile_keys: the keys that the tiles' last queries see, added up (0: not known; the tiles are then taken to be one
     request's last ones).  Every layer of a step asks the same question: the answers are kept."""
     if query_tiles is None:
         query_tiles = PREFILL_QUERY_TILES
-    return _prefill_plan_of(num_tiles, H, KV, D, max_context, window, query_tiles, tile_keys, PREFILL_PIECES, compute_units())
+    return _prefill_plan_of(num_tiles, H, KV, D, max_context, window, query_tiles, tile_keys, PREFILL_PIECES, compute_units(), keep_first)
 
 
 @functools.lru_cache(maxsize=1024)
-def _prefill_plan_of(num_tiles, H, KV, D, max_context, window, query_tiles, tile_keys, forced_pieces, units) -> tuple:
-    span = min(max_context, window + 64) if window > 0 else max_context  # the keys that the longest item walks
+def _prefill_plan_of(num_tiles, H, KV, D, max_context, window, query_tiles, tile_keys, forced_pieces, units, keep_first=0) -> tuple:
+    span = min(max_context, window + 64 + keep_first) if window > 0 else max_context  # the keys that the longest item walks
     rounds = max(1, -(-span // 64))
     if tile_keys > 0:
         mean_rounds = min(rounds, max(1.0, tile_keys / num_tiles / 64))
@@ -482,7 +507,7 @@ def _prefill_plan_of(num_tiles, H, KV, D, max_context, window, query_tiles, tile
 
 
 def attn_prefill(q, k_pages, v_pages, tiles, block_tables, out, scale, window, max_context, query_tiles=None,
-                 tile_keys: int = 0) -> None:  # fmt: skip
+                 tile_keys: int = 0, keep_first=0, softcap=0.0, sink=False) -> None:  # fmt: skip
     """Causal attention of prompt portions over the paged cache, bfloat16, on the matrix cores.
 
     tiles [Nt, 4] int32: (first flat token, count <= 64, block-table row, position of the first
@@ -490,9 +515,11 @@ def attn_prefill(q, k_pages, v_pages, tiles, block_tables, out, scale, window, m
     the pages.  max_context: host bound on the last position + 1 of any tile.
     query_tiles: column tiles of 16 queries that a wave owns, 2 or 1; None: chosen here.
     tile_keys: the sum over the tiles of (position of the first token + count), if the caller knows it: how the
-    work is cut is chosen better with it (speed only)."""
+    work is cut is chosen better with it (speed only).
+    window, keep_first, softcap, sink: as for `attn_single_query`."""
     _check(q, "q", BF16, (None, None, None))
     T, H, D = q.shape
+    sight = _sight(window, keep_first, softcap, sink)
     _check(out, "out", BF16, (T, H, D))
     _check(k_pages, "k_pages", BF16, (None, None, None, D))
     _, KV, bs, _ = k_pages.shape
@@ -505,14 +532,14 @@ def attn_prefill(q, k_pages, v_pages, tiles, block_tables, out, scale, window, m
         raise KernelError(f"prefill attention: unsupported heads {H}/{KV}, head width {D} or page size {bs}")
     if max_context > block_tables.shape[1] * bs:
         raise KernelError("attention: block tables are shorter than the longest context")
-    query_tiles, pieces, piece_rounds = _prefill_plan(tiles.shape[0], H, KV, D, max_context, window, query_tiles, tile_keys)
+    query_tiles, pieces, piece_rounds = _prefill_plan(tiles.shape[0], H, KV, D, max_context, window, query_tiles, tile_keys, sight[1])
     cut = part_ml = part_acc = None
     if pieces > 1:
         cut = torch.empty(tiles.shape[0] * KV * _prefill_units(query_tiles, H // KV), dtype=I32, device=q.device)
         part_ml = torch.empty((T, H, pieces, 2), dtype=F32, device=q.device)
         part_acc = torch.empty((T, H, pieces, D), dtype=F32, device=q.device)
     call("as_attn_prefill_mfma", _ptr(q), _ptr(k_pages), _ptr(v_pages), _ptr(tiles), tiles.shape[0],
-         _ptr(block_tables), block_tables.shape[1], _ptr(out), H, KV, D, bs, float(scale), int(window),
+         _ptr(block_tables), block_tables.shape[1], _ptr(out), H, KV, D, bs, float(scale), *sight,
          int(query_tiles), pieces, piece_rounds, _ptr(cut), _ptr(part_ml), _ptr(part_acc), _stream())  # fmt: skip
 
 
@@ -1011,6 +1038,53 @@ def topk(logits, k, values, indices) -> None:
     call("as_topk", _ptr(logits), B, V, k, _ptr(values), _ptr(indices), _stream())
 
 
+# ---- sublayers whose output is normed before it enters the stream ----------------------------------------------------
+
+
+def post_norm_add(x, y, post, eps_post, gain=None, eps: float = 0.0, out=None, rows=None, update_x=True, other=None, gains=None,
+                  biases=(None, None), eps_in: float = 0.0) -> None:  # fmt: skip
+    """v = x[s] + norm(d[s]) * post with s = rows[r] or r (eps_post inside the root), x fp32 [T, n] receiving v when
+    `update_x`; out[r] = norm(v) * gain (gain None: no norm is taken).  d = y (+ biases[0]); with `other`, d =
+    norm(y + biases[0]) * gains[0] + norm(other + biases[1]) * gains[1] (eps_in).  y, other [T, n] and out in the compute
+    dtype; post, gain, gains and biases fp32 [n]."""
+    _check(x, "x", F32, (None, None))
+    T, n = x.shape
+    _check(y, "y", (F32, BF16), (T, n))
+    n_out = T
+    if rows is not None:
+        _check(rows, "rows", I32, (None,))
+        n_out = rows.shape[0]
+        if update_x:
+            raise KernelError("post_norm_add: the stream is updated whole, not by rows")
+    if (gain is None) != (out is None):
+        raise KernelError("post_norm_add: a norm's gain and its output come together")
+    for name, t in (("post", post), ("gain", gain), ("bias", biases[0]), ("other bias", biases[1])):
+        if t is not None or name == "post":
+            _check(t, name, F32, (n,))
+    if out is not None:
+        _check(out, "out", y.dtype, (n_out, n))
+    g1 = g2 = None
+    if other is not None:
+        _check(other, "other", y.dtype, (T, n))
+        g1, g2 = gains
+        _check(g1, "gain of y", F32, (n,))
+        _check(g2, "gain of other", F32, (n,))
+    elif biases[1] is not None:
+        raise KernelError("post_norm_add: a second bias belongs to a second output")
+    call("as_post_norm_add", _ptr(x), _ptr(y), _ptr(other), _DT[y.dtype], _ptr(biases[0]), _ptr(biases[1]), _ptr(g1), _ptr(g2),
+         float(eps_in), _ptr(post), float(eps_post), _ptr(gain), float(eps), _ptr(rows), _ptr(out), n_out, n,
+         int(bool(update_x)), _stream())  # fmt: skip
+
+
+def poly_norm(z, coef, eps, out) -> None:
+    """out = a N(z) + b N(z^2) + c N(z^3) + e per row, N the division by the row's root mean square (eps inside the root);
+    coef fp32 [4] = a, b, c, e."""
+    _check(z, "z", (F32, BF16), (None, None))
+    _check(coef, "coef", F32, (4,))
+    _check(out, "out", z.dtype, tuple(z.shape))
+    call("as_poly_norm", _ptr(z), _DT[z.dtype], _ptr(coef), float(eps), _ptr(out), z.shape[0], z.shape[1], _stream())
+
+
 # ---- layers whose parts read one stream side by side -------------------------------------------------
 
 
@@ -1084,25 +1158,32 @@ def head_norm_store(proj, q_off, k_off, v_off, num_heads, num_kv_heads, dim, vdi
 
 def whole_norm_store(proj, q_off, k_off, v_off, num_heads, num_kv_heads, dim, vdim, slots, q_out, k_pages, v_pages,
                      store_kv=True, biases=None, gains=None, eps: float = 0.0, cos_sin=None, v_keep=None,
-                     v_mode: str = "none", lam: float = 0.0) -> None:  # fmt: skip
+                     v_mode: str = "none", lam: float = 0.0, maps: int = 1) -> None:  # fmt: skip
     """`head_norm_store` for heads that are normed over their whole projection.  biases: (q [H dim], k [KV dim], v [KV
     vdim]) fp32, added to the projection's output first, or None.  gains: (q [H dim], k [KV dim]) fp32: queries and keys
     are divided by the root mean square over ALL their heads (eps inside the root) and multiplied by the gains; None: no
     norm.  cos_sin: the rotation (after the norm), as in `head_norm_store`.  v_mode "keep": the values (bias added) are
-    also written to v_keep fp32 [T, KV vdim]; "mix": (1 - lam) v + lam v_keep[t] is stored instead of v."""
+    also written to v_keep fp32 [T, KV vdim]; "mix": (1 - lam) v + lam v_keep[t] is stored instead of v.
+    maps > 1: every head has that many queries and keys over the same values.  num_heads counts the queries (heads x
+    maps, `dim` / maps wide each in proj), dim is all of a head's keys side by side, and a query is laid out at its map's
+    place among them, zeros elsewhere; no norm and no rotation.  store_kv off: proj need not hold keys and values."""
     _check(proj, "proj", (F32, BF16), (None, None))
     T, ld = proj.shape
     H, KV = num_heads, num_kv_heads
     _check(q_out, "q_out", proj.dtype, (T, H, None))
     Dp = q_out.shape[2]
-    if Dp < max(dim, vdim) or min(q_off, k_off, v_off) < 0 or q_off + H * dim > ld or k_off + KV * dim > ld \
-            or v_off + KV * vdim > ld:  # fmt: skip
+    if maps < 1 or dim % maps or H % maps or (maps > 1 and (gains is not None or cos_sin is not None)):
+        raise KernelError(f"whole_norm_store: {maps} maps of {dim} coordinates in all, {H} queries, no norm and no rotation")
+    if Dp < max(dim, vdim) or q_off < 0 or q_off + H * (dim // maps) > ld or \
+            ((store_kv or gains is not None or v_mode != "none") and
+             (min(k_off, v_off) < 0 or k_off + KV * dim > ld or v_off + KV * vdim > ld)):  # fmt: skip
         raise KernelError("whole_norm_store: heads lie outside the projection's columns or the padded head width")
     qb = kb = vb = qw = kw = None
     if biases is not None:
         qb, kb, vb = biases
-        for name, t, n in (("q bias", qb, H * dim), ("k bias", kb, KV * dim), ("v bias", vb, KV * vdim)):
-            _check(t, name, F32, (n,))
+        for name, t, n in (("q bias", qb, H * (dim // maps)), ("k bias", kb, KV * dim), ("v bias", vb, KV * vdim)):
+            if t is not None or store_kv or name == "q bias":
+                _check(t, name, F32, (n,))
     if gains is not None:
         qw, kw = gains
         _check(qw, "q gain", F32, (H * dim,))
@@ -1127,7 +1208,19 @@ def whole_norm_store(proj, q_off, k_off, v_off, num_heads, num_kv_heads, dim, vd
     call("as_whole_norm_store", _ptr(proj), _DT[proj.dtype], ld, q_off, k_off, v_off, H, KV, dim, vdim, Dp, _ptr(qb),
          _ptr(kb), _ptr(vb), _ptr(qw), _ptr(kw), float(eps), _ptr(cos_sin), R, _ptr(v_keep) if modes[v_mode] else 0,
          modes[v_mode], float(lam), _ptr(slots) if store_kv else 0, _ptr(q_out), _ptr(k_pages) if store_kv else 0,
-         _ptr(v_pages) if store_kv else 0, bs, int(bool(store_kv)), T, _stream())  # fmt: skip
+         _ptr(v_pages) if store_kv else 0, bs, int(bool(store_kv)), int(maps), T, _stream())  # fmt: skip
+
+
+def map_difference(heads, vdim, lam, eps, mult, out, out_off: int = 0) -> None:
+    """heads [T, 2 H, Dp]: head h's two attention maps at 2 h and 2 h + 1, `vdim` coordinates wide.  With o = a1 - lam a2:
+    out[t, out_off + h * vdim + j] = mult * o_j / sqrt(mean(o^2) + eps)."""
+    _check(heads, "heads", (F32, BF16), (None, None, None))
+    T, H2, Dp = heads.shape
+    _check(out, "out", heads.dtype, (T, None))
+    if H2 % 2 or not 1 <= vdim <= Dp or out_off < 0 or out_off + H2 // 2 * vdim > out.shape[1]:
+        raise KernelError(f"map_difference: {H2} maps of {Dp} coordinates, {vdim} of them values, columns {out_off}.. of {out.shape[1]}")
+    call("as_map_difference", _ptr(heads), _DT[heads.dtype], H2 // 2, vdim, Dp, float(lam), float(eps), float(mult), _ptr(out),
+         out.shape[1], out_off, T, _stream())  # fmt: skip
 
 
 STREAMS_MAX = 16
@@ -1618,7 +1711,7 @@ MOE_MAX_EXPERTS = 1024
 class ExpertRoute:
     """Where a step's (token, chosen expert) pairs stand once sorted by expert: what the grouped products read."""
 
-    __slots__ = ("order", "tiles", "counts", "max_tiles", "top", "num_tokens", "pair_weight")
+    __slots__ = ("order", "tiles", "counts", "max_tiles", "top", "num_tokens", "pair_weight", "pair_expert")
 
     def __init__(self, num_tokens: int, top: int, experts: int, device):
         pairs = num_tokens * top
@@ -1628,6 +1721,7 @@ class ExpertRoute:
         self.counts = torch.empty(1, dtype=I32, device=device)
         self.top, self.num_tokens = top, num_tokens
         self.pair_weight = None  # fp32 [pairs]: what each pair weighs, where a router says (else all weigh alike)
+        self.pair_expert = None  # int32 [pairs]: each pair's expert, where a router says
 
 
 def moe_route_table(token_ids, table, experts: int) -> ExpertRoute:
@@ -1639,7 +1733,7 @@ def moe_route_table(token_ids, table, experts: int) -> ExpertRoute:
         raise KernelError(f"routing sorts up to {MOE_MAX_EXPERTS} experts, not {experts}")
     route = ExpertRoute(token_ids.shape[0], top, experts, token_ids.device)
     call("as_moe_route_table", _ptr(token_ids), _ptr(table), vocab, top, experts, token_ids.shape[0], _ptr(route.order),
-         _ptr(route.tiles), _ptr(route.counts), route.max_tiles, _stream())  # fmt: skip
+         _ptr(route.tiles), _ptr(route.counts), route.max_tiles, 0, _stream())  # fmt: skip
     return route
 
 
@@ -1654,16 +1748,24 @@ ROUTER_SCORES = {"sigmoid": 0, "softmax_of_chosen": 1, "softmax": 2}
 
 
 def moe_route_scores(h, router, top: int, score: str, bias=None, groups: int = 1, keep_groups: int = 1,
-                     weight_scale: float = 1.0) -> ExpertRoute:  # fmt: skip
+                     weight_scale: float = 1.0, correction=None, identity: int = 0) -> ExpertRoute:  # fmt: skip
     """Routes by a router's logits z = router h + bias in fp32 (bias fp32 [experts] or None).  score "sigmoid": the
     `top` largest sigmoid(z), weighing s / (their sum + 1e-20); "softmax_of_chosen": the `top` largest z, weighing the
     softmax over those z alone; "softmax": s = softmax(z) over all experts, the `top` largest among the experts of the
     `keep_groups` best of `groups` equal groups of neighbours (a group scores its largest s), weighing s * weight_scale.
-    The route carries `pair_weight` fp32 [T * top] for `moe_combine`."""
+    correction fp32 [experts] ("softmax" without groups): the `top` largest s + correction are chosen, weighing s.
+    identity: the router's last so many outputs are experts without matrices; their pairs stand in no tile of the route.
+    The route carries `pair_weight` fp32 [T * top] and `pair_expert` int32 [T * top] for `moe_combine`."""
     _check(h, "h", (F32, BF16), (None, None))
     T, K = h.shape
     _check(router, "router", h.dtype, (None, K))
     experts = router.shape[0]
+    if correction is not None:
+        _check(correction, "correction", F32, (experts,))
+        if score != "softmax" or groups != 1:
+            raise KernelError("corrected choices belong to the score 'softmax' without groups")
+    if not 0 <= identity < experts:
+        raise KernelError(f"{identity} of {experts} experts have no matrices")
     if score not in ROUTER_SCORES:
         raise KernelError(f"a router scores by one of {sorted(ROUTER_SCORES)}, not by {score!r}")
     if bias is not None:
@@ -1674,14 +1776,14 @@ def moe_route_scores(h, router, top: int, score: str, bias=None, groups: int = 1
         raise KernelError("groups of experts and a scale of the weights belong to the score 'softmax'")
     if groups < 1 or experts % groups or not 1 <= keep_groups <= groups or keep_groups * (experts // groups) < top:
         raise KernelError(f"{experts} experts in {groups} groups of which {keep_groups} are kept do not give {top} to choose")
-    route = ExpertRoute(T, top, experts, h.device)
-    pair_expert = torch.empty(max(T * top, 1), dtype=I32, device=h.device)
+    route = ExpertRoute(T, top, experts - identity, h.device)
+    pair_expert = route.pair_expert = torch.empty(max(T * top, 1), dtype=I32, device=h.device)
     route.pair_weight = torch.empty(max(T * top, 1), dtype=F32, device=h.device)
-    call("as_moe_route_scores", _ptr(h), _ptr(router), _ptr(bias), ROUTER_SCORES[score], int(groups), int(keep_groups),
-         float(weight_scale), _DT[h.dtype], K, experts, top, T,
+    call("as_moe_route_scores", _ptr(h), _ptr(router), _ptr(bias), ROUTER_SCORES[score], _ptr(correction), int(groups),
+         int(keep_groups), float(weight_scale), _DT[h.dtype], K, experts, top, T,
          _ptr(pair_expert), _ptr(route.pair_weight), _stream())  # fmt: skip
-    call("as_moe_route_table", 0, _ptr(pair_expert), 0, top, experts, T, _ptr(route.order), _ptr(route.tiles),
-         _ptr(route.counts), route.max_tiles, _stream())  # fmt: skip
+    call("as_moe_route_table", 0, _ptr(pair_expert), 0, top, experts - identity, T, _ptr(route.order), _ptr(route.tiles),
+         _ptr(route.counts), route.max_tiles, int(identity), _stream())  # fmt: skip
     return route
 
 
@@ -1711,9 +1813,10 @@ def moe_gemm(a, w, route: ExpertRoute, out, gated: bool, per_token: bool, activa
          _ptr(route.order), _ptr(route.tiles), _ptr(route.counts), route.max_tiles, _ptr(out), _DT[out.dtype], float(limit), _stream())  # fmt: skip
 
 
-def moe_combine(pair_out, top: int, weight: float, out, pair_weight=None, add=None) -> None:
+def moe_combine(pair_out, top: int, weight: float, out, pair_weight=None, add=None, same=None, pair_expert=None, experts: int = 0) -> None:
     """out[t] = sum_j weight * pair_weight[t * top + j] * pair_out[t * top + j] + add[t]; pair_out fp32 [T * top, N];
-    pair_weight fp32 [T * top] (None: 1); add [T, N] of out's dtype (None: nothing)."""
+    pair_weight fp32 [T * top] (None: 1); add [T, N] of out's dtype (None: nothing).  same [T, N] (out's dtype) with
+    pair_expert int32 [T * top]: a pair whose expert is numbered `experts` or more has same[t] as its output."""
     _check(out, "out", (F32, BF16), (None, None))
     T, N = out.shape
     _check(pair_out, "pair_out", F32, (T * top, N))
@@ -1721,8 +1824,11 @@ def moe_combine(pair_out, top: int, weight: float, out, pair_weight=None, add=No
         _check(pair_weight, "pair_weight", F32, (max(T * top, 1),))
     if add is not None:
         _check(add, "add", out.dtype, (T, N))
+    if same is not None:
+        _check(same, "same", out.dtype, (T, N))
+        _check(pair_expert, "pair_expert", I32, (max(T * top, 1),))
     call("as_moe_combine", _ptr(pair_out), top, float(weight), N, _ptr(out), _DT[out.dtype], T, _ptr(pair_weight),
-         _ptr(add), _stream())  # fmt: skip
+         _ptr(add), _ptr(same), _ptr(pair_expert) if same is not None else 0, int(experts), _stream())  # fmt: skip
 
 
 # ---- what a layer does to the stream around its parts ------------------------------------------------------
@@ -1901,6 +2007,62 @@ def decay_attention(proj, q_off, k_off, v_off, num_heads, dim, vdim, activation,
     kernel(proj, q_off, k_off, v_off, num_heads, dim, vdim, activation, k_scale, decay, state, step_rows, out, writes)
 
 
+# ---- and with a decay per token, head and key channel ------------------------------------------------------------
+
+CHANNEL_RANK_MAX = 960  # widest first step of the decays' two-step projection (a tile of tokens' fills a workgroup's LDS)
+
+
+def channel_decays(proj, low_off, rank, up, bias, tau, alpha) -> None:
+    """alpha[t, c] = sigmoid(z)^(1 / tau), z = up[c] . proj[t, low_off:low_off + rank] + bias[c] in fp32 (never below 1e-9).
+    up [C, rank] of proj's dtype, bias fp32 [C], alpha fp32 [T, C]."""
+    _check(proj, "proj", (F32, BF16), (None, None))
+    T, ld = proj.shape
+    _check(up, "up", proj.dtype, (None, rank))
+    C = up.shape[0]
+    _check(bias, "bias", F32, (C,))
+    _check(alpha, "alpha", F32, (T, C))
+    if low_off < 0 or low_off + rank > ld or not 1 <= rank <= CHANNEL_RANK_MAX or not tau > 0:
+        raise KernelError(f"channel_decays: {rank} columns at {low_off} of {ld} (at most {CHANNEL_RANK_MAX}), tau {tau}")
+    call("as_channel_decays", _ptr(proj), _DT[proj.dtype], ld, low_off, rank, _ptr(up), _ptr(bias), float(tau), _ptr(alpha), C, T,
+         _stream())  # fmt: skip
+
+
+CHANNEL_KERNELS = ("scan", "step", "chunks")
+
+
+def channel_attention(proj, q_off, k_off, v_off, num_heads, dim, vdim, k_scale, alpha, state, step_rows, out, writes=True,
+                      kernel: str = None) -> None:  # fmt: skip
+    """S = diag(alpha_t) S + k v^T, o = S^T q per head and token, in the order of a row's tokens.  q, k [heads, dim] and v
+    [heads, vdim] are columns of proj [T, ld], k times k_scale; alpha fp32 [T, heads * dim]; state fp32 [slots, heads, dim,
+    vdim]; out fp32 [T, heads, vdim].  kernel: "scan" (token by token, keys of up to DECAY_SCAN_MAX_DIM), "step" (every
+    row ONE token, the state moved in whole lines: values in fours) or "chunks" (32 tokens at a time on the matrix cores in
+    fp32), the last two for keys of up to DECAY_CHUNKS_MAX_DIM; None: by what the step and the sizes allow."""
+    _check(proj, "proj", (F32, BF16), (None, None))
+    T, ld = proj.shape
+    H, D, E = num_heads, dim, vdim
+    if kernel is None:
+        if D > DECAY_CHUNKS_MAX_DIM:
+            kernel = "scan"
+        elif step_rows[0] is None:
+            kernel = "step" if E % 4 == 0 else "scan"
+        else:
+            kernel = "chunks"
+    if kernel not in CHANNEL_KERNELS:
+        raise KernelError(f"channel_attention: kernel {kernel!r} (one of {CHANNEL_KERNELS})")
+    most = DECAY_SCAN_MAX_DIM if kernel == "scan" else DECAY_CHUNKS_MAX_DIM
+    if min(H, D, E) < 1 or D > most or max(q_off + H * D, k_off + H * D, v_off + H * E) > ld or min(q_off, k_off, v_off) < 0 \
+            or (kernel == "step" and E % 4):  # fmt: skip
+        raise KernelError(f"channel_attention ({kernel}): {H} heads of {D} and {E} at columns {q_off}, {k_off}, {v_off} of {ld}")
+    _check(alpha, "alpha", F32, (T, H * D))
+    _check(state, "state", F32, (None, H, D, E))
+    _check(out, "out", F32, (T, H, E))
+    R = _check_rows(step_rows, T)
+    _, row_first, row_len, row_start, row_slots = step_rows
+    lens = () if kernel == "step" else (_ptr(row_len),)
+    call(f"as_channel_{kernel}", _ptr(proj), _DT[proj.dtype], ld, q_off, k_off, v_off, H, D, E, float(k_scale), _ptr(alpha),
+         _ptr(state), _ptr(row_first), *lens, _ptr(row_start), _ptr(row_slots), R, _ptr(out), int(bool(writes)), _stream())  # fmt: skip
+
+
 def decay_finish(o, groups: int, eps, gain, proj, g_off, gate_activation, out) -> None:
     """out = norm(o) * gain * act(gate): o fp32 [T, n] normed in `groups` equal parts (RMS, eps inside the root),
     gain fp32 [n] or None, the gate columns g_off.. of proj [T, ld], act "sigmoid" or "silu"; out [T, n] proj's dtype."""
@@ -1952,12 +2114,14 @@ def latent_kv_store(proj, off, rank, rot, gain, eps, cos_sin, slots, k_pages, v_
          _ptr(slots), _ptr(k_pages), _ptr(v_pages), bs, width, T, _stream())  # fmt: skip
 
 
-def latent_q_absorb(q, uk, num_heads, dim, rot, rank, cos_sin, out, uk_t=None) -> None:
-    """q [T, heads * (dim + rot)], uk [heads * dim, rank]: out[t, h] = [uk_h^T q_h[:dim] | q_h[dim:] turned by
+def latent_q_absorb(q, uk, num_heads, dim, rot, rank, cos_sin, out, uk_t=None, q_off: int = 0) -> None:
+    """q: columns q_off .. q_off + heads * (dim + rot) of rows [T, ld], uk [heads * dim, rank]: out[t, h] = [uk_h^T q_h[:dim] | q_h[dim:] turned by
     cos_sin | zeros]; out [T, heads, width].  uk_t [heads, rank, dim]: the same matrices transposed, with which
     bfloat16 prompts multiply on the matrix cores."""
-    _check(q, "q", (F32, BF16), (None, num_heads * (dim + rot)))
-    T = q.shape[0]
+    _check(q, "q", (F32, BF16), (None, None))
+    T, ld = q.shape
+    if q_off < 0 or q_off + num_heads * (dim + rot) > ld:
+        raise KernelError("latent_q_absorb: the queries lie outside the rows")
     _check(uk, "uk", q.dtype, (num_heads * dim, rank))
     if uk_t is not None:
         _check(uk_t, "uk_t", q.dtype, (num_heads, rank, dim))
@@ -1966,7 +2130,7 @@ def latent_q_absorb(q, uk, num_heads, dim, rot, rank, cos_sin, out, uk_t=None) -
         _check(cos_sin, "cos_sin", F32, (T, rot // 2, 2))
     if rank + rot > out.shape[2] or rot % 2 or dim > LATENT_MAX_HEAD_DIM:
         raise KernelError("latent_q_absorb: the latent and the turned part exceed the output's width, or the heads the kernel's")
-    call("as_latent_q_absorb", _ptr(q), _ptr(uk), _ptr(uk_t), _DT[q.dtype], num_heads, dim, rot, rank, _ptr(cos_sin),
+    call("as_latent_q_absorb", _ptr(q), ld, q_off, _ptr(uk), _ptr(uk_t), _DT[q.dtype], num_heads, dim, rot, rank, _ptr(cos_sin),
          _ptr(out), out.shape[2], T, _stream())  # fmt: skip
 
 
@@ -1996,16 +2160,20 @@ def latent_v_expand(heads, uv_t, rank, gate, g_off, out, uv=None) -> None:
 WIDE_ATTEND_MAX_WIDTH = 2048
 
 
-def wide_attend(q, k_pages, v_pages, positions, tok_row, block_tables, out, scale, max_context) -> None:
-    """Causal attention of every token's heads q [T, H, width] over ONE kv head of any width up to
-    WIDE_ATTEND_MAX_WIDTH (k_pages [pages, 1, bs, width], v_pages [pages, 1, width, bs]): for pages wider than the
-    paged attention kernels' heads.  positions, tok_row [T] int32 (tok_row None: token t is row t); out like q."""
+def wide_attend(q, k_pages, v_pages, positions, tok_row, block_tables, out, scale, max_context, window=0, keep_first=0,
+                softcap=0.0, sink=False) -> None:  # fmt: skip
+    """Causal attention of every token's heads q [T, H, width] over kv heads of any width up to
+    WIDE_ATTEND_MAX_WIDTH (k_pages [pages, KV, bs, width], v_pages [pages, KV, width, bs]): for pages wider than the
+    paged attention kernels' heads.  positions, tok_row [T] int32 (tok_row None: token t is row t); out like q.
+    window, keep_first, softcap, sink: as for `attn_single_query`."""
     _check(q, "q", (F32, BF16), (None, None, None))
     T, H, width = q.shape
     _check(out, "out", q.dtype, (T, H, width))
-    _check(k_pages, "k_pages", q.dtype, (None, 1, None, width))
-    pages, _, bs, _ = k_pages.shape
-    _check(v_pages, "v_pages", q.dtype, (pages, 1, width, bs))
+    _check(k_pages, "k_pages", q.dtype, (None, None, None, width))
+    pages, KV, bs, _ = k_pages.shape
+    _check(v_pages, "v_pages", q.dtype, (pages, KV, width, bs))
+    if KV < 1 or H % KV:
+        raise KernelError(f"attention: {H} query heads do not divide over {KV} kv heads")
     _check(positions, "positions", I32, (T,))
     if tok_row is not None:
         _check(tok_row, "tok_row", I32, (T,))
@@ -2017,4 +2185,5 @@ def wide_attend(q, k_pages, v_pages, positions, tok_row, block_tables, out, scal
     if max_context > block_tables.shape[1] * bs:
         raise KernelError("attention: block tables are shorter than the longest context")
     call("as_wide_attend", _ptr(q), _ptr(k_pages), _ptr(v_pages), _DT[q.dtype], _ptr(positions), _ptr(tok_row),
-         _ptr(block_tables), block_tables.shape[1], _ptr(out), H, width, bs, float(scale), T, _stream())
+         _ptr(block_tables), block_tables.shape[1], _ptr(out), H, KV, width, bs, float(scale),
+         *_sight(window, keep_first, softcap, sink), T, _stream())  # fmt: skip

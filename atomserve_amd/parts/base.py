@@ -150,6 +150,22 @@ class GatedDelta:
         return GatedDelta(self.y, self.gate, self.gate_off, self.bias, self.mult * factor)
 
 
+class NormedSum:
+    """Outputs of two parts [T, hidden] that read the same input, still to be put together: norm(y_1 + bias_1) * gain_1 +
+    norm(y_2 + bias_2) * gain_2, RMS norms over the width with eps (gains and biases fp32; a bias may be None)."""
+
+    def __init__(self, ys, biases, gains, eps: float):
+        self.ys, self.biases, self.gains, self.eps = tuple(ys), tuple(biases), tuple(gains), eps
+
+
+class NormedDelta:
+    """A part's output `y` (a tensor [T, hidden] in the compute dtype, or a `NormedSum`) still to be normed by `norm` and
+    added into the stream: a norm that says `takes_normed_delta` does both on its way."""
+
+    def __init__(self, y, norm: "Norm"):
+        self.y, self.norm = y, norm
+
+
 class StreamsDelta:
     """A part's output `y` [T, hidden] still to be written into several residual streams: every stream r becomes
     sum_s mix[s, r] x_s + mult out[r] y (mix fp32 [S, S] or None for the identity, out fp32 [S]).  The kernel that reads
@@ -198,6 +214,7 @@ class FeedForward(Part):
 class Norm(Part):
     takes_split_sums = False  # whether `forward` accepts a SplitSums as `delta`
     takes_gated_delta = False  # whether `forward` accepts a GatedDelta as `delta`
+    takes_normed_delta = False  # whether `forward` accepts a NormedDelta as `delta`
 
     def forward(self, x, delta=None, rows=None, update_residual=True) -> torch.Tensor:
         raise NotImplementedError

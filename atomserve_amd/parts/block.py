@@ -7,6 +7,7 @@
               results of all layers before it
 "streams_prenorm": "prenorm" over several residual streams that a sublayer reads as one weighted sum and writes
               through a mixing matrix
+"sandwich":   x += post1(mixer(norm1(x)));  x += post2(ffn(norm2(x))): a norm before and after every sublayer
 
 The residual stream `x` is fp32 in both precisions.  A part's output is not added at
 once: it travels as the pending `delta` to the next norm, whose kernel adds it into
@@ -22,6 +23,8 @@ from atomserve_amd.parts.base import (
     Arrangement,
     DeltaSum,
     GatedDelta,
+    NormedDelta,
+    NormedSum,
     Part,
     PendingNorm,
     StateCacheRequest,
@@ -150,6 +153,53 @@ class GatedPreNormBlock(Arrangement):
 
 
 register("arrangement", "gated_prenorm", GatedPreNormBlock)
+
+
+class SandwichBlock(Arrangement):
+    """x += post1(mixer(norm1(x)));  x += post2(ffn(norm2(x)))  (spec.ffn None: the mixer alone).  A sublayer's output
+    travels as a pending `NormedDelta` to the kernel of the next norm, which norms it, adds it into the fp32 stream and
+    norms the sum in one pass over the row."""
+
+    def __init__(self, spec, env):
+        super().__init__(spec, env)
+        self.mixer_norm = build("norm", spec.mixer_norm, env)
+        self.mixer = build("mixer", spec.mixer, env)
+        self.mixer_post_norm = build("norm", spec.mixer_post_norm, env)
+        self.ffn_norm = self.ffn = self.ffn_post_norm = None
+        if spec.ffn is not None:
+            self.ffn_norm = build("norm", spec.ffn_norm, env)
+            self.ffn = build("feed_forward", spec.ffn, env)
+            self.ffn_post_norm = build("norm", spec.ffn_post_norm, env)
+        for norm in (self.mixer_norm, self.mixer_post_norm, self.ffn_norm, self.ffn_post_norm):
+            if norm is not None and not norm.takes_normed_delta:
+                raise ValueError(f"a norm of kind {norm.spec.kind!r} does not norm outputs on their way into the stream")
+
+    def parts(self) -> dict:
+        parts = {"mixer_norm": self.mixer_norm, "mixer": self.mixer, "mixer_post_norm": self.mixer_post_norm}
+        if self.ffn is not None:
+            parts.update(ffn_norm=self.ffn_norm, ffn=self.ffn, ffn_post_norm=self.ffn_post_norm)
+        return parts
+
+    def first_norm(self):
+        return None  # nothing is left pending inside a product for this layer
+
+    def forward(self, x, delta, step, cache, next_norm=None):
+        if delta is not None and not isinstance(delta, NormedDelta):
+            raise ValueError("a layer of this arrangement takes an output that is still to be normed, or none")
+        y = self.mixer.forward(self.mixer_norm.forward(x, delta), step, cache)
+        delta = self.pending(y, self.mixer_post_norm)
+        if self.ffn is None:
+            return delta
+        return self.pending(self.ffn.forward(self.ffn_norm.forward(x, delta), step), self.ffn_post_norm)
+
+    @staticmethod
+    def pending(y, norm) -> NormedDelta:
+        if not isinstance(y, (torch.Tensor, NormedSum)):
+            raise ValueError("a part of a layer with norms after its sublayers returns its output, or a sum of normed outputs")
+        return NormedDelta(y, norm)
+
+
+register("arrangement", "sandwich", SandwichBlock)
 
 
 class LayerVectors(Part):

@@ -149,6 +149,8 @@ class GatedRoutedExperts(FeedForward):
         that softmax times a factor ("softmax", `GatedRoutedExpertsSpec`)
         expert e: down_e(act(gate_e h, up_e h)), act the gated activation of the spec with its limit
         with spec.shared_size one more such expert (with a limit of its own) runs for every token and is added
+        with spec.correction the softmax scores plus numbers of the layer's own decide who is chosen (not what it weighs)
+        with spec.identity the router has so many more outputs, experts whose output is h itself
 
     The routed experts run through the grouped products, the shared one through the dense ones."""
 
@@ -162,27 +164,34 @@ class GatedRoutedExperts(FeedForward):
             raise ValueError("the activation with limits needs positive limits")
         if spec.score not in ops.ROUTER_SCORES:
             raise ValueError(f"a router scores by one of {sorted(ops.ROUTER_SCORES)}, not by {spec.score!r}")
-        if not 1 <= spec.top <= spec.num_experts <= ops.MOE_MAX_EXPERTS:
-            raise ValueError(f"{spec.top} of {spec.num_experts} experts (at most {ops.MOE_MAX_EXPERTS}) cannot be chosen")
+        self.outputs = spec.num_experts + spec.identity  # of the router
+        if spec.identity < 0 or spec.num_experts < 1 or not 1 <= spec.top <= self.outputs <= ops.MOE_MAX_EXPERTS:
+            raise ValueError(f"{spec.top} of {self.outputs} experts (at most {ops.MOE_MAX_EXPERTS}) cannot be chosen")
+        if spec.correction and (spec.score != "softmax" or spec.groups != 1):
+            raise ValueError("corrected choices belong to the score 'softmax' without groups")
 
     def weight_decls(self) -> dict:
         s = self.spec
         decls = {
-            "router.weight": WeightDecl((s.num_experts, s.hidden_size)),
+            "router.weight": WeightDecl((self.outputs, s.hidden_size)),
             "gate.weight": WeightDecl((s.num_experts, s.intermediate_size, s.hidden_size)),
             "up.weight": WeightDecl((s.num_experts, s.intermediate_size, s.hidden_size)),
             "down.weight": WeightDecl((s.num_experts, s.hidden_size, s.intermediate_size)),
         }
         if s.router_bias:
-            decls["router.bias"] = WeightDecl((s.num_experts,), role="vector")
+            decls["router.bias"] = WeightDecl((self.outputs,), role="vector")
+        if s.correction:
+            decls["correction"] = WeightDecl((self.outputs,), role="vector")
         if s.shared_size:
             decls["shared_gate_up.weight"] = WeightDecl((2 * s.shared_size, s.hidden_size))
             decls["shared_down.weight"] = WeightDecl((s.hidden_size, s.shared_size))
         return decls
 
     def bind(self, tensors: dict) -> None:
-        self.router_bias = None
+        self.router_bias = self.correction = None
         super().bind(tensors)
+        if self.correction is not None:
+            self.correction = self.correction.float().contiguous()
         if self.router_bias is not None:
             self.router_bias = self.router_bias.float().contiguous()
         # every expert's gate rows, then its up rows: what the first grouped product reads
@@ -201,7 +210,7 @@ class GatedRoutedExperts(FeedForward):
         T, dev = h.shape[0], h.device
         clamped = s.activation == "clamped_swish"
         route = ops.moe_route_scores(h, self.router_weight, s.top, s.score, self.router_bias, s.groups, s.keep_groups,
-                                     s.weight_scale)  # fmt: skip
+                                     s.weight_scale, self.correction, s.identity)  # fmt: skip
         pairs = T * s.top
         act = torch.empty((pairs, s.intermediate_size), dtype=env.dtype, device=dev)
         ops.moe_gemm(h, self.gate_up_weight, route, act, gated=True, per_token=True, limit=s.limit if clamped else 0.0)
@@ -217,7 +226,8 @@ class GatedRoutedExperts(FeedForward):
             shared = torch.empty((T, s.hidden_size), dtype=env.dtype, device=dev)
             ops.gemm(a, self.shared_down, shared, env.products)
         y = torch.empty((T, s.hidden_size), dtype=env.dtype, device=dev)
-        ops.moe_combine(each, s.top, 1.0, y, pair_weight=route.pair_weight, add=shared)
+        ops.moe_combine(each, s.top, 1.0, y, pair_weight=route.pair_weight, add=shared, same=h if s.identity else None,
+                        pair_expert=route.pair_expert, experts=s.num_experts)  # fmt: skip
         return y
 
 

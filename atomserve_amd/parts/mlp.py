@@ -59,3 +59,41 @@ class GatedMLP(FeedForward):
 
 
 register("feed_forward", "gated_mlp", GatedMLP)
+
+
+class PolyNormMLP(FeedForward):
+    """down(act(up h)), act(z) = a N(z) + b N(z^2) + c N(z^3) + e (`PolyNormMLPSpec`); the powers, their root mean squares
+    and the polynomial are fp32, one pass over the row between the two products."""
+
+    capturable = True
+
+    def weight_decls(self) -> dict:
+        s = self.spec
+        return {
+            "up.weight": WeightDecl((s.intermediate_size, s.hidden_size)),
+            "down.weight": WeightDecl((s.hidden_size, s.intermediate_size)),
+            "act": WeightDecl((4,), role="vector"),
+        }
+
+    def bind(self, tensors: dict) -> None:
+        super().bind(tensors)
+        self.act = self.act.float().contiguous()
+        self.up = ops.Streamed(self.up_weight, self.env.stream_copies)
+        self.down = ops.Streamed(self.down_weight, self.env.stream_copies)
+
+    def streamed(self) -> list:
+        return [self.up, self.down]
+
+    def forward(self, h, step):
+        s, env = self.spec, self.env
+        T, dev = h.shape[0], h.device
+        z = torch.empty((T, s.intermediate_size), dtype=env.dtype, device=dev)
+        ops.gemm(h, self.up, z, env.products)
+        act = torch.empty_like(z)
+        ops.poly_norm(z, self.act, s.eps, act)
+        y = torch.empty((T, s.hidden_size), dtype=env.dtype, device=dev)
+        ops.gemm(act, self.down, y, env.products)
+        return y
+
+
+register("feed_forward", "poly_norm_mlp", PolyNormMLP)

@@ -6,7 +6,7 @@ pre-norm layer is fused into the same kernel: the fp32 residual stream `x` recei
 import torch
 
 from atomserve_amd.kernels import ops
-from atomserve_amd.parts.base import DeltaSum, GatedDelta, Norm, PendingNorm, SplitSums, WeightDecl, register
+from atomserve_amd.parts.base import DeltaSum, GatedDelta, Norm, NormedDelta, NormedSum, PendingNorm, SplitSums, WeightDecl, register
 
 
 class PendingRMSNorm(PendingNorm):
@@ -31,12 +31,15 @@ class RMSNorm(Norm):
     capturable = True
     takes_split_sums = True
     takes_gated_delta = True
+    takes_normed_delta = True
 
     def weight_decls(self) -> dict:
-        return {"weight": WeightDecl((self.spec.size,), role="vector")}
+        return {"weight": WeightDecl(() if self.spec.one_gain else (self.spec.size,), role="vector")}
 
     def bind(self, tensors: dict) -> None:
         super().bind(tensors)
+        if self.spec.one_gain:  # the kernels read a gain per coordinate
+            self.weight = self.weight.float().reshape(1).expand(self.spec.size).contiguous()
         if self.spec.offset:  # a gain stored around zero: the sum is made once, in 32 bits, and stays so
             self.weight = (self.weight.float() + float(self.spec.offset)).contiguous()
         self.gain_f32 = self.weight.float()  # what the fused product reads (exact: bf16 widens)
@@ -61,12 +64,23 @@ class RMSNorm(Norm):
                                self.spec.eps, out, rows=rows, update_x=update_residual)  # fmt: skip
         elif isinstance(delta, DeltaSum):
             self.with_sibling(None, x, delta, rows, update_residual, out)
+        elif isinstance(delta, NormedDelta):
+            self.after_normed(x, delta, rows, update_residual, out)
         elif isinstance(delta, SplitSums):
             ops.rmsnorm(x, self.weight, self.spec.eps, out, rows=rows, update_x=update_residual, split_sums=delta.sums)
         else:
             ops.rmsnorm(x, self.weight, self.spec.eps, out, delta=delta, rows=rows, update_x=update_residual)
         return out
 
+    def after_normed(self, x, delta, rows, update_residual, out) -> None:
+        """x += the delta's norm of its output; out = this norm of x: one kernel."""
+        s = self.spec
+        y, post = delta.y, delta.norm
+        if isinstance(y, NormedSum):
+            ops.post_norm_add(x, y.ys[0], post.gain_f32, post.spec.eps, self.gain_f32, s.eps, out, rows, update_residual,
+                              other=y.ys[1], gains=y.gains, biases=y.biases, eps_in=y.eps)  # fmt: skip
+        else:
+            ops.post_norm_add(x, y, post.gain_f32, post.spec.eps, self.gain_f32, s.eps, out, rows, update_residual)
 
     def stream(self, x) -> torch.Tensor:
         """The norm of the fp32 rows x as a new fp32 tensor: for a norm whose result is itself a residual stream

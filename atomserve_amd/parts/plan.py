@@ -20,6 +20,7 @@ class NormSpec:
     eps: float
     groups: int = 1
     offset: float = 0.0  # added to the stored gain (1.0: a gain stored around zero); the sum is kept in 32 bits
+    one_gain: bool = False  # the gain is one number, for all coordinates
 
 
 @dataclass(frozen=True)
@@ -52,7 +53,8 @@ class ScaledRotarySpec:
 @dataclass(frozen=True)
 class NeighbourRotarySpec:
     """Rotary position encoding of a head's first `rotary_dim` coordinates whose pairs are neighbours, (2i, 2i + 1).
-    kind "rope_neighbours".  With `factor` > 0 the frequencies are stretched as `ScaledRotarySpec` says."""
+    kind "rope_neighbours".  With `factor` > 0 the frequencies are stretched as `ScaledRotarySpec` says; `slower` divides
+    every frequency (linear scaling)."""
 
     kind: str
     rotary_dim: int
@@ -61,6 +63,7 @@ class NeighbourRotarySpec:
     original: float = 0.0
     fast: float = 0.0
     slow: float = 0.0
+    slower: float = 1.0
 
 
 @dataclass(frozen=True)
@@ -87,11 +90,12 @@ class DecayAttentionSpec:
 @dataclass(frozen=True)
 class LatentAttentionSpec:
     """Causal softmax attention whose keys and values are matrices times a cached latent [kv_rank] per token, beside
-    one rotated key part [rot_dim] shared by all heads; queries pass a normed latent of their own [q_rank] and are,
+    one rotated key part [rot_dim] shared by all heads; queries pass a normed latent of their own [q_rank] (q_rank 0:
+    they are a projection of the input) and are,
     per head, `head_dim` coordinates that are not rotated and then `rot_dim` that are.  score = scale (q . k of both
-    parts).  The concatenated heads [heads, value_dim] times sigmoid of a projection of the input go through the
-    output projection.  own_latent False: the layer has no projection to the latent; it reads the pages of the run
-    that its run names as its cache."""
+    parts).  The concatenated heads [heads, value_dim], with `out_gate` times sigmoid of a projection of the input, go
+    through the output projection.  own_latent False: the layer has no projection to the latent; it reads the pages of
+    the run that its run names as its cache.  window, keep_first: as for `SoftmaxCoreSpec`."""
 
     kind: str  # "latent_attention"
     hidden_size: int
@@ -103,8 +107,11 @@ class LatentAttentionSpec:
     kv_rank: int
     scale: float
     norm_eps: float
-    position: Any  # of the rot_dim coordinates; a position spec of pairs "half", or None
+    position: Any  # of the rot_dim coordinates; a position spec of pairs "half" or "neighbours", or None
     own_latent: bool = True
+    out_gate: bool = True
+    window: int = 0
+    keep_first: int = 0
 
 
 @dataclass(frozen=True)
@@ -225,7 +232,16 @@ class SoftmaxCoreSpec:
     whole projection (all heads at once) with gains of that size.  position: a rotation of q and k, or None.
     value_mix "first": the core's values (of the step's tokens) are kept for later layers under `value_mix_key`;
     "later": its values become (1 - lam) v + lam v_first before they are cached, lam a scalar of its own.
-    out_gate: the concatenated heads are multiplied by sigmoid of a projection of the input."""
+    out_gate: the concatenated heads are multiplied by sigmoid of a projection of the input.
+    window > 0: a query at p sees the keys p - window + 1 .. p and those of the sequence's first `keep_first` tokens.
+    softcap > 0: a score s counts as softcap tanh(s / softcap).  sink: one more score of 0 in the softmax's denominator,
+    without a value.
+    maps 2: differential attention: a head has two queries and two keys of `key_dim` over one value, laid out [map 1, map
+    2], and its output is a1 - lambda a2 over its root mean square (difference_eps), times (1 - difference), with lambda =
+    exp(lq1 . lk1) - exp(lq2 . lk2) + difference.
+    own_kv False: no projections to keys and values; the core reads the pages of the run that its run names as its
+    cache.  cache_window, cache_keep_first: what those pages keep where another run reads them too and sees more than
+    this core (None: what this core sees)."""
 
     kind: str  # "softmax_core"
     num_heads: int
@@ -239,6 +255,32 @@ class SoftmaxCoreSpec:
     value_mix: str = "none"
     value_mix_key: str = "values"
     out_gate: bool = False
+    window: int = 0
+    keep_first: int = 0
+    softcap: float = 0.0
+    sink: bool = False
+    maps: int = 1
+    difference: float = 0.0
+    difference_eps: float = 0.0
+    own_kv: bool = True
+    cache_window: Optional[int] = None
+    cache_keep_first: Optional[int] = None
+
+
+@dataclass(frozen=True)
+class ChannelDecaySpec:
+    """Gated linear attention, per head: S = diag(alpha) S + k v^T, o = S^T q with q times key_dim^(-1/2) and a decay per key
+    channel alpha = sigmoid(z)^(1 / tau), z = W_2 (W_1 h) + b laid out heads x key_dim (rank: the rows of W_1).  Every
+    head's o is RMS-normed with a gain [value_dim] shared by the heads, the heads times silu of a projection of the
+    input.  One of the cores of a "joined" mixer."""
+
+    kind: str  # "channel_decay"
+    num_heads: int
+    key_dim: int
+    value_dim: int
+    rank: int
+    tau: float
+    out_norm_eps: float
 
 
 @dataclass(frozen=True)
@@ -260,12 +302,17 @@ class MatrixMemorySpec:
 @dataclass(frozen=True)
 class JoinedMixerSpec:
     """Several cores that read the same input; one input product makes what all of them need and one output product
-    takes scales[c] * core c's result side by side, so the weighted sum of the cores is the product's own sum."""
+    takes scales[c] * core c's result side by side, so the weighted sum of the cores is the product's own sum.
+    out_norm_eps > 0 (two cores): every core has an output product of its own whose result is RMS-normed over the width
+    with a gain [hidden_size] of its own, and the cores' weighted sum is taken of the normed outputs.
+    out_bias: which cores' output products have a bias [hidden_size] (empty: none; with out_norm_eps)."""
 
     kind: str  # "joined"
     hidden_size: int
     cores: tuple
     scales: tuple
+    out_norm_eps: float = 0.0
+    out_bias: tuple = ()
 
 
 @dataclass(frozen=True)
@@ -327,7 +374,9 @@ class GatedRoutedExpertsSpec:
     largest s among the experts of the `keep_groups` best groups are chosen; they weigh s * weight_scale, not
     renormalised.  An expert is down(act(gate h, up h)) with the
     activation of `GatedMLPSpec` and `limit`.  shared_size > 0: one more such expert (with `shared_limit`) runs for
-    every token and is added."""
+    every token and is added.  correction ("softmax" without groups): numbers, one per router output, that are added to
+    s for the choice alone.  identity: the router has so many more outputs, experts without matrices whose output is the
+    input itself."""
 
     kind: str  # "gated_routed_experts"
     hidden_size: int
@@ -343,6 +392,19 @@ class GatedRoutedExpertsSpec:
     groups: int = 1
     keep_groups: int = 1
     weight_scale: float = 1.0
+    correction: bool = False
+    identity: int = 0
+
+
+@dataclass(frozen=True)
+class PolyNormMLPSpec:
+    """Dense feed-forward down(act(up x)) without a gate, act(z) = a N(z) + b N(z^2) + c N(z^3) + e with four numbers of
+    the layer's own; powers are taken element by element and N divides a row by its root mean square (eps inside)."""
+
+    kind: str  # "poly_norm_mlp"
+    hidden_size: int
+    intermediate_size: int
+    eps: float
 
 
 @dataclass(frozen=True)
@@ -361,7 +423,9 @@ class BlockSpec:
     arrangement "streams_prenorm": the stream is `streams` copies x_1 .. x_s (all what the embedding gave before the
     layer marked streams_first); a sublayer reads u = sum_s a[s] x_s through its norm and writes x_t <- sum_s M[s, t]
     x_s + residual_scale c[t] y with a, M, c of its own; the layer marked streams_last leaves their sum as the
-    stream.  streams 0: one stream with a = M = c = 1, that is x += residual_scale y."""
+    stream.  streams 0: one stream with a = M = c = 1, that is x += residual_scale y.
+    arrangement "sandwich": x += mixer_post_norm(mixer(mixer_norm(x))); x += ffn_post_norm(ffn(ffn_norm(x))) (ffn None:
+    the mixer alone)."""
 
     arrangement: str
     mixer: Any
@@ -375,6 +439,8 @@ class BlockSpec:
     streams: int = 0
     streams_first: bool = False
     streams_last: bool = False
+    mixer_post_norm: Optional[NormSpec] = None
+    ffn_post_norm: Optional[NormSpec] = None
 
 
 @dataclass(frozen=True)

@@ -100,6 +100,9 @@ class NeighbourRotary(Position):
             raise ValueError("a rotation needs theta > 1")
         i = torch.arange(0, s.rotary_dim // 2, dtype=torch.float64)
         freq = float(s.theta) ** (-2.0 * i / s.rotary_dim)
+        if not s.slower > 0:
+            raise ValueError("what divides a rotation's frequencies is positive")
+        freq = freq / s.slower
         self.magnitude = 1.0
         if s.factor > 0:
             if not (s.original > 0 and s.fast > 0 and s.slow > 0):

@@ -60,7 +60,11 @@ def test_how_single_queries_contexts_are_partitioned():
     size, P, m, l, acc = ops._partitions(64, 32, 8, 128, 2100, 0, True, None, "cpu")
     assert (size, P, m) == (2112, 1, None)  # 512 pairs: the whole context, rounded up to steps of 32 keys
     size, P, *_ = ops._partitions(8, 32, 8, 128, 5000, 1024, True, None, "cpu")
-    assert size == 128 and P == 40  # a window: the span decides the size, the context how many there are
+    assert size == 256 and P == 5  # a window: the keys it shows (in whole steps of 32) decide the size and how many there are
+    size, P, *_ = ops._partitions(8, 32, 8, 128, 5000, 1024, True, 128, "cpu", keep_first=100)
+    assert size == 128 and P == 10  # and the kept first ones
+    assert ops._seen_keys(5000, 1, 0, True) == 32 and ops._seen_keys(5000, 2, 5, True) == 96 and ops._seen_keys(5000, 2, 5, False) == 7
+    assert ops._seen_keys(90, 100, 30, True) == 96 and ops._seen_keys(90, 0, 0, True) == 90
     with pytest.raises(ops.KernelError, match="multiples of 32"):
         ops._partitions(8, 32, 8, 128, 2048, 0, True, 100, "cpu")
 
