@@ -30,12 +30,20 @@ struct Sight {
   int keep;    // with a window: the sequence's first `keep` keys stay visible behind it
   float cap;   // > 0: a score s counts as cap tanh(s / cap)
   int sink;    // 1: the denominator has one more score, of 0, which has no value
+  int wide;    // 1: the kernels of bfloat16 heads write their results in fp32 (for a consumer that takes differences of them)
 };
+// The result of a head's coordinate i, in the type of the heads or in fp32 (`Sight::wide`).
+template <typename T>
+__device__ __forceinline__ void put(T* out, size_t i, float v, int wide) {
+  if (wide) reinterpret_cast<float*>(out)[i] = v;
+  else out[i] = from_f32<T>(v);
+}
 __device__ __forceinline__ int first_in_window(const Sight& sight, int ctx) {
   return sight.window > 0 ? max(0, ctx - sight.window) : 0;
 }
 static inline bool sight_ok(const Sight& s) {
-  return s.window >= 0 && s.keep >= 0 && (s.keep == 0 || s.window > 0) && s.cap >= 0.f && (s.sink == 0 || s.sink == 1);
+  return s.window >= 0 && s.keep >= 0 && (s.keep == 0 || s.window > 0) && s.cap >= 0.f && (s.sink == 0 || s.sink == 1) &&
+         (s.wide == 0 || s.wide == 1);
 }
 
 // tanh through the hardware's exponential and reciprocal: an absolute error of 1e-7, which is what a capped score
@@ -219,7 +227,7 @@ __global__ __launch_bounds__(256) void attn_single_query_kernel(
         num *= e;
         den = den * e + fexp<T>(-top);
       }
-      out[((size_t)t * H + h) * D + d] = from_f32<T>(num / den);
+      put(out, ((size_t)t * H + h) * D + d, num / den, sight.wide);
     } else {
       const size_t o = ((size_t)item * H + h) * P + part;
       part_acc[o * D + d] = num;
@@ -238,7 +246,7 @@ __global__ __launch_bounds__(256) void attn_reduce_kernel(const int* __restrict_
                                                           const float* __restrict__ part_m,
                                                           const float* __restrict__ part_l,
                                                           const float* __restrict__ part_acc, T* __restrict__ out,
-                                                          int H, int D, int P, int sink) {
+                                                          int H, int D, int P, int sink, int wide) {
   const int item = blockIdx.x, h = blockIdx.y;
   const size_t base = ((size_t)item * H + h) * P;
   float mx = NEG_INF;
@@ -259,7 +267,7 @@ __global__ __launch_bounds__(256) void attn_reduce_kernel(const int* __restrict_
       const float wgt = (mp == NEG_INF) ? 0.f : fexp<T>(mp - mx);
       num += part_acc[(base + p) * D + d] * wgt;
     }
-    out[((size_t)t * H + h) * D + d] = from_f32<T>(num * inv);
+    put(out, ((size_t)t * H + h) * D + d, num * inv, wide);
   }
 }
 
@@ -673,7 +681,7 @@ __global__ __launch_bounds__(256) void attn_decode_mfma_kernel(
         num *= e;
         den = den * e + __expf(-top);
       }
-      out[((size_t)t * H + h) * D + d] = (bf16)(num / den);
+      put(out, ((size_t)t * H + h) * D + d, num / den, sight.wide);
     } else {
       const size_t ob = ((size_t)item * H + h) * P + part;
       part_acc[ob * D + d] = num;
@@ -1079,7 +1087,14 @@ __global__ __launch_bounds__(256, 2) void attn_prefill_mfma_kernel(
       const float top = fmaxf(m[qt], 0.f), e = __builtin_amdgcn_exp2f(m[qt] - top);
       inv = e / (l[qt] * e + __builtin_amdgcn_exp2f(-top));
     }
-    bf16* orow = out + ((size_t)(tok0 + q0 + qt * 16 + col) * H + head) * D + 4 * grp;
+    const size_t at = ((size_t)(tok0 + q0 + qt * 16 + col) * H + head) * D + 4 * grp;
+    if (sight.wide) {
+      float* orow = reinterpret_cast<float*>(out) + at;
+#pragma unroll
+      for (int dt = 0; dt < DT; ++dt) *reinterpret_cast<f32x4_t*>(orow + dt * 16) = o[qt][dt] * inv;
+      continue;
+    }
+    bf16* orow = out + at;
 #pragma unroll
     for (int dt = 0; dt < DT; ++dt) {
       const bf16x4_t r4 = {(bf16)(o[qt][dt][0] * inv), (bf16)(o[qt][dt][1] * inv), (bf16)(o[qt][dt][2] * inv),
@@ -1094,7 +1109,7 @@ __global__ __launch_bounds__(256, 2) void attn_prefill_mfma_kernel(
 // largest maximum; a piece that saw no key has m = -inf and l = 0.
 template <int DC, int QT>
 __global__ __launch_bounds__(256) void attn_prefill_merge_kernel(const int* __restrict__ tiles, bf16* __restrict__ out,
-                                                                  int H, int KV, int units_z, PrefillSplit split, int sink) {
+                                                                  int H, int KV, int units_z, PrefillSplit split, int sink, int wide) {
   constexpr int D = DC * 32, DT = DC * 2, WQ = 16 * QT, PARTS = 64 / WQ;
   const int item = blockIdx.x;
   const int n = split.cut[item];
@@ -1127,6 +1142,12 @@ __global__ __launch_bounds__(256) void attn_prefill_merge_kernel(const int* __re
       for (int dt = 0; dt < DT; ++dt) sum[dt] += *reinterpret_cast<const f32x4_t*>(a + dt * 16) * w;
     }
     const float inv = 1.0f / den;
+    if (wide) {
+      float* orow = reinterpret_cast<float*>(out) + ((size_t)(tok0 + qi) * H + head) * D + 4 * grp;
+#pragma unroll
+      for (int dt = 0; dt < DT; ++dt) *reinterpret_cast<f32x4_t*>(orow + dt * 16) = sum[dt] * inv;
+      continue;
+    }
     bf16* orow = out + ((size_t)(tok0 + qi) * H + head) * D + 4 * grp;
 #pragma unroll
     for (int dt = 0; dt < DT; ++dt) {
@@ -1150,10 +1171,10 @@ __global__ __launch_bounds__(256) void attn_prefill_merge_kernel(const int* __re
 extern "C" int as_attn_prefill_mfma(const void* q, const void* k_pages, const void* v_pages, const int* tiles,
                                     int num_tiles, const int* block_tables, int table_width, void* out, int H,
                                     int KV, int D, int bs, float scale, int window, int keep, float cap, int sink,
-                                    int query_tiles, int pieces, int piece_rounds, int* cut, float* part_ml,
+                                    int wide, int query_tiles, int pieces, int piece_rounds, int* cut, float* part_ml,
                                     float* part_acc, hipStream_t stream) {
   if (num_tiles <= 0) return AS_OK;
-  const Sight sight{window, keep, cap, sink};
+  const Sight sight{window, keep, cap, sink, wide};
   if (!sight_ok(sight)) return AS_BAD_SHAPE;
   if (H <= 0 || KV <= 0 || H % KV || bs <= 0 || table_width <= 0) return AS_BAD_SHAPE;
   const int G = H / KV;
@@ -1175,7 +1196,7 @@ extern "C" int as_attn_prefill_mfma(const void* q, const void* k_pages, const vo
   if (cap > 0.f) LAUNCH2(DCV, QTV, true);                                                             \
   else LAUNCH2(DCV, QTV, false);                                                                      \
   if (pieces > 1)                                                                                     \
-    attn_prefill_merge_kernel<DCV, QTV><<<(int)items, 256, 0, stream>>>(tiles, (bf16*)out, H, KV, units_z, split, sink);
+    attn_prefill_merge_kernel<DCV, QTV><<<(int)items, 256, 0, stream>>>(tiles, (bf16*)out, H, KV, units_z, split, sink, wide);
 #define LAUNCH(DCV)              \
   if (query_tiles == 1) {        \
     LAUNCH1(DCV, 1)              \
@@ -1251,7 +1272,7 @@ static int launch_decode_mfma(const void* q, const void* k_pages, const void* v_
   if (hipGetLastError() != hipSuccess) return AS_LAUNCH_FAILED;
   if (P > 1) {
     attn_reduce_kernel<bf16><<<dim3(num_items, H), D <= 64 ? 64 : (D <= 128 ? 128 : 256), 0, stream>>>(
-        items, part_m, part_l, part_acc, (bf16*)out, H, D, P, sight.sink);
+        items, part_m, part_l, part_acc, (bf16*)out, H, D, P, sight.sink, sight.wide);
   }
   return launch_status();
 }
@@ -1261,14 +1282,14 @@ extern "C" int as_attn_decode_mfma(const void* q, const void* k_pages, const voi
                                    int num_items, const int* positions, const int* tok_row,
                                    const int* block_tables, int table_width, void* out, float* part_m,
                                    float* part_l, float* part_acc, int H, int KV, int D, int bs, float scale,
-                                   int window, int keep, float cap, int sink, int part_size, int P,
+                                   int window, int keep, float cap, int sink, int wide, int part_size, int P,
                                    hipStream_t stream) {
   if (num_items <= 0) return AS_OK;
   if (H <= 0 || KV <= 0 || H % KV || D <= 0 || bs <= 0 || part_size <= 0 || P <= 0 || table_width <= 0)
     return AS_BAD_SHAPE;
   if (P > 1 && (!part_m || !part_l || !part_acc)) return AS_BAD_SHAPE;
   return launch_decode_mfma(q, k_pages, v_pages, items, num_items, positions, tok_row, block_tables, table_width,
-                            out, part_m, part_l, part_acc, H, KV, D, bs, scale, Sight{window, keep, cap, sink},
+                            out, part_m, part_l, part_acc, H, KV, D, bs, scale, Sight{window, keep, cap, sink, wide},
                             part_size, P, nullptr, DT_BF16, stream);
 }
 
@@ -1278,14 +1299,14 @@ extern "C" int as_attn_decode_mfma_shared(const void* q, const void* k_pages, co
                                           int num_items, const int* positions, const int* tok_row,
                                           const int* block_tables, int table_width, void* out, float* part_m,
                                           float* part_l, float* part_acc, int H, int KV, int D, int bs, float scale,
-                                          int window, int keep, float cap, int sink, int part_size, int P,
+                                          int window, int keep, float cap, int sink, int wide, int part_size, int P,
                                           int share, hipStream_t stream) {
   if (num_items <= 0) return AS_OK;
   if (H <= 0 || KV <= 0 || H % KV || D <= 0 || bs <= 0 || part_size <= 0 || P <= 0 || table_width <= 0)
     return AS_BAD_SHAPE;
   if (P > 1 && (!part_m || !part_l || !part_acc)) return AS_BAD_SHAPE;
   return launch_decode_mfma(q, k_pages, v_pages, items, num_items, positions, tok_row, block_tables, table_width,
-                            out, part_m, part_l, part_acc, H, KV, D, bs, scale, Sight{window, keep, cap, sink},
+                            out, part_m, part_l, part_acc, H, KV, D, bs, scale, Sight{window, keep, cap, sink, wide},
                             part_size, P, nullptr, DT_BF16, stream, share);
 }
 
@@ -1309,7 +1330,7 @@ extern "C" int as_attn_decode_fresh(const void* qkv, const void* qw, const void*
   const FreshQKV fresh = {(const bf16*)qkv, qw, kw, (const float2*)cs, slots, (bf16*)k_pages, (bf16*)v_pages,
                           eps, store};
   return launch_decode_mfma(nullptr, k_pages, v_pages, items, num_tokens, positions, nullptr, block_tables,
-                            table_width, out, part_m, part_l, part_acc, H, KV, D, bs, scale, Sight{window, 0, 0.f, 0},
+                            table_width, out, part_m, part_l, part_acc, H, KV, D, bs, scale, Sight{window, 0, 0.f, 0, 0},
                             part_size, P, &fresh, gains_dtype, stream);
 }
 
@@ -1344,7 +1365,7 @@ static int launch_single_query(const void* q, const void* k_pages, const void* v
   if (hipGetLastError() != hipSuccess) return AS_LAUNCH_FAILED;
   if (P > 1) {
     attn_reduce_kernel<T><<<dim3(num_items, H), D <= 64 ? 64 : (D <= 128 ? 128 : 256), 0, stream>>>(
-        items, part_m, part_l, part_acc, (T*)out, H, D, P, sight.sink);
+        items, part_m, part_l, part_acc, (T*)out, H, D, P, sight.sink, sight.wide);
   }
   return launch_status();
 }
@@ -1355,7 +1376,7 @@ extern "C" int as_attn_single_query(const void* q, const void* k_pages, const vo
                                     const int* items, int num_items, const int* positions,
                                     const int* tok_row, const int* block_tables, int table_width, void* out,
                                     float* part_m, float* part_l, float* part_acc, int H, int KV, int D,
-                                    int bs, float scale, int window, int keep, float cap, int sink,
+                                    int bs, float scale, int window, int keep, float cap, int sink, int wide,
                                     int part_size, int P, hipStream_t stream) {
   if (num_items <= 0) return AS_OK;
   if (H <= 0 || KV <= 0 || H % KV || D <= 0 || bs <= 0 || part_size <= 0 || P <= 0 || table_width <= 0)
@@ -1364,11 +1385,11 @@ extern "C" int as_attn_single_query(const void* q, const void* k_pages, const vo
   if (dtype == DT_F32)
     return launch_single_query<float>(q, k_pages, v_pages, items, num_items, positions, tok_row, block_tables,
                                       table_width, out, part_m, part_l, part_acc, H, KV, D, bs, scale,
-                                      Sight{window, keep, cap, sink}, part_size, P, stream);
+                                      Sight{window, keep, cap, sink, wide}, part_size, P, stream);
   if (dtype == DT_BF16)
     return launch_single_query<bf16>(q, k_pages, v_pages, items, num_items, positions, tok_row, block_tables,
                                      table_width, out, part_m, part_l, part_acc, H, KV, D, bs, scale,
-                                     Sight{window, keep, cap, sink}, part_size, P, stream);
+                                     Sight{window, keep, cap, sink, wide}, part_size, P, stream);
   return AS_BAD_DTYPE;
 }
 
@@ -1400,6 +1421,10 @@ extern "C" int as_attn_single_query_static(const void* q, const void* k_pages, c
   if (num_items <= 0) return AS_OK;
   if (H <= 0 || KV <= 0 || H % KV || D <= 0 || bs <= 0 || part_size <= 0 || P <= 0 || table_width <= 0)
     return AS_BAD_SHAPE;
+  if (window > 0) {  // partitions cut the keys that the window shows: no more than these are ever filled
+    const int most = (int)(((long)window + part_size - 1) / part_size);
+    if (most < P) P = most;
+  }
   float *part_m = nullptr, *part_l = nullptr, *part_acc = nullptr;
   if (P > 1) {
     const unsigned long long rows = (unsigned long long)num_items * (unsigned long long)H * (unsigned long long)P;
@@ -1413,6 +1438,6 @@ extern "C" int as_attn_single_query_static(const void* q, const void* k_pages, c
     part_l = part_m + rows;
   }
   return as_attn_single_query(q, k_pages, v_pages, dtype, items, num_items, positions, tok_row, block_tables,
-                              table_width, out, part_m, part_l, part_acc, H, KV, D, bs, scale, window, 0, 0.f, 0,
+                              table_width, out, part_m, part_l, part_acc, H, KV, D, bs, scale, window, 0, 0.f, 0, 0,
                               part_size, P, stream);
 }

@@ -302,7 +302,8 @@ __global__ __launch_bounds__(256) void wide_attend_kernel(const T* __restrict__ 
                                                           const int* __restrict__ tok_row,
                                                           const int* __restrict__ block_tables, int table_width,
                                                           T* __restrict__ out, int H, int KV, int width, int bs,
-                                                          float scale, int window, int keep, float cap, int sink) {
+                                                          float scale, int window, int keep, float cap, int sink,
+                                                          int wide) {
   extern __shared__ float lds[];  // [width] the query, [256] the block's weights
   __shared__ float red[17];
   float* qs = lds;
@@ -363,13 +364,16 @@ __global__ __launch_bounds__(256) void wide_attend_kernel(const T* __restrict__ 
 #pragma unroll
   for (int c = 0; c < WIDE_MAX_COLS; ++c) {
     const int d = tid + 256 * c;
-    if (d < width) out[((size_t)t * H + h) * width + d] = from_f32<T>(acc[c] * shrink / l);
+    if (d >= width) continue;
+    const size_t at = ((size_t)t * H + h) * width + d;
+    if (wide) reinterpret_cast<float*>(out)[at] = acc[c] * shrink / l;  // a bfloat16 head's result in fp32
+    else out[at] = from_f32<T>(acc[c] * shrink / l);
   }
 }
 
 extern "C" int as_wide_attend(const void* q, const void* k_pages, const void* v_pages, int dtype, const int* positions,
                               const int* tok_row, const int* block_tables, int table_width, void* out, int H, int KV,
-                              int width, int bs, float scale, int window, int keep, float cap, int sink, int num_tokens,
+                              int width, int bs, float scale, int window, int keep, float cap, int sink, int wide, int num_tokens,
                               hipStream_t stream) {
   if (num_tokens <= 0) return AS_OK;
   if (H <= 0 || H > 65535 || KV <= 0 || H % KV || width <= 0 || width > 256 * WIDE_MAX_COLS || bs <= 0 || table_width <= 0) return AS_BAD_SHAPE;
@@ -378,10 +382,10 @@ extern "C" int as_wide_attend(const void* q, const void* k_pages, const void* v_
   const size_t lds = (size_t)(width + 256) * sizeof(float);
   if (dtype == DT_F32)
     wide_attend_kernel<float><<<grid, 256, lds, stream>>>((const float*)q, (const float*)k_pages, (const float*)v_pages, positions,
-                                                         tok_row, block_tables, table_width, (float*)out, H, KV, width, bs, scale, window, keep, cap, sink);
+                                                         tok_row, block_tables, table_width, (float*)out, H, KV, width, bs, scale, window, keep, cap, sink, wide);
   else if (dtype == DT_BF16)
     wide_attend_kernel<bf16><<<grid, 256, lds, stream>>>((const bf16*)q, (const bf16*)k_pages, (const bf16*)v_pages, positions,
-                                                        tok_row, block_tables, table_width, (bf16*)out, H, KV, width, bs, scale, window, keep, cap, sink);
+                                                        tok_row, block_tables, table_width, (bf16*)out, H, KV, width, bs, scale, window, keep, cap, sink, wide);
   else return AS_BAD_DTYPE;
   return launch_status();
 }

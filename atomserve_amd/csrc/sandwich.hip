@@ -165,7 +165,7 @@ static bool row_shape(int rows, int n, int vec, int* threads, int* pieces) {
   const int want = (n + vec - 1) / vec;
   int ch = rows >= 512 ? 4 : 1;
   while (ch > 1 && want <= 64 * ch / 2) ch /= 2;
-  while (ch < 8 && (want + ch - 1) / ch > 1024) ch *= 2;
+  while (ch < (vec == 1 ? 32 : 8) && (want + ch - 1) / ch > 1024) ch *= 2;
   const int t = ((want + ch - 1) / ch + 63) / 64 * 64;
   if (t > 1024) return false;
   *threads = t;
@@ -187,7 +187,13 @@ static int launch_post_norm(float* x, const void* y1, const void* y2, const Post
     case 1: LAUNCH(1); break;
     case 2: LAUNCH(2); break;
     case 4: LAUNCH(4); break;
-    default: LAUNCH(8); break;
+    case 8: LAUNCH(8); break;
+    default:  // long rows of a width that is no multiple of four
+      if constexpr (VEC == 1) {
+        if (ch == 16) { LAUNCH(16); }
+        else { LAUNCH(32); }
+      }
+      break;
   }
 #undef LAUNCH
   return launch_status();
@@ -253,7 +259,13 @@ static int launch_poly_norm(const void* z, const float* coef, float eps, void* o
     case 1: LAUNCH(1); break;
     case 2: LAUNCH(2); break;
     case 4: LAUNCH(4); break;
-    default: LAUNCH(8); break;
+    case 8: LAUNCH(8); break;
+    default:  // long rows of a width that is no multiple of four
+      if constexpr (VEC == 1) {
+        if (ch == 16) { LAUNCH(16); }
+        else { LAUNCH(32); }
+      }
+      break;
   }
 #undef LAUNCH
   return launch_status();
@@ -278,9 +290,9 @@ extern "C" int as_poly_norm(const void* z, int dtype, const float* coef, float e
 // (token, head): o = a1 - lam a2; out[t, out_off + h E + j] = mult * o_j / sqrt(mean(o^2) + eps).  E <= 4 * WAVE * PIECES.
 #define DIFF_PIECES 8
 
-template <typename T, int VEC>
+template <typename T, typename O, int VEC>
 __global__ __launch_bounds__(256) void map_difference_kernel(const T* __restrict__ heads, int H, int E, int Dp, float lam,
-                                                             float eps, float mult, T* __restrict__ out, int ld_out,
+                                                             float eps, float mult, O* __restrict__ out, int ld_out,
                                                              int out_off, int total) {
   const int item = blockIdx.x * 4 + threadIdx.x / WAVE, lane = threadIdx.x & (WAVE - 1);
   if (item >= total) return;
@@ -305,7 +317,7 @@ __global__ __launch_bounds__(256) void map_difference_kernel(const T* __restrict
   }
   ss = wave_sum(ss);
   const float f = mult / sqrtf(ss / (float)E + eps);
-  T* dst = out + t * ld_out + out_off + h * E;
+  O* dst = out + t * ld_out + out_off + h * E;
 #pragma unroll
   for (int c = 0; c < DIFF_PIECES; ++c) {
     const int i = (c * WAVE + lane) * VEC;
@@ -318,17 +330,21 @@ __global__ __launch_bounds__(256) void map_difference_kernel(const T* __restrict
 }
 
 extern "C" int as_map_difference(const void* heads, int dtype, int H, int E, int Dp, float lam, float eps, float mult, void* out,
-                                 int ld_out, int out_off, int num_tokens, hipStream_t stream) {
+                                 int out_dtype, int ld_out, int out_off, int num_tokens, hipStream_t stream) {
   if (num_tokens <= 0) return AS_OK;
   if (H <= 0 || E <= 0 || Dp < E || out_off < 0 || out_off + H * E > ld_out) return AS_BAD_SHAPE;
   const bool four = E % 4 == 0 && Dp % 4 == 0 && ld_out % 4 == 0 && out_off % 4 == 0;
   if (E > (four ? 4 : 1) * WAVE * DIFF_PIECES) return AS_BAD_SHAPE;
   if ((long)num_tokens * H > 0x7fffffffL) return AS_BAD_SHAPE;
   const int total = num_tokens * H, blocks = (total + 3) / 4;
-#define LAUNCH(T, VEC) \
-  map_difference_kernel<T, VEC><<<blocks, 256, 0, stream>>>((const T*)heads, H, E, Dp, lam, eps, mult, (T*)out, ld_out, out_off, total)
-  if (dtype == DT_F32) { if (four) LAUNCH(float, 4); else LAUNCH(float, 1); }
-  else if (dtype == DT_BF16) { if (four) LAUNCH(bf16, 4); else LAUNCH(bf16, 1); }
+#define LAUNCH(T, O)                                                                                                              \
+  if (four) map_difference_kernel<T, O, 4><<<blocks, 256, 0, stream>>>((const T*)heads, H, E, Dp, lam, eps, mult, (O*)out, ld_out, \
+                                                                       out_off, total);                                          \
+  else map_difference_kernel<T, O, 1><<<blocks, 256, 0, stream>>>((const T*)heads, H, E, Dp, lam, eps, mult, (O*)out, ld_out,      \
+                                                                  out_off, total)
+  if (dtype == DT_F32 && out_dtype == DT_F32) { LAUNCH(float, float); }
+  else if (dtype == DT_F32 && out_dtype == DT_BF16) { LAUNCH(float, bf16); }
+  else if (dtype == DT_BF16 && out_dtype == DT_BF16) { LAUNCH(bf16, bf16); }
   else return AS_BAD_DTYPE;
 #undef LAUNCH
   return launch_status();

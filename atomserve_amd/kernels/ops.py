@@ -208,11 +208,13 @@ def silu_mul(gate_up, out) -> None:
 SINGLE_QUERY_MAX_HEAD_DIM = 256
 
 
-def _sight(window, keep_first, softcap, sink) -> tuple:
-    """(window, keep, cap, sink) as the attention kernels take them: what a query sees and how scores become weights."""
+def _sight(window, keep_first, softcap, sink, q, out) -> tuple:
+    """(window, keep, cap, sink, wide) as the attention kernels take them: what a query sees, how scores become weights and
+    whether bfloat16 heads' results are written in fp32."""
+    _check(out, "out", (q.dtype, F32), tuple(q.shape))
     if window < 0 or keep_first < 0 or softcap < 0:
         raise KernelError("attention: a window, a number of kept tokens and a cap of the scores are not negative")
-    return int(window), int(keep_first) if window > 0 else 0, float(softcap), int(bool(sink))
+    return int(window), int(keep_first) if window > 0 else 0, float(softcap), int(bool(sink)), int(out.dtype != q.dtype)
 
 
 def attn_single_query(q, k_pages, v_pages, items, positions, tok_row, block_tables, out, scale, window,
@@ -222,15 +224,14 @@ def attn_single_query(q, k_pages, v_pages, items, positions, tok_row, block_tabl
     heads, or of wide heads that overfill a workgroup's LDS, as several equal groups that read the same kv
     head); everything else (and all of fp32) on the general kernel.
 
-    q, out [T, H, D]; items [N] int32: the tokens (rows of q) to process, None for all of them in
+    q, out [T, H, D] (out fp32 for bfloat16 heads: the results unrounded); items [N] int32: the tokens (rows of q) to process, None for all of them in
     order; positions, tok_row [T] int32 (tok_row None: token t belongs to row t, a decode step);
     block_tables [R, W] int32; max_context: host bound on positions[items] + 1.
     window > 0: a query at p sees the keys p - window + 1 .. p and those of the first `keep_first` positions.
     softcap > 0: a score s counts as softcap tanh(s / softcap).  sink: the softmax's denominator has one more score of 0."""
     _check(q, "q", (F32, BF16), (None, None, None))
     T, H, D = q.shape
-    sight = _sight(window, keep_first, softcap, sink)
-    _check(out, "out", q.dtype, (T, H, D))
+    sight = _sight(window, keep_first, softcap, sink, q, out)
     _check(k_pages, "k_pages", q.dtype, (None, None, None, D))
     _, KV, bs, _ = k_pages.shape
     _check(v_pages, "v_pages", q.dtype, (k_pages.shape[0], KV, D, bs))
@@ -519,8 +520,7 @@ def attn_prefill(q, k_pages, v_pages, tiles, block_tables, out, scale, window, m
     window, keep_first, softcap, sink: as for `attn_single_query`."""
     _check(q, "q", BF16, (None, None, None))
     T, H, D = q.shape
-    sight = _sight(window, keep_first, softcap, sink)
-    _check(out, "out", BF16, (T, H, D))
+    sight = _sight(window, keep_first, softcap, sink, q, out)
     _check(k_pages, "k_pages", BF16, (None, None, None, D))
     _, KV, bs, _ = k_pages.shape
     _check(v_pages, "v_pages", BF16, (k_pages.shape[0], KV, D, bs))
@@ -1212,15 +1212,15 @@ def whole_norm_store(proj, q_off, k_off, v_off, num_heads, num_kv_heads, dim, vd
 
 
 def map_difference(heads, vdim, lam, eps, mult, out, out_off: int = 0) -> None:
-    """heads [T, 2 H, Dp]: head h's two attention maps at 2 h and 2 h + 1, `vdim` coordinates wide.  With o = a1 - lam a2:
+    """heads [T, 2 H, Dp] (out's dtype, or fp32): head h's two attention maps at 2 h and 2 h + 1, `vdim` coordinates wide.  With o = a1 - lam a2:
     out[t, out_off + h * vdim + j] = mult * o_j / sqrt(mean(o^2) + eps)."""
     _check(heads, "heads", (F32, BF16), (None, None, None))
     T, H2, Dp = heads.shape
-    _check(out, "out", heads.dtype, (T, None))
+    _check(out, "out", (F32, BF16) if heads.dtype == F32 else BF16, (T, None))
     if H2 % 2 or not 1 <= vdim <= Dp or out_off < 0 or out_off + H2 // 2 * vdim > out.shape[1]:
         raise KernelError(f"map_difference: {H2} maps of {Dp} coordinates, {vdim} of them values, columns {out_off}.. of {out.shape[1]}")
     call("as_map_difference", _ptr(heads), _DT[heads.dtype], H2 // 2, vdim, Dp, float(lam), float(eps), float(mult), _ptr(out),
-         out.shape[1], out_off, T, _stream())  # fmt: skip
+         _DT[out.dtype], out.shape[1], out_off, T, _stream())  # fmt: skip
 
 
 STREAMS_MAX = 16
@@ -2165,10 +2165,10 @@ def wide_attend(q, k_pages, v_pages, positions, tok_row, block_tables, out, scal
     """Causal attention of every token's heads q [T, H, width] over kv heads of any width up to
     WIDE_ATTEND_MAX_WIDTH (k_pages [pages, KV, bs, width], v_pages [pages, KV, width, bs]): for pages wider than the
     paged attention kernels' heads.  positions, tok_row [T] int32 (tok_row None: token t is row t); out like q.
-    window, keep_first, softcap, sink: as for `attn_single_query`."""
+    window, keep_first, softcap, sink, and out in fp32 for bfloat16 heads: as for `attn_single_query`."""
     _check(q, "q", (F32, BF16), (None, None, None))
     T, H, width = q.shape
-    _check(out, "out", q.dtype, (T, H, width))
+    sight = _sight(window, keep_first, softcap, sink, q, out)
     _check(k_pages, "k_pages", q.dtype, (None, None, None, width))
     pages, KV, bs, _ = k_pages.shape
     _check(v_pages, "v_pages", q.dtype, (pages, KV, width, bs))
@@ -2186,4 +2186,4 @@ def wide_attend(q, k_pages, v_pages, positions, tok_row, block_tables, out, scal
         raise KernelError("attention: block tables are shorter than the longest context")
     call("as_wide_attend", _ptr(q), _ptr(k_pages), _ptr(v_pages), _DT[q.dtype], _ptr(positions), _ptr(tok_row),
          _ptr(block_tables), block_tables.shape[1], _ptr(out), H, KV, width, bs, float(scale),
-         *_sight(window, keep_first, softcap, sink), T, _stream())  # fmt: skip
+         *sight, T, _stream())  # fmt: skip

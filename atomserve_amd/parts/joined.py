@@ -157,7 +157,8 @@ class SoftmaxCore:
             # the core alone, its heads as wide as they are laid out: the attention writes the output product's input itself
             attend(q, act.view(T, H, Dp), step, pages, s.scale, s.window, (SHORT_ROW, TILE_Q), **how)
             return
-        heads = torch.empty((T, queries, Dp), dtype=env.dtype, device=dev)
+        # two maps may nearly cancel: their heads reach the difference unrounded
+        heads = torch.empty((T, queries, Dp), dtype=torch.float32 if s.maps == 2 else env.dtype, device=dev)
         attend(q, heads, step, pages, s.scale, s.window, (SHORT_ROW, TILE_Q), **how)
         if s.maps == 2:
             ops.map_difference(heads, s.value_dim, self.map_lambda, s.difference_eps, scale * (1.0 - s.difference), act, out_off)

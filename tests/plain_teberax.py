@@ -112,7 +112,7 @@ def differential_attention(h, W, p, m, eps, bf16, kept, index):
     a1 = attention(q[:, :, 0], k1, v, m["scale"], m.get("mask"))
     a2 = attention(q[:, :, 1], k2, v, m["scale"], m.get("mask"))
     lam = differential_lambda(W, p, m["diff"], h.dtype)
-    o = differential_combine(rnd(a1, bf16), rnd(a2, bf16), lam, m["diff"], eps)
+    o = differential_combine(a1, a2, lam, m["diff"], eps)
     return linear(W[p + "o"], o.reshape(T, H * E), bf16)
 
 
