@@ -762,6 +762,89 @@ __global__ __launch_bounds__(256) void whole_norm_store_kernel(
   }
 }
 
+// The same for bfloat16 without a norm over the projection and without mixed values, where every width and offset is a
+// multiple of eight: 16 bytes of a head a thread (its bias, its partner if it turns), and for values of a prompt the
+// eight tokens that fill eight slots in a row together, each an eighth of the coordinates (see
+// qk_norm_rope_store_bf16x8_kernel).
+__global__ __launch_bounds__(256) void whole_store_bf16x8_kernel(
+    const bf16* __restrict__ proj, int ld, int q_off, int k_off, int v_off, int H, int KV, int dim, int vdim, int Dp,
+    const float* __restrict__ q_bias, const float* __restrict__ k_bias, const float* __restrict__ v_bias,
+    const float2* __restrict__ cs, int half, const int* __restrict__ slots, bf16* __restrict__ q_out,
+    bf16* __restrict__ k_pages, bf16* __restrict__ v_pages, int bs, int store, int maps, int num_tokens, size_t units) {
+  typedef __bf16 bf16x8 __attribute__((ext_vector_type(8)));
+  const size_t unit = (size_t)blockIdx.x * blockDim.x + threadIdx.x;
+  if (unit >= units) return;
+  const int pieces = Dp >> 3, heads = store ? H + 2 * KV : H;
+  const int p = (int)(unit % pieces);
+  const int head = (int)(unit / pieces % heads);
+  const int t = (int)(unit / pieces / heads);
+  const bf16* row = proj + (size_t)t * ld;
+  const int slot = (store && head >= H) ? slots[t] : 0;
+  if (slot < 0) return;
+  if (head < H + KV) {  // a query or a key head
+    const bool is_k = head >= H;
+    const int hh = is_k ? head - H : head, wide = is_k ? dim : dim / maps, at = is_k ? 0 : (hh % maps) * wide;
+    const int d = 8 * p;
+    const float* bias = is_k ? k_bias : q_bias;
+    float v[8] = {0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f}, u[8], b[8];
+    auto piece = [&](int dd, float* x) {  // eight coordinates of the head, bias added
+      const int c = hh * wide + dd - at;
+      const bf16x8 r = *reinterpret_cast<const bf16x8*>(row + (is_k ? k_off : q_off) + c);
+#pragma unroll
+      for (int j = 0; j < 8; ++j) x[j] = (float)r[j];
+      if (bias) {
+        Gain8<float>::load(bias + c, b);
+#pragma unroll
+        for (int j = 0; j < 8; ++j) x[j] += b[j];
+      }
+    };
+    if (d >= at && d < at + wide) piece(d, v);
+    if (d < 2 * half) {
+      piece(d < half ? d + half : d - half, u);
+      const float4* turn = reinterpret_cast<const float4*>(cs + (size_t)t * half + (d < half ? d : d - half));
+#pragma unroll
+      for (int j = 0; j < 4; ++j) {
+        const float4 a = turn[j];
+        v[2 * j] = d < half ? v[2 * j] * a.x - u[2 * j] * a.y : v[2 * j] * a.x + u[2 * j] * a.y;
+        v[2 * j + 1] = d < half ? v[2 * j + 1] * a.z - u[2 * j + 1] * a.w : v[2 * j + 1] * a.z + u[2 * j + 1] * a.w;
+      }
+    }
+    bf16x8 o;
+#pragma unroll
+    for (int j = 0; j < 8; ++j) o[j] = (bf16)finite_or_zero(v[j]);
+    bf16* dst = is_k ? k_pages + (((size_t)(slot / bs) * KV + hh) * bs + slot % bs) * Dp : q_out + ((size_t)t * H + hh) * Dp;
+    *reinterpret_cast<bf16x8*>(dst + d) = o;
+    return;
+  }
+  const int g = head - H - KV;  // a value head
+  bf16* page = v_pages + ((size_t)(slot / bs) * KV + g) * Dp * bs;
+  const int nth = slot & 7, lead = t - nth;
+  bool run = lead >= 0 && lead + 8 <= num_tokens;
+  if (run) {
+#pragma unroll
+    for (int i = 0; i < 8; ++i) run = run && slots[lead + i] == slot - nth + i;
+  }
+  if (run) {  // the same for all eight tokens: this one takes its eighth of the coordinates of all of them
+    const int d = nth * pieces + p;
+    bf16x8 o;
+#pragma unroll
+    for (int i = 0; i < 8; ++i) {
+      float v = 0.f;
+      if (d < vdim) v = (float)proj[(size_t)(lead + i) * ld + v_off + g * vdim + d] + (v_bias ? v_bias[g * vdim + d] : 0.f);
+      o[i] = (bf16)finite_or_zero(v);
+    }
+    *reinterpret_cast<bf16x8*>(page + (size_t)d * bs + (slot - nth) % bs) = o;
+    return;
+  }
+#pragma unroll
+  for (int j = 0; j < 8; ++j) {
+    const int d = 8 * p + j;
+    float v = 0.f;
+    if (d < vdim) v = (float)row[v_off + g * vdim + d] + (v_bias ? v_bias[g * vdim + d] : 0.f);
+    page[(size_t)d * bs + slot % bs] = (bf16)finite_or_zero(v);
+  }
+}
+
 extern "C" int as_whole_norm_store(const void* proj, int dtype, int ld, int q_off, int k_off, int v_off, int H, int KV,
                                    int dim, int vdim, int Dp, const float* q_bias, const float* k_bias,
                                    const float* v_bias, const float* qw, const float* kw, float eps, const float* cs,
@@ -774,6 +857,17 @@ extern "C" int as_whole_norm_store(const void* proj, int dtype, int ld, int q_of
     return AS_BAD_SHAPE;
   if (v_mode < 0 || v_mode > 2 || (v_mode && !v_keep)) return AS_BAD_SHAPE;
   if (maps < 1 || (maps > 1 && (cs || qw || dim % maps || H % maps))) return AS_BAD_SHAPE;
+  const int eights = ld | q_off | k_off | v_off | dim | dim / maps | vdim | Dp | (cs ? R / 2 : 0) | (store ? bs : 0);
+  if (dtype == DT_BF16 && !qw && v_mode == 0 && (eights & 7) == 0) {
+    const size_t units = (size_t)num_tokens * (store ? H + 2 * KV : H) * (Dp / 8);
+    const size_t blocks = (units + 255) / 256;
+    if (blocks > 0x7fffffffUL) return AS_BAD_SHAPE;
+    whole_store_bf16x8_kernel<<<(int)blocks, 256, 0, stream>>>((const bf16*)proj, ld, q_off, k_off, v_off, H, KV, dim, vdim, Dp,
+                                                               q_bias, k_bias, v_bias, (const float2*)cs, cs ? R / 2 : 0, slots,
+                                                               (bf16*)q_out, (bf16*)k_pages, (bf16*)v_pages, bs, store, maps,
+                                                               num_tokens, units);
+    return launch_status();
+  }
   // few tokens (a decode step): a token's heads are dealt out over several workgroups; many: one takes them all
   int across = num_tokens >= 256 ? 1 : (H + 2 * KV < 32 ? H + 2 * KV : 32);
   const int threads = across > 1 && Dp <= 128 ? (Dp > 64 ? 128 : 64) : 256;

@@ -633,8 +633,57 @@ extern "C" int as_channel_chunks(const void* proj, int dtype, int ld, int q_off,
 // ---- decays per channel from a two-step projection ---------------------------------------------------------------------
 // low: columns low_off .. + rank of proj [T, ld] (the first step's result); up [C, rank] (T-typed), bias [C] fp32.
 //   alpha[t, c] = max(sigmoid(z)^(1 / tau), CHANNEL_MIN),  z = sum_r low[t, r] up[c, r] + bias[c],  all of it in fp32.
-// grid (tiles of DECAY_TOKENS tokens, 256 channels): a thread owns a channel for the tile's tokens.
+// Two kernels: bfloat16 with rows on 16 bytes on the matrix cores (a wave 16 tokens of 64 channels: the products' sums are
+// fp32 as they are), anything else with a thread per channel for DECAY_TOKENS tokens.
 #define DECAY_TOKENS 16
+
+// sigmoid(z)^(1 / tau); for bfloat16 inputs through the hardware's exponential and logarithm, whose error is that of the
+// 32-bit result.
+template <typename T> __device__ __forceinline__ float root_sigmoid(float z, float inv_tau) {
+  const float log_s = fminf(z, 0.f) - log1pf(expf(-fabsf(z)));
+  return fmaxf(expf(log_s * inv_tau), CHANNEL_MIN);
+}
+template <> __device__ __forceinline__ float root_sigmoid<bf16>(float z, float inv_tau) {
+  const float z2 = z * 1.4426950408889634f;  // in base 2
+  const float log_s = fminf(z2, 0.f) - __builtin_amdgcn_logf(1.f + __builtin_amdgcn_exp2f(-fabsf(z2)));
+  return fmaxf(__builtin_amdgcn_exp2f(log_s * inv_tau), CHANNEL_MIN);
+}
+
+typedef __bf16 bf16x8 __attribute__((ext_vector_type(8)));
+#define DECAY_STRIP 64
+__global__ __launch_bounds__(256) void channel_decays_mfma_kernel(const bf16* __restrict__ proj, int ld, int low_off, int rank,
+                                                                  const bf16* __restrict__ up, const float* __restrict__ bias,
+                                                                  float inv_tau, float* __restrict__ alpha, int C,
+                                                                  int num_tokens) {
+  const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6, lr = lane & 15, lg = lane >> 4;
+  const int t = (blockIdx.x * 4 + wave) * 16 + lr, c0 = blockIdx.y * DECAY_STRIP;
+  if ((blockIdx.x * 4 + wave) * 16 >= num_tokens) return;
+  const bf16x8 zero = {0, 0, 0, 0, 0, 0, 0, 0};
+  floatx4 acc[4];
+#pragma unroll
+  for (int n = 0; n < 4; ++n) acc[n] = floatx4{0.f, 0.f, 0.f, 0.f};
+  for (int k0 = 0; k0 < rank; k0 += 32) {
+    const int k = k0 + lg * 8;
+    const bf16x8 b = t < num_tokens && k < rank ? *reinterpret_cast<const bf16x8*>(proj + (size_t)t * ld + low_off + k) : zero;
+#pragma unroll
+    for (int n = 0; n < 4; ++n) {
+      const int c = c0 + n * 16 + lr;
+      const bf16x8 a = c < C && k < rank ? *reinterpret_cast<const bf16x8*>(up + (size_t)c * rank + k) : zero;
+      acc[n] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(a, b, acc[n], 0, 0, 0);
+    }
+  }
+  if (t >= num_tokens) return;
+#pragma unroll
+  for (int n = 0; n < 4; ++n) {  // this lane: channels c .. c + 3 of token t
+    const int c = c0 + n * 16 + 4 * lg;
+    if (c >= C) continue;
+    float b4[4], v[4];
+    load4(bias + c, b4);
+#pragma unroll
+    for (int i = 0; i < 4; ++i) v[i] = root_sigmoid<bf16>(acc[n][i] + b4[i], inv_tau);
+    store4(alpha + (size_t)t * C + c, v);
+  }
+}
 
 template <typename T>
 __global__ __launch_bounds__(256) void channel_decays_kernel(const T* __restrict__ proj, int ld, int low_off, int rank,
@@ -671,10 +720,7 @@ __global__ __launch_bounds__(256) void channel_decays_kernel(const T* __restrict
   }
 #pragma unroll
   for (int tq = 0; tq < DECAY_TOKENS; ++tq) {
-    if (tq < nt) {
-      const float log_s = fminf(z[tq], 0.f) - log1pf(expf(-fabsf(z[tq])));
-      alpha[(size_t)(t0 + tq) * C + c] = fmaxf(expf(log_s * inv_tau), CHANNEL_MIN);
-    }
+    if (tq < nt) alpha[(size_t)(t0 + tq) * C + c] = root_sigmoid<T>(z[tq], inv_tau);
   }
 }
 
@@ -685,6 +731,12 @@ extern "C" int as_channel_decays(const void* proj, int dtype, int ld, int low_of
   dim3 grid((num_tokens + DECAY_TOKENS - 1) / DECAY_TOKENS, (C + 255) / 256);
   if (grid.y > 65535) return AS_BAD_SHAPE;
   const size_t lds = (size_t)rank * DECAY_TOKENS * sizeof(float);
+  if (dtype == DT_BF16 && rank % 8 == 0 && ld % 8 == 0 && low_off % 8 == 0 && C % 4 == 0) {
+    dim3 tiles((num_tokens + 63) / 64, (C + DECAY_STRIP - 1) / DECAY_STRIP);
+    if (tiles.y > 65535) return AS_BAD_SHAPE;
+    channel_decays_mfma_kernel<<<tiles, 256, 0, stream>>>((const bf16*)proj, ld, low_off, rank, (const bf16*)up, bias, 1.0f / tau, alpha, C, num_tokens);
+    return launch_status();
+  }
   if (dtype == DT_F32)
     channel_decays_kernel<float><<<grid, 256, lds, stream>>>((const float*)proj, ld, low_off, rank, (const float*)up, bias, 1.0f / tau, alpha, C, num_tokens);
   else if (dtype == DT_BF16)

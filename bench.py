@@ -6,6 +6,7 @@
     python bench.py --design koravik [--widths 1024,2048,4096]   (Koravik layers beside Qwen3 layers of equal size)
     python bench.py --design mumizen [--widths 1024,2048,4096]   (Mumizen layers beside Qwen3 layers of equal size)
     python bench.py --design natatar [--widths 1024,2048,4096]   (Natatar layers beside Dozusun and Qwen3 layers of equal size)
+    python bench.py --design teberax [--widths 1024,2048,4096]   (Teberax layers beside Mumizen and Qwen3 layers of equal size)
 
 A step is one decode step of the engine (scheduler, one pass over the GPU, sampling).
 Prints ONE JSON line: decoded tokens per second at batch 8 with 2,048-token contexts,
@@ -78,7 +79,7 @@ def parse_args():
                         "(half of them share their first 32), chunks of 512, 128 tokens decoded each, through the "
                         "scheduler from submission to the last token")  # fmt: skip
     p.add_argument("--chunk-budget", type=int, default=512, help="token budget of a step in the mixed workload")
-    p.add_argument("--design", choices=["qwen3", "dozusun", "koravik", "mumizen", "natatar"], default="qwen3",
+    p.add_argument("--design", choices=["qwen3", "dozusun", "koravik", "mumizen", "natatar", "teberax"], default="qwen3",
                    help="dozusun: prefill and decode throughput of random-weight Dozusun layers (an attention beside a "
                         "gated linear recurrence, gated delta rules, dense and table-routed feed-forwards) at a few "
                         "widths, beside Qwen3 layers of the same width, heads, depth and vocabulary; koravik: the same "
@@ -86,7 +87,7 @@ def parse_args():
                         "shared one, gated residual sums, a stretch of layers run twice); mumizen: the same for Mumizen "
                         "layers (linear attentions with fixed decays, attention through a cached latent, gated "
                         "feed-forwards with limits, dense and routed, an average over all layers' results)")  # fmt: skip
-    p.add_argument("--widths", default="1024,2048,4096", help="stream widths of --design dozusun / koravik / mumizen")
+    p.add_argument("--widths", default="1024,2048,4096", help="stream widths of the designs")
     p.add_argument("--profile", action="store_true",
                    help="also split the host's time of a decode step into schedule / pack / launch / sample / wait / "
                         "update (steps run one at a time meanwhile, none sent ahead), as the reference's "
@@ -262,12 +263,48 @@ def natatar_config(width: int, layers: int, vocab: int):
                                     "layers": [{"type": kinds[i % 4][0], "mixer": kinds[i % 4][1], "mlp": mlp} for i in range(layers)]})  # fmt: skip
 
 
+def teberax_config(width: int, layers: int, vocab: int):
+    """Layers as a model of this design of that width would have them: values of 128 everywhere; differential attentions
+    with two maps of 64, a kv head to four query heads and a window of 1,024 that keeps the first 64 tokens, every second
+    one reading the keys of the one before; a rotary attention with heads of 128 (64 coordinates turned, capped scores,
+    a sink) beside a linear attention with as many heads of 128 x 128 and decays of rank 64; attention through a latent of
+    192 beside a turned part of 64 over a window of 1,024; feed-forwards dense and four times the width (without a gate), or
+    16 experts of three quarters of the width and 4 identity experts, two to a token; the four kinds of layers in turn."""
+    from atomserve_amd.config.model_config import TeberaxConfig
+
+    heads = width // 128
+    kv = max(1, heads // 4)
+    mask = {"size": 1024, "keep_first": 64}
+    attention = {"heads": heads, "kv_heads": kv, "dim": 64, "vdim": 128, "scale": 0.125, "diff": 0.4, "mask": mask}
+    side = {"left": {"heads": heads, "kv_heads": kv, "dim": 128, "vdim": 128, "scale": 128**-0.5, "softcap": 30.0,
+                     "rot": {"dims": 64, "base": 1e6, "scaling": {"factor": 4.0}}},
+            "right": {"heads": heads, "dim": 128, "vdim": 128, "tau": 8.0, "rank": 64}}  # fmt: skip
+    latent = {"heads": heads, "dim": 128, "rot_dim": 64, "vdim": 128, "kv_rank": 192, "scale": 192**-0.5, "rot": {"dims": 64, "base": 1e6},
+              "mask": {"size": 1024}}  # fmt: skip
+    dense = {"kind": "dense", "ff": 4 * width}
+    moe = {"kind": "moe", "expert": {"ff": 3 * width // 4}, "router": {"experts": 16, "top": 2, "identity": 4}}
+    made = []
+    for i in range(layers):
+        kind = i % 4
+        if kind == 0:
+            made.append({"type": "attention", "mixer": attention, "mlp": dense})
+        elif kind == 1:
+            made.append({"type": "parallel", "mixer": side, "mlp": moe})
+        elif kind == 2:
+            made.append({"type": "attention", "mixer": dict(attention, kv_from=i - 2), "mlp": dense})
+        else:
+            made.append({"type": "latent_attention", "mixer": latent, "mlp": moe})
+    return TeberaxConfig.from_dict({"architecture": "Teberax", "vocab": vocab, "width": width, "norm": {"eps": 1e-6},
+                                    "logit_softcap": 25.0, "layers": made})  # fmt: skip
+
+
 def design_comparison(args) -> dict:
     """Prefill of --prefill-tokens tokens and decode at batch 1 and --batch with --context tokens of context, for
     the layers of --design and for Qwen3 layers of equal width, heads, depth and vocabulary; random weights, the
     engine's own entry point (scheduler, captured decode steps, sampling)."""
     design = args.design
-    make = {"dozusun": dozusun_config, "koravik": koravik_config, "mumizen": mumizen_config, "natatar": natatar_config}[design]
+    make = {"dozusun": dozusun_config, "koravik": koravik_config, "mumizen": mumizen_config, "natatar": natatar_config,
+            "teberax": teberax_config}[design]  # fmt: skip
     import torch
 
     from atomserve_amd.config import EngineConfig, Qwen3Config
@@ -336,6 +373,8 @@ def design_comparison(args) -> dict:
         sizes[str(width)] = {design: measure(make(width, layers, vocab)), "qwen3": measure(qwen)}
         if design == "natatar":  # its closest relative among the designs: a delta rule, an attention beside a recurrence, experts
             sizes[str(width)]["dozusun"] = measure(dozusun_config(width, layers, vocab))
+        if design == "teberax":  # its closest relative: a linear attention with decays, a latent that layers share, dense and routed
+            sizes[str(width)]["mumizen"] = measure(mumizen_config(width, layers, vocab))
         print(f"width {width}: {json.dumps(sizes[str(width)])}", file=sys.stderr, flush=True)
     widest = sizes[max(sizes, key=int)]
     return {
@@ -390,7 +429,7 @@ def main() -> int:
     from atomserve_amd.weights.loader import DictSource, bind_checkpoint
     from atomserve_amd.weights.random_init import random_checkpoint
 
-    if args.design in ("dozusun", "koravik", "mumizen", "natatar"):
+    if args.design != "qwen3":
         print(json.dumps(design_comparison(args)))
         return 0
     device = "cuda:0"

@@ -678,6 +678,12 @@ def test_channel_decays_and_the_three_ways_to_run_them(sizes, dtype):
     z = proj[:, -rank:].double() @ up.double().t() + bias.double()
     exact = plain.channel_decays(z, tau)
     assert (alpha.cpu().double() - exact).abs().max() <= 2e-6
+    for n, wide, tau_ in ((8, 8, 0.25), (77, 40, 16.0), (130, 64, 1.0)):  # ranks whose second step runs on the matrix cores
+        low, up_, b_ = bf(torch.randn(n, wide + 8, generator=gen)), bf(torch.randn(H * D, wide, generator=gen)), torch.randn(H * D, generator=gen) * 20
+        out = torch.full((n, H * D), float("nan"), dtype=torch.float32, device=DEV)
+        ops.channel_decays(low.to(DEV).to(dt), 8, wide, up_.to(DEV).to(dt), b_.to(DEV), tau_, out)
+        want_ = plain.channel_decays(low[:, 8:].double() @ up_.double().t() + b_.double(), tau_)
+        assert (out.cpu().double() - want_).abs().max() <= 2e-6, (n, wide, tau_)
     al = exact.float().view(T, H, D).clone()
     pick = torch.rand(T, H, D, generator=gen)
     al[pick < 0.1] = 1.0
