@@ -86,7 +86,8 @@ def parse_args():
                         "for Koravik layers (attention with mixed heads and kept first tokens, routed experts with a "
                         "shared one, gated residual sums, a stretch of layers run twice); mumizen: the same for Mumizen "
                         "layers (linear attentions with fixed decays, attention through a cached latent, gated "
-                        "feed-forwards with limits, dense and routed, an average over all layers' results)")  # fmt: skip
+                        "feed-forwards with limits, dense and routed, an average over all layers' results); natatar: the same for "
+                        "Natatar layers, Dozusun's beside them; teberax: the same for Teberax layers, Mumizen's beside them")  # fmt: skip
     p.add_argument("--widths", default="1024,2048,4096", help="stream widths of the designs")
     p.add_argument("--profile", action="store_true",
                    help="also split the host's time of a decode step into schedule / pack / launch / sample / wait / "
