@@ -45,6 +45,8 @@ static inline bool sight_ok(const Sight& s) {
   return s.window >= 0 && s.keep >= 0 && (s.keep == 0 || s.window > 0) && s.cap >= 0.f && (s.sink == 0 || s.sink == 1) &&
          (s.wide == 0 || s.wide == 1);
 }
+// Which instance of the matrix-core kernels computes it (`SEE` below).
+static inline int needed_sight(const Sight& s) { return s.cap > 0.f ? 2 : (s.keep > 0 || s.sink || s.wide) ? 1 : 0; }
 
 // tanh through the hardware's exponential and reciprocal: an absolute error of 1e-7, which is what a capped score
 // (times the cap) of the bf16 kernels may carry.
@@ -396,7 +398,9 @@ __device__ __forceinline__ void load_gains8(const bf16* w, float* g) {
   for (int j = 0; j < 8; ++j) g[j] = (float)v[j];
 }
 
-template <int DC, int FRESH, bool CAP>  // D / 32; FRESH 0: finished queries, 1: qkv with bf16 gains, 2: with fp32 gains
+// D / 32; FRESH 0: finished queries, 1: qkv with bf16 gains, 2: with fp32 gains; SEE 0: a window at most (nothing of the rest of
+// `sight` is read), 1: kept first tokens, a sink and fp32 outputs too, 2: also capped scores
+template <int DC, int FRESH, int SEE>
 __global__ __launch_bounds__(256) void attn_decode_mfma_kernel(
     const bf16* __restrict__ q, const bf16* __restrict__ k_pages, const bf16* __restrict__ v_pages,
     const int* __restrict__ items, const int* __restrict__ positions, const int* __restrict__ tok_row,
@@ -430,18 +434,23 @@ __global__ __launch_bounds__(256) void attn_decode_mfma_kernel(
   const int ctx = pos + 1;
   // The keys are walked in steps of 32: first those that hold kept tokens (`kept_steps` from the sequence's start), then
   // those of the window (from step `base` on); where the two meet it is one run from the start.  Partitions cut this list.
-  const int lo = first_in_window(sight, ctx), kept = min(sight.keep, lo);
+  // Without kept tokens a place in the list is counted in keys, from the step that the window starts in (`k0` ..).
+  const int lo = first_in_window(sight, ctx), kept = SEE >= 1 ? min(sight.keep, lo) : 0;
   int kept_steps = (kept + 31) / 32, base = lo / 32;
   if (kept_steps > 0 && kept_steps >= base) kept_steps = base = 0;
   const int steps = kept_steps + (ctx - 1) / 32 - base + 1;
-  const int s0 = part * (part_size / 32), s1 = min(steps, (part + 1) * (part_size / 32));
-  auto first_key = [&](int step) { return 32 * (step < kept_steps ? step : step - kept_steps + base); };
+  const int k0 = 32 * base + part * part_size, k1 = min(ctx, k0 + part_size);
+  const int from = SEE >= 1 ? part * (part_size / 32) : k0;
+  const int to = SEE >= 1 ? min(steps, from + part_size / 32) : k1;
+  constexpr int NEXT = SEE >= 1 ? 1 : 32;  // from a step to the next one
+  const int bound = SEE >= 1 ? ctx : k1;
+  auto first_key = [&](int at) { return SEE >= 1 ? 32 * (at < kept_steps ? at : at - kept_steps + base) : at; };
   const int h0 = kvh * G;
   const int page_heads = KV / share, page_head = kvh / share;
   const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
   const int col = lane & 15, grp = lane >> 4;  // col: head within the group (and key row of A)
 
-  if (s0 >= s1) {  // an empty partition (P > 1 only): mark it so for the reduce
+  if (from >= to) {  // an empty partition (P > 1 only): mark it so for the reduce
     if (tid < G) {
       const size_t o = ((size_t)item * H + h0 + tid) * P + part;
       part_m[o] = NEG_INF;
@@ -484,7 +493,7 @@ __global__ __launch_bounds__(256) void attn_decode_mfma_kernel(
 #pragma unroll
       for (int j = 0; j < 4; ++j) angle[c * 4 + j] = cs4[j];
     }
-    fresh_here = fresh.store && s1 == steps;  // the same for the whole workgroup
+    fresh_here = fresh.store && pos >= k0 && pos < k1;  // the same for the whole workgroup
     if (fresh_here && wave == 0) {
       slot = fresh.slots[t];
       const bf16* src = fresh.qkv + (row + H + kvh) * D;
@@ -505,7 +514,8 @@ __global__ __launch_bounds__(256) void attn_decode_mfma_kernel(
     }
   }
   KVStep<DC> cur, nxt;
-  if (s0 + wave < s1) load_kv_step<DC>(cur, k_pages, v_pages, table, first_key(s0 + wave), ctx, page_heads, page_head, bs, col, grp);
+  int at = from + NEXT * wave;
+  if (at < to) load_kv_step<DC>(cur, k_pages, v_pages, table, first_key(at), bound, page_heads, page_head, bs, col, grp);
 
   if constexpr (FRESH != 0) {
     // the queries of this lane's head: norm over the head (its D values lie in four lanes), rotation
@@ -574,14 +584,14 @@ __global__ __launch_bounds__(256) void attn_decode_mfma_kernel(
   for (int dt = 0; dt < DT; ++dt) o[dt] = f32x4_t{0.f, 0.f, 0.f, 0.f};
   float m = NEG_INF, l = 0.f;
 
-  for (int step = s0 + wave; step < s1; step += 4) {
-    const int kb = first_key(step);
-    const bool more = step + 4 < s1;
-    if (more) load_kv_step<DC>(nxt, k_pages, v_pages, table, first_key(step + 4), ctx, page_heads, page_head, bs, col, grp);
+  for (; at < to; at += 4 * NEXT) {
+    const int kb = first_key(at);
+    const bool more = at + 4 * NEXT < to;
+    if (more) load_kv_step<DC>(nxt, k_pages, v_pages, table, first_key(at + 4 * NEXT), bound, page_heads, page_head, bs, col, grp);
     if constexpr (FRESH != 0) {
       if (fresh_here && pos >= kb && pos < kb + 32) {  // this wave's step holds the token itself: take it from LDS
-        const int at = pos - kb;  // = KEY_OF_ROW(tile, row) for
-        const int tile = (at >> 2) & 1, row = 4 * (at >> 3) + (at & 3);
+        const int nth = pos - kb;  // = KEY_OF_ROW(tile, row) for
+        const int tile = (nth >> 2) & 1, row = 4 * (nth >> 3) + (nth & 3);
         if (col == row) {
 #pragma unroll
           for (int tt = 0; tt < 2; ++tt)
@@ -590,12 +600,12 @@ __global__ __launch_bounds__(256) void attn_decode_mfma_kernel(
               for (int c = 0; c < DC; ++c) cur.k[tt][c] = *reinterpret_cast<const bf16x8_t*>(&fresh_kv[0][c * 32 + grp * 8]);
             }
         }
-        if (grp == (at >> 3)) {
+        if (grp == (nth >> 3)) {
 #pragma unroll
           for (int dt = 0; dt < DT; ++dt)
 #pragma unroll
             for (int j = 0; j < 8; ++j)
-              if (j == (at & 7)) cur.v[dt][j] = fresh_kv[1][dt * 16 + col];
+              if (j == (nth & 7)) cur.v[dt][j] = fresh_kv[1][dt * 16 + col];
         }
       }
     }
@@ -614,9 +624,9 @@ __global__ __launch_bounds__(256) void attn_decode_mfma_kernel(
 #pragma unroll
       for (int r = 0; r < 4; ++r) {
         const int key = kb + KEY_OF_ROW(tt, 4 * grp + r);
-        const bool seen = key < ctx && (key >= lo || key < kept);
+        const bool seen = key < bound && (key >= lo || key < kept);
         float sc = s[tt][r] * scale;
-        if (CAP) sc = sight.cap * quick_tanh(sc / sight.cap);
+        if (SEE == 2) sc = sight.cap * quick_tanh(sc / sight.cap);
         s[tt][r] = seen ? sc : NEG_INF;
         mx = fmaxf(mx, s[tt][r]);
       }
@@ -676,12 +686,12 @@ __global__ __launch_bounds__(256) void attn_decode_mfma_kernel(
     }
     const int h = h0 + g;
     if (P == 1) {
-      if (sight.sink) {
+      if (SEE >= 1 && sight.sink) {
         const float top = fmaxf(mxw, 0.f), e = __expf(mxw - top);
         num *= e;
         den = den * e + __expf(-top);
       }
-      put(out, ((size_t)t * H + h) * D + d, num / den, sight.wide);
+      put(out, ((size_t)t * H + h) * D + d, num / den, SEE >= 1 ? sight.wide : 0);
     } else {
       const size_t ob = ((size_t)item * H + h) * P + part;
       part_acc[ob * D + d] = num;
@@ -742,7 +752,7 @@ constexpr int PREFILL_MIN_PIECE_ROUNDS = 2;  // an item's last two rounds hold i
 
 // With kept first tokens behind a window the rounds of 64 keys are first those from the sequence's start that hold kept
 // tokens, then those of the window (`first_key`); pieces cut this list.
-template <int DC, int QT, bool CAP>  // D / 32; column tiles of 16 queries that a wave owns: 2, or 1 (see the launcher)
+template <int DC, int QT, int SEE>  // D / 32; column tiles of 16 queries that a wave owns: 2, or 1 (see the launcher); SEE: see above
 __global__ __launch_bounds__(256, 2) void attn_prefill_mfma_kernel(
     const bf16* __restrict__ q, const bf16* __restrict__ k_pages, const bf16* __restrict__ v_pages,
     const int* __restrict__ tiles, const int* __restrict__ block_tables, int table_width,
@@ -795,7 +805,7 @@ __global__ __launch_bounds__(256, 2) void attn_prefill_mfma_kernel(
     if (split.pieces > 1 && piece == 0 && threadIdx.x == 0) split.cut[item] = 1;
     return;
   }
-  const int kept = min(sight.keep, wg_lo);  // kept tokens that lie before every query's window
+  const int keep = SEE >= 1 ? sight.keep : 0, kept = min(keep, wg_lo);  // kept tokens that lie before every query's window
   int kept_rounds = (kept + 63) / 64, kb0 = (wg_lo / 32) * 32;
   if (kept_rounds > 0 && 64 * kept_rounds >= kb0) kept_rounds = kb0 = 0;  // one run from the start
   int rd_first = 0, rd_end = kept_rounds + ((wg_last - kb0) / 32 + 2) / 2;
@@ -821,7 +831,7 @@ __global__ __launch_bounds__(256, 2) void attn_prefill_mfma_kernel(
   const int nq = working ? min(WQ, count - q0) : 1;
   const int my_last = working ? pos0 + q0 + nq - 1 : -1;
   const int my_first_q = pos0 + q0;                  // position of this wave's first query
-  const float scale2 = CAP ? 1.f : scale * 1.4426950408889634f;  // scores are kept in base 2
+  const float scale2 = SEE == 2 ? 1.f : scale * 1.4426950408889634f;  // scores are kept in base 2
   const int my_lo = working ? (window > 0 ? max(0, pos0 + q0 - window + 1) : 0) : 0x7fffffff;
 
   bf16x8_t qop[QT][DC];
@@ -863,7 +873,9 @@ __global__ __launch_bounds__(256, 2) void attn_prefill_mfma_kernel(
   // shared by all waves of the compute unit.  A piece that would start beyond the last key
   // repeats the last one (finite numbers; its scores are masked).
   unsigned long long k_at = 0, v_at = 0;  // byte offsets of this lane's piece in k_pages and v_pages
-  auto key_of = [&](int piece) { return min(first_key(rd_first + (piece >> 2)) + 16 * (piece & 3), last_piece); };
+  auto key_of = [&](int piece) {
+    return min(SEE >= 1 ? first_key(rd_first + (piece >> 2)) + 16 * (piece & 3) : first_key(rd_first) + 16 * piece, last_piece);
+  };
   auto entry_of = [&](int piece) { return key_of(piece) / bs; };
   int page_ahead = table[entry_of(lane)];
   auto locate = [&](int batch) {  // pieces 64 batch .. 64 batch + 63
@@ -943,7 +955,7 @@ __global__ __launch_bounds__(256, 2) void attn_prefill_mfma_kernel(
     __syncthreads();  // ... and everyone's; and everyone is done with the round before
     const bool more = rd + 1 < nrounds;  // copies into the two stages the round before used
     const int kb = first_key(rd_first + rd);
-    const bool active = working && kb <= my_last && (kb + 63 >= my_lo || kb < sight.keep);
+    const bool active = working && kb <= my_last && (kb + 63 >= my_lo || kb < keep);
     if (more) {
       aim(2 * rd + 2);
       if (!active) {
@@ -990,7 +1002,7 @@ __global__ __launch_bounds__(256, 2) void attn_prefill_mfma_kernel(
       bf16x8_t pop[QT][2];
       float alpha[QT];
       bool rescale = false;
-      if (CAP) {  // the capped scores, in base 2 already
+      if (SEE == 2) {  // the capped scores, in base 2 already
         const float inner = scale / sight.cap, outer = sight.cap * 1.4426950408889634f;
 #pragma unroll
         for (int qt = 0; qt < QT; ++qt)
@@ -1007,7 +1019,7 @@ __global__ __launch_bounds__(256, 2) void attn_prefill_mfma_kernel(
 #pragma unroll
             for (int r = 0; r < 4; ++r) {
               const int key = kb + 32 * (tt >> 1) + KEY_OF_ROW(tt & 1, 4 * grp + r);
-              const bool seen = key <= qpos[qt] && (window <= 0 || key > qpos[qt] - window || key < sight.keep);
+              const bool seen = key <= qpos[qt] && (window <= 0 || key > qpos[qt] - window || key < keep);
               sc[qt][tt][r] = seen ? sc[qt][tt][r] : NEG_INF;
             }
         }
@@ -1083,12 +1095,12 @@ __global__ __launch_bounds__(256, 2) void attn_prefill_mfma_kernel(
   for (int qt = 0; qt < QT; ++qt) {
     if (!qok[qt]) continue;
     float inv = 1.0f / l[qt];
-    if (sight.sink) {
+    if (SEE >= 1 && sight.sink) {
       const float top = fmaxf(m[qt], 0.f), e = __builtin_amdgcn_exp2f(m[qt] - top);
       inv = e / (l[qt] * e + __builtin_amdgcn_exp2f(-top));
     }
     const size_t at = ((size_t)(tok0 + q0 + qt * 16 + col) * H + head) * D + 4 * grp;
-    if (sight.wide) {
+    if (SEE >= 1 && sight.wide) {
       float* orow = reinterpret_cast<float*>(out) + at;
 #pragma unroll
       for (int dt = 0; dt < DT; ++dt) *reinterpret_cast<f32x4_t*>(orow + dt * 16) = o[qt][dt] * inv;
@@ -1188,13 +1200,15 @@ extern "C" int as_attn_prefill_mfma(const void* q, const void* k_pages, const vo
   if (blocks > 0x7fffffffL) return AS_BAD_SHAPE;
   const int pass = compute_units();
   const PrefillSplit split{pieces, piece_rounds, cut, part_ml, part_acc};
-#define LAUNCH2(DCV, QTV, CAPV)                                                                       \
-  attn_prefill_mfma_kernel<DCV, QTV, CAPV><<<(int)blocks, 256, 0, stream>>>(                          \
+  const int see = needed_sight(sight);
+#define LAUNCH2(DCV, QTV, SEEV)                                                                       \
+  attn_prefill_mfma_kernel<DCV, QTV, SEEV><<<(int)blocks, 256, 0, stream>>>(                          \
       (const bf16*)q, (const bf16*)k_pages, (const bf16*)v_pages, tiles, block_tables, table_width,   \
       (bf16*)out, H, KV, bs, scale, sight, units_z, pass, split)
 #define LAUNCH1(DCV, QTV)                                                                             \
-  if (cap > 0.f) LAUNCH2(DCV, QTV, true);                                                             \
-  else LAUNCH2(DCV, QTV, false);                                                                      \
+  if (see == 2) LAUNCH2(DCV, QTV, 2);                                                                 \
+  else if (see == 1) LAUNCH2(DCV, QTV, 1);                                                            \
+  else LAUNCH2(DCV, QTV, 0);                                                                          \
   if (pieces > 1)                                                                                     \
     attn_prefill_merge_kernel<DCV, QTV><<<(int)items, 256, 0, stream>>>(tiles, (bf16*)out, H, KV, units_z, split, sink, wide);
 #define LAUNCH(DCV)              \
@@ -1224,7 +1238,7 @@ static int launch_decode_mfma(const void* q, const void* k_pages, const void* v_
                               int table_width, void* out, float* part_m, float* part_l, float* part_acc, int H,
                               int KV, int D, int bs, float scale, const Sight& sight, int part_size, int P,
                               const FreshQKV* fresh, int gains_dtype, hipStream_t stream, int share = 1) {
-  if (!sight_ok(sight) || (fresh && sight.cap > 0.f)) return AS_BAD_SHAPE;
+  if (!sight_ok(sight) || (fresh && needed_sight(sight) > 0)) return AS_BAD_SHAPE;
   const int G = H / KV;
   if (D % 32 || D > 256 || G > 16 || bs % 16 || part_size % 32) return AS_BAD_SHAPE;
   if (fresh && D % 64) return AS_BAD_SHAPE;
@@ -1233,15 +1247,17 @@ static int launch_decode_mfma(const void* q, const void* k_pages, const void* v_
   const size_t shmem = sizeof(float) * (size_t)(128 + 4 * D * G);
   if (shmem + 1024 > (64u << 10)) return AS_BAD_SHAPE;  // wide heads in large groups: the general kernel's
   const FreshQKV none = {};
-#define LAUNCH3(DCV, FRESHV, CAPV)                                                                        \
-  attn_decode_mfma_kernel<DCV, FRESHV, CAPV><<<grid, 256, shmem, stream>>>(                               \
+  const int see = needed_sight(sight);
+#define LAUNCH3(DCV, FRESHV, SEEV)                                                                        \
+  attn_decode_mfma_kernel<DCV, FRESHV, SEEV><<<grid, 256, shmem, stream>>>(                               \
       (const bf16*)q, (const bf16*)k_pages, (const bf16*)v_pages, items, positions, tok_row, block_tables, \
       table_width, (bf16*)out, part_m, part_l, part_acc, H, KV, bs, scale, sight, part_size, P,           \
       compute_units(), share, FRESHV ? *fresh : none)
-#define LAUNCH(DCV, FRESHV) LAUNCH3(DCV, FRESHV, false)
+#define LAUNCH(DCV, FRESHV) LAUNCH3(DCV, FRESHV, 0)
 #define LAUNCH_PLAIN(DCV)                          \
-  if (sight.cap > 0.f) LAUNCH3(DCV, 0, true);      \
-  else LAUNCH3(DCV, 0, false)
+  if (see == 2) LAUNCH3(DCV, 0, 2);                \
+  else if (see == 1) LAUNCH3(DCV, 0, 1);           \
+  else LAUNCH3(DCV, 0, 0)
 #define LAUNCH_FRESH(FRESHV)            \
   switch (D / 64) {                     \
     case 1: LAUNCH(2, FRESHV); break;   \
