@@ -1199,3 +1199,169 @@ class TeberaxConfig:
         if self.logit_softcap:
             raw["logit_softcap"] = self.logit_softcap
         return raw
+
+
+# ---- Tokuvik ------------------------------------------------------------------------------------------
+
+
+def _sizes_from(cls, raw: dict, where: str, names, **more):
+    return cls(*(int(_need(raw, k, where)) for k in names), **more)
+
+
+@dataclass(frozen=True)
+class TokuvikAttention:
+    """A grouped-query attention over chunks ("attention").  chunk 0: every earlier key is seen.  kv_from >= 0: the layer has
+    no keys and values of its own and reads that layer's."""
+
+    heads: int
+    kv_heads: int
+    dim: int
+    vdim: int
+    scale: float
+    chunk: int = 0
+    kv_from: int = -1
+
+    @classmethod
+    def from_dict(cls, raw: dict, where: str) -> "TokuvikAttention":
+        return _sizes_from(cls, raw, where, ("heads", "kv_heads", "dim", "vdim"), scale=float(_need(raw, "scale", where)),
+                           chunk=int((raw.get("mask") or {}).get("size") or 0),
+                           kv_from=int(raw["kv_from"]) if raw.get("kv_from") is not None else -1)  # fmt: skip
+
+    def to_dict(self) -> dict:
+        raw = {"heads": self.heads, "kv_heads": self.kv_heads, "dim": self.dim, "vdim": self.vdim, "scale": self.scale}
+        if self.chunk:
+            raw["mask"] = {"size": self.chunk}
+        if self.kv_from >= 0:
+            raw["kv_from"] = self.kv_from
+        return raw
+
+
+@dataclass(frozen=True)
+class TokuvikLatent:
+    """An attention through a cached latent with a sink per head ("latent_attention")."""
+
+    heads: int
+    dim: int
+    vdim: int
+    q_rank: int
+    kv_rank: int
+    scale: float
+
+    @classmethod
+    def from_dict(cls, raw: dict, where: str) -> "TokuvikLatent":
+        return _sizes_from(cls, raw, where, ("heads", "dim", "vdim", "q_rank", "kv_rank"), scale=float(_need(raw, "scale", where)))
+
+    def to_dict(self) -> dict:
+        return {"heads": self.heads, "dim": self.dim, "vdim": self.vdim, "q_rank": self.q_rank, "kv_rank": self.kv_rank,
+                "scale": self.scale}  # fmt: skip
+
+
+@dataclass(frozen=True)
+class TokuvikStateSpace:
+    """A state space per head ("mamba2"): heads of `vdim` columns over `state` rows, `groups` of B and C."""
+
+    heads: int
+    vdim: int
+    state: int
+    groups: int
+    conv: int
+    norm_groups: int
+
+    @classmethod
+    def from_dict(cls, raw: dict, where: str) -> "TokuvikStateSpace":
+        return _sizes_from(cls, raw, where, ("heads", "vdim", "state", "groups", "conv", "norm_groups"))
+
+    def to_dict(self) -> dict:
+        return {"heads": self.heads, "vdim": self.vdim, "state": self.state, "groups": self.groups, "conv": self.conv,
+                "norm_groups": self.norm_groups}  # fmt: skip
+
+
+@dataclass(frozen=True)
+class TokuvikLayer:
+    type: str  # "attention", "latent_attention" or "mamba2"
+    mixer: object
+    ff: int  # width inside the gated feed-forward; 0: the layer has none
+
+
+@dataclass(frozen=True)
+class TokuvikConfig:
+    """A Tokuvik decoder: layers with a layer norm (a gain, no bias) before and after each sublayer and an input of the tokens'
+    own at the end; mixers of three kinds (a gated attention over chunks that may read an earlier layer's keys and values, an
+    attention through a latent with a sink per head, a state space per head); gated feed-forwards or none; the embedding
+    table is also the head."""
+
+    vocab_size: int
+    hidden_size: int
+    norm_eps: float
+    layers: tuple  # of TokuvikLayer
+    side_dim: int = 0  # a layer's share of the token's row of the second table; 0: layers have no such input
+
+    architecture = "Tokuvik"
+    MIXERS = {"attention": TokuvikAttention, "latent_attention": TokuvikLatent, "mamba2": TokuvikStateSpace}
+
+    @classmethod
+    def from_dict(cls, raw: dict) -> "TokuvikConfig":
+        _require(raw, ["vocab", "width", "layers", "norm"])
+        layers = []
+        for i, entry in enumerate(raw["layers"]):
+            where = f"layers[{i}]."
+            kind = _need(entry, "type", where)
+            if kind not in cls.MIXERS:
+                raise ConfigError(f"{where}type={kind!r} is not supported (one of {', '.join(cls.MIXERS)})")
+            mixer = cls.MIXERS[kind].from_dict(_need(entry, "mixer", where), where + "mixer.")
+            mlp, ff = entry.get("mlp"), 0
+            if mlp is not None:
+                if _need(mlp, "kind", where + "mlp.") != "dense":
+                    raise ConfigError(f"{where}mlp.kind={mlp['kind']!r} is not supported ('dense')")
+                ff = int(_need(mlp, "ff", where + "mlp."))
+                if ff < 1:
+                    raise ConfigError(f"{where}mlp.ff must be positive")
+            layers.append(TokuvikLayer(kind, mixer, ff))
+        side = raw.get("token_side")
+        cfg = cls(
+            vocab_size=int(raw["vocab"]),
+            hidden_size=int(raw["width"]),
+            norm_eps=float(_need(raw["norm"], "eps", "norm.")),
+            layers=tuple(layers),
+            side_dim=int(_need(side, "dim", "token_side.")) if side else 0,
+        )
+        cfg.validate()
+        return cfg
+
+    def validate(self) -> None:
+        if self.vocab_size < 1 or self.hidden_size < 1 or not self.layers:
+            raise ConfigError("vocab, width and the number of layers must be positive")
+        if not self.norm_eps > 0:
+            raise ConfigError("norm.eps must be positive")
+        if self.side_dim < 0:
+            raise ConfigError("token_side.dim is not negative")
+        for i, layer in enumerate(self.layers):
+            m, at = layer.mixer, f"layers[{i}]"
+            if layer.type == "mamba2":
+                if min(m.heads, m.vdim, m.state, m.groups, m.conv, m.norm_groups) < 1 or m.heads % m.groups:
+                    raise ConfigError(f"{at}: sizes must be positive, heads a multiple of groups")
+                if (m.heads * m.vdim) % m.norm_groups:
+                    raise ConfigError(f"{at}: norm_groups {m.norm_groups} does not divide heads x vdim")
+            elif layer.type == "latent_attention":
+                if min(m.heads, m.dim, m.vdim, m.q_rank, m.kv_rank) < 1:
+                    raise ConfigError(f"{at}: sizes must be positive")
+            else:
+                if min(m.heads, m.kv_heads, m.dim, m.vdim) < 1 or m.heads % m.kv_heads or m.chunk < 0:
+                    raise ConfigError(f"{at}: sizes must be positive, heads a multiple of kv_heads, mask.size not negative")
+                if m.kv_from >= 0:
+                    src = self.layers[m.kv_from] if m.kv_from < i else None
+                    if src is None or src.type != "attention" or src.mixer.kv_from >= 0:
+                        raise ConfigError(f"{at}: kv_from names an earlier attention layer with keys and values of its own")
+                    s = src.mixer
+                    if (s.kv_heads, s.dim, s.vdim) != (m.kv_heads, m.dim, m.vdim):
+                        raise ConfigError(f"{at}: kv_heads, dim and vdim must equal those of layer {m.kv_from}, whose keys it reads (kv_from)")
+
+    def to_dict(self) -> dict:
+        """The config.json that `from_dict` reads back to this object."""
+        layers = [{"type": layer.type, "mixer": layer.mixer.to_dict(), "mlp": {"kind": "dense", "ff": layer.ff} if layer.ff else None}
+                  for layer in self.layers]  # fmt: skip
+        raw = {"architecture": self.architecture, "vocab": self.vocab_size, "width": self.hidden_size,
+               "norm": {"eps": self.norm_eps}, "layers": layers}  # fmt: skip
+        if self.side_dim:
+            raw["token_side"] = {"dim": self.side_dim}
+        return raw

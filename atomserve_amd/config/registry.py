@@ -92,3 +92,4 @@ def _load_builtin() -> None:
     import atomserve_amd.models.natatar  # noqa: F401
     import atomserve_amd.models.qwen3  # noqa: F401
     import atomserve_amd.models.teberax  # noqa: F401
+    import atomserve_amd.models.tokuvik  # noqa: F401

@@ -3,7 +3,8 @@
 // Cache pages of one layer: k_pages [num_pages, KV, block_size, D] and v_pages
 // [num_pages, KV, D, block_size] (values transposed within a page); a token at position p
 // of a request lives in page table[p / block_size] at offset p % block_size.  A query at position p sees the keys at positions lo..p, with
-// lo = max(0, p - window + 1) if window > 0, else 0, and beside a window the first `keep` of the sequence (`Sight`).
+// lo = max(0, p - window + 1) if window > 0, the start of p's chunk if the sequence is cut into chunks, else 0, and beside a
+// window the first `keep` of the sequence (`Sight`).
 // Query head h reads kv head h / (H / KV).  Scores, softmax and the weighted sum are fp32.
 //
 // attn_single_query: one work item per query token.  A workgroup (4 waves) takes one
@@ -28,8 +29,10 @@ template <> __device__ __forceinline__ float fexp<bf16>(float x) { return __expf
 struct Sight {
   int window;  // > 0: keys p - window + 1 .. p; 0: every key up to p
   int keep;    // with a window: the sequence's first `keep` keys stay visible behind it
+  int chunk;   // > 0: keys of the query's own chunk only, chunks of this many positions counted from 0 (without a window)
   float cap;   // > 0: a score s counts as cap tanh(s / cap)
-  int sink;    // 1: the denominator has one more score, of 0, which has no value
+  int sink;    // 1: the denominator has one more score, which has no value
+  const float* sinks;  // [H]: that score per query head (not scaled); null: 0 for all
   int wide;    // 1: the kernels of bfloat16 heads write their results in fp32 (for a consumer that takes differences of them)
 };
 // The result of a head's coordinate i, in the type of the heads or in fp32 (`Sight::wide`).
@@ -39,14 +42,16 @@ __device__ __forceinline__ void put(T* out, size_t i, float v, int wide) {
   else out[i] = from_f32<T>(v);
 }
 __device__ __forceinline__ int first_in_window(const Sight& sight, int ctx) {
+  if (sight.chunk > 0) return (ctx - 1) / sight.chunk * sight.chunk;
   return sight.window > 0 ? max(0, ctx - sight.window) : 0;
 }
+__device__ __forceinline__ float sink_score(int sink, const float* sinks, int head) { return sink && sinks ? sinks[head] : 0.f; }
 static inline bool sight_ok(const Sight& s) {
   return s.window >= 0 && s.keep >= 0 && (s.keep == 0 || s.window > 0) && s.cap >= 0.f && (s.sink == 0 || s.sink == 1) &&
-         (s.wide == 0 || s.wide == 1);
+         (s.wide == 0 || s.wide == 1) && s.chunk >= 0 && (s.chunk == 0 || s.window == 0);
 }
 // Which instance of the matrix-core kernels computes it (`SEE` below).
-static inline int needed_sight(const Sight& s) { return s.cap > 0.f ? 2 : (s.keep > 0 || s.sink || s.wide) ? 1 : 0; }
+static inline int needed_sight(const Sight& s) { return s.cap > 0.f ? 2 : (s.keep > 0 || s.sink || s.wide || s.chunk > 0) ? 1 : 0; }
 
 // tanh through the hardware's exponential and reciprocal: an absolute error of 1e-7, which is what a capped score
 // (times the cap) of the bf16 kernels may carry.
@@ -225,9 +230,9 @@ __global__ __launch_bounds__(256) void attn_single_query_kernel(
     const int h = h0 + g;
     if (P == 1) {
       if (sight.sink) {
-        const float top = fmaxf(mx, 0.f), e = fexp<T>(mx - top);
+        const float sk = sink_score(1, sight.sinks, h), top = fmaxf(mx, sk), e = fexp<T>(mx - top);
         num *= e;
-        den = den * e + fexp<T>(-top);
+        den = den * e + fexp<T>(sk - top);
       }
       put(out, ((size_t)t * H + h) * D + d, num / den, sight.wide);
     } else {
@@ -248,13 +253,14 @@ __global__ __launch_bounds__(256) void attn_reduce_kernel(const int* __restrict_
                                                           const float* __restrict__ part_m,
                                                           const float* __restrict__ part_l,
                                                           const float* __restrict__ part_acc, T* __restrict__ out,
-                                                          int H, int D, int P, int sink, int wide) {
+                                                          int H, int D, int P, int sink, const float* __restrict__ sinks, int wide) {
   const int item = blockIdx.x, h = blockIdx.y;
   const size_t base = ((size_t)item * H + h) * P;
   float mx = NEG_INF;
   for (int p = 0; p < P; ++p) mx = fmaxf(mx, part_m[base + p]);
-  if (sink) mx = fmaxf(mx, 0.f);
-  float den = sink ? fexp<T>(-mx) : 0.f;
+  const float sk = sink_score(sink, sinks, h);
+  if (sink) mx = fmaxf(mx, sk);
+  float den = sink ? fexp<T>(sk - mx) : 0.f;
   for (int p = 0; p < P; ++p) {
     const float mp = part_m[base + p];
     den += (mp == NEG_INF) ? 0.f : part_l[base + p] * fexp<T>(mp - mx);
@@ -399,7 +405,7 @@ __device__ __forceinline__ void load_gains8(const bf16* w, float* g) {
 }
 
 // D / 32; FRESH 0: finished queries, 1: qkv with bf16 gains, 2: with fp32 gains; SEE 0: a window at most (nothing of the rest of
-// `sight` is read), 1: kept first tokens, a sink and fp32 outputs too, 2: also capped scores
+// `sight` is read), 1: kept first tokens, chunks, a sink and fp32 outputs too, 2: also capped scores
 template <int DC, int FRESH, int SEE>
 __global__ __launch_bounds__(256) void attn_decode_mfma_kernel(
     const bf16* __restrict__ q, const bf16* __restrict__ k_pages, const bf16* __restrict__ v_pages,
@@ -687,9 +693,9 @@ __global__ __launch_bounds__(256) void attn_decode_mfma_kernel(
     const int h = h0 + g;
     if (P == 1) {
       if (SEE >= 1 && sight.sink) {
-        const float top = fmaxf(mxw, 0.f), e = __expf(mxw - top);
+        const float sk = sink_score(1, sight.sinks, h), top = fmaxf(mxw, sk), e = __expf(mxw - top);
         num *= e;
-        den = den * e + __expf(-top);
+        den = den * e + __expf(sk - top);
       }
       put(out, ((size_t)t * H + h) * D + d, num / den, SEE >= 1 ? sight.wide : 0);
     } else {
@@ -791,6 +797,9 @@ __global__ __launch_bounds__(256, 2) void attn_prefill_mfma_kernel(
   const int pos0 = tiles[4 * tile + 3];
   const int* table = block_tables + (size_t)row * table_width;
   const int window = sight.window;
+  auto first_seen = [&](int pos) {  // the oldest key that a query at `pos` sees, kept first ones apart
+    return SEE >= 1 ? first_in_window(sight, pos + 1) : window > 0 ? max(0, pos - window + 1) : 0;
+  };
 
   // the keys this workgroup walks: from the first key any of its waves sees to the last
   int wg_lo = 0x7fffffff, wg_last = -1;
@@ -799,7 +808,7 @@ __global__ __launch_bounds__(256, 2) void attn_prefill_mfma_kernel(
     const int uq0 = (u / G) * WQ;
     if (uq0 >= count) continue;
     wg_last = max(wg_last, pos0 + min(count, uq0 + WQ) - 1);
-    wg_lo = min(wg_lo, window > 0 ? max(0, pos0 + uq0 - window + 1) : 0);
+    wg_lo = min(wg_lo, first_seen(pos0 + uq0));
   }
   if (wg_last < 0) {  // uniform over the workgroup
     if (split.pieces > 1 && piece == 0 && threadIdx.x == 0) split.cut[item] = 1;
@@ -832,10 +841,12 @@ __global__ __launch_bounds__(256, 2) void attn_prefill_mfma_kernel(
   const int my_last = working ? pos0 + q0 + nq - 1 : -1;
   const int my_first_q = pos0 + q0;                  // position of this wave's first query
   const float scale2 = SEE == 2 ? 1.f : scale * 1.4426950408889634f;  // scores are kept in base 2
-  const int my_lo = working ? (window > 0 ? max(0, pos0 + q0 - window + 1) : 0) : 0x7fffffff;
+  const int my_lo = working ? first_seen(pos0 + q0) : 0x7fffffff;
+  [[maybe_unused]] const int last_lo = first_seen(my_last);  // of this wave's last query
 
   bf16x8_t qop[QT][DC];
   int qpos[QT];
+  [[maybe_unused]] int qlo[QT];
   bool qok[QT];
 #pragma unroll
   for (int qt = 0; qt < QT; ++qt) {
@@ -843,6 +854,7 @@ __global__ __launch_bounds__(256, 2) void attn_prefill_mfma_kernel(
     qok[qt] = working && qi < nq;
     const int qc = min(qi, nq - 1);  // columns past the end repeat the last query and are not stored
     qpos[qt] = pos0 + q0 + qc;
+    if (SEE >= 1) qlo[qt] = first_seen(qpos[qt]);
     if (working) {
       const bf16* qrow = q + ((size_t)(tok0 + q0 + qc) * H + head) * D + grp * 8;
 #pragma unroll
@@ -998,7 +1010,7 @@ __global__ __launch_bounds__(256, 2) void attn_prefill_mfma_kernel(
       }
       // Only rounds that touch the causal diagonal, the window's edge or the end of the context
       // need a mask; the others see all 64 keys (uniform over the wave).
-      const bool masked = kb + 63 > my_first_q || (window > 0 && kb < my_last - window + 1);
+      const bool masked = kb + 63 > my_first_q || (SEE >= 1 ? kb < last_lo : window > 0 && kb < my_last - window + 1);
       bf16x8_t pop[QT][2];
       float alpha[QT];
       bool rescale = false;
@@ -1019,7 +1031,7 @@ __global__ __launch_bounds__(256, 2) void attn_prefill_mfma_kernel(
 #pragma unroll
             for (int r = 0; r < 4; ++r) {
               const int key = kb + 32 * (tt >> 1) + KEY_OF_ROW(tt & 1, 4 * grp + r);
-              const bool seen = key <= qpos[qt] && (window <= 0 || key > qpos[qt] - window || key < keep);
+              const bool seen = key <= qpos[qt] && (SEE >= 1 ? key >= qlo[qt] || key < keep : window <= 0 || key > qpos[qt] - window);
               sc[qt][tt][r] = seen ? sc[qt][tt][r] : NEG_INF;
             }
         }
@@ -1096,8 +1108,9 @@ __global__ __launch_bounds__(256, 2) void attn_prefill_mfma_kernel(
     if (!qok[qt]) continue;
     float inv = 1.0f / l[qt];
     if (SEE >= 1 && sight.sink) {
-      const float top = fmaxf(m[qt], 0.f), e = __builtin_amdgcn_exp2f(m[qt] - top);
-      inv = e / (l[qt] * e + __builtin_amdgcn_exp2f(-top));
+      const float sk = sink_score(1, sight.sinks, head) * 1.4426950408889634f, top = fmaxf(m[qt], sk);
+      const float e = __builtin_amdgcn_exp2f(m[qt] - top);
+      inv = e / (l[qt] * e + __builtin_amdgcn_exp2f(sk - top));
     }
     const size_t at = ((size_t)(tok0 + q0 + qt * 16 + col) * H + head) * D + 4 * grp;
     if (SEE >= 1 && sight.wide) {
@@ -1121,7 +1134,8 @@ __global__ __launch_bounds__(256, 2) void attn_prefill_mfma_kernel(
 // largest maximum; a piece that saw no key has m = -inf and l = 0.
 template <int DC, int QT>
 __global__ __launch_bounds__(256) void attn_prefill_merge_kernel(const int* __restrict__ tiles, bf16* __restrict__ out,
-                                                                  int H, int KV, int units_z, PrefillSplit split, int sink, int wide) {
+                                                                  int H, int KV, int units_z, PrefillSplit split, int sink,
+                                                                  const float* __restrict__ sinks, int wide) {
   constexpr int D = DC * 32, DT = DC * 2, WQ = 16 * QT, PARTS = 64 / WQ;
   const int item = blockIdx.x;
   const int n = split.cut[item];
@@ -1140,11 +1154,12 @@ __global__ __launch_bounds__(256) void attn_prefill_merge_kernel(const int* __re
     const float2* ml = reinterpret_cast<const float2*>(split.ml) + at;  // (m, l) of the pieces
     float m = NEG_INF;
     for (int j = 0; j < n; ++j) m = fmaxf(m, ml[j].x);
-    if (sink) m = fmaxf(m, 0.f);
+    const float sk = sink_score(sink, sinks, head) * 1.4426950408889634f;
+    if (sink) m = fmaxf(m, sk);
     f32x4_t sum[DT];
 #pragma unroll
     for (int dt = 0; dt < DT; ++dt) sum[dt] = f32x4_t{0.f, 0.f, 0.f, 0.f};
-    float den = sink ? __builtin_amdgcn_exp2f(-m) : 0.f;
+    float den = sink ? __builtin_amdgcn_exp2f(sk - m) : 0.f;
     for (int j = 0; j < n; ++j) {
       const float2 p = ml[j];
       const float w = p.x == NEG_INF ? 0.f : __builtin_amdgcn_exp2f(p.x - m);
@@ -1182,11 +1197,11 @@ __global__ __launch_bounds__(256) void attn_prefill_merge_kernel(const int* __re
 // piece_rounds * pieces covers the longest item.  pieces <= 1: none is cut, the three may be null.
 extern "C" int as_attn_prefill_mfma(const void* q, const void* k_pages, const void* v_pages, const int* tiles,
                                     int num_tiles, const int* block_tables, int table_width, void* out, int H,
-                                    int KV, int D, int bs, float scale, int window, int keep, float cap, int sink,
+                                    int KV, int D, int bs, float scale, int window, int keep, int chunk, float cap, int sink, const float* sinks,
                                     int wide, int query_tiles, int pieces, int piece_rounds, int* cut, float* part_ml,
                                     float* part_acc, hipStream_t stream) {
   if (num_tiles <= 0) return AS_OK;
-  const Sight sight{window, keep, cap, sink, wide};
+  const Sight sight{window, keep, chunk, cap, sink, sinks, wide};
   if (!sight_ok(sight)) return AS_BAD_SHAPE;
   if (H <= 0 || KV <= 0 || H % KV || bs <= 0 || table_width <= 0) return AS_BAD_SHAPE;
   const int G = H / KV;
@@ -1210,7 +1225,7 @@ extern "C" int as_attn_prefill_mfma(const void* q, const void* k_pages, const vo
   else if (see == 1) LAUNCH2(DCV, QTV, 1);                                                            \
   else LAUNCH2(DCV, QTV, 0);                                                                          \
   if (pieces > 1)                                                                                     \
-    attn_prefill_merge_kernel<DCV, QTV><<<(int)items, 256, 0, stream>>>(tiles, (bf16*)out, H, KV, units_z, split, sink, wide);
+    attn_prefill_merge_kernel<DCV, QTV><<<(int)items, 256, 0, stream>>>(tiles, (bf16*)out, H, KV, units_z, split, sink, sinks, wide);
 #define LAUNCH(DCV)              \
   if (query_tiles == 1) {        \
     LAUNCH1(DCV, 1)              \
@@ -1288,7 +1303,7 @@ static int launch_decode_mfma(const void* q, const void* k_pages, const void* v_
   if (hipGetLastError() != hipSuccess) return AS_LAUNCH_FAILED;
   if (P > 1) {
     attn_reduce_kernel<bf16><<<dim3(num_items, H), D <= 64 ? 64 : (D <= 128 ? 128 : 256), 0, stream>>>(
-        items, part_m, part_l, part_acc, (bf16*)out, H, D, P, sight.sink, sight.wide);
+        items, part_m, part_l, part_acc, (bf16*)out, H, D, P, sight.sink, sight.sinks, sight.wide);
   }
   return launch_status();
 }
@@ -1298,14 +1313,14 @@ extern "C" int as_attn_decode_mfma(const void* q, const void* k_pages, const voi
                                    int num_items, const int* positions, const int* tok_row,
                                    const int* block_tables, int table_width, void* out, float* part_m,
                                    float* part_l, float* part_acc, int H, int KV, int D, int bs, float scale,
-                                   int window, int keep, float cap, int sink, int wide, int part_size, int P,
+                                   int window, int keep, int chunk, float cap, int sink, const float* sinks, int wide, int part_size, int P,
                                    hipStream_t stream) {
   if (num_items <= 0) return AS_OK;
   if (H <= 0 || KV <= 0 || H % KV || D <= 0 || bs <= 0 || part_size <= 0 || P <= 0 || table_width <= 0)
     return AS_BAD_SHAPE;
   if (P > 1 && (!part_m || !part_l || !part_acc)) return AS_BAD_SHAPE;
   return launch_decode_mfma(q, k_pages, v_pages, items, num_items, positions, tok_row, block_tables, table_width,
-                            out, part_m, part_l, part_acc, H, KV, D, bs, scale, Sight{window, keep, cap, sink, wide},
+                            out, part_m, part_l, part_acc, H, KV, D, bs, scale, Sight{window, keep, chunk, cap, sink, sinks, wide},
                             part_size, P, nullptr, DT_BF16, stream);
 }
 
@@ -1315,14 +1330,14 @@ extern "C" int as_attn_decode_mfma_shared(const void* q, const void* k_pages, co
                                           int num_items, const int* positions, const int* tok_row,
                                           const int* block_tables, int table_width, void* out, float* part_m,
                                           float* part_l, float* part_acc, int H, int KV, int D, int bs, float scale,
-                                          int window, int keep, float cap, int sink, int wide, int part_size, int P,
+                                          int window, int keep, int chunk, float cap, int sink, const float* sinks, int wide, int part_size, int P,
                                           int share, hipStream_t stream) {
   if (num_items <= 0) return AS_OK;
   if (H <= 0 || KV <= 0 || H % KV || D <= 0 || bs <= 0 || part_size <= 0 || P <= 0 || table_width <= 0)
     return AS_BAD_SHAPE;
   if (P > 1 && (!part_m || !part_l || !part_acc)) return AS_BAD_SHAPE;
   return launch_decode_mfma(q, k_pages, v_pages, items, num_items, positions, tok_row, block_tables, table_width,
-                            out, part_m, part_l, part_acc, H, KV, D, bs, scale, Sight{window, keep, cap, sink, wide},
+                            out, part_m, part_l, part_acc, H, KV, D, bs, scale, Sight{window, keep, chunk, cap, sink, sinks, wide},
                             part_size, P, nullptr, DT_BF16, stream, share);
 }
 
@@ -1346,7 +1361,7 @@ extern "C" int as_attn_decode_fresh(const void* qkv, const void* qw, const void*
   const FreshQKV fresh = {(const bf16*)qkv, qw, kw, (const float2*)cs, slots, (bf16*)k_pages, (bf16*)v_pages,
                           eps, store};
   return launch_decode_mfma(nullptr, k_pages, v_pages, items, num_tokens, positions, nullptr, block_tables,
-                            table_width, out, part_m, part_l, part_acc, H, KV, D, bs, scale, Sight{window, 0, 0.f, 0, 0},
+                            table_width, out, part_m, part_l, part_acc, H, KV, D, bs, scale, Sight{window, 0, 0, 0.f, 0, nullptr, 0},
                             part_size, P, &fresh, gains_dtype, stream);
 }
 
@@ -1381,7 +1396,7 @@ static int launch_single_query(const void* q, const void* k_pages, const void* v
   if (hipGetLastError() != hipSuccess) return AS_LAUNCH_FAILED;
   if (P > 1) {
     attn_reduce_kernel<T><<<dim3(num_items, H), D <= 64 ? 64 : (D <= 128 ? 128 : 256), 0, stream>>>(
-        items, part_m, part_l, part_acc, (T*)out, H, D, P, sight.sink, sight.wide);
+        items, part_m, part_l, part_acc, (T*)out, H, D, P, sight.sink, sight.sinks, sight.wide);
   }
   return launch_status();
 }
@@ -1392,7 +1407,7 @@ extern "C" int as_attn_single_query(const void* q, const void* k_pages, const vo
                                     const int* items, int num_items, const int* positions,
                                     const int* tok_row, const int* block_tables, int table_width, void* out,
                                     float* part_m, float* part_l, float* part_acc, int H, int KV, int D,
-                                    int bs, float scale, int window, int keep, float cap, int sink, int wide,
+                                    int bs, float scale, int window, int keep, int chunk, float cap, int sink, const float* sinks, int wide,
                                     int part_size, int P, hipStream_t stream) {
   if (num_items <= 0) return AS_OK;
   if (H <= 0 || KV <= 0 || H % KV || D <= 0 || bs <= 0 || part_size <= 0 || P <= 0 || table_width <= 0)
@@ -1401,11 +1416,11 @@ extern "C" int as_attn_single_query(const void* q, const void* k_pages, const vo
   if (dtype == DT_F32)
     return launch_single_query<float>(q, k_pages, v_pages, items, num_items, positions, tok_row, block_tables,
                                       table_width, out, part_m, part_l, part_acc, H, KV, D, bs, scale,
-                                      Sight{window, keep, cap, sink, wide}, part_size, P, stream);
+                                      Sight{window, keep, chunk, cap, sink, sinks, wide}, part_size, P, stream);
   if (dtype == DT_BF16)
     return launch_single_query<bf16>(q, k_pages, v_pages, items, num_items, positions, tok_row, block_tables,
                                      table_width, out, part_m, part_l, part_acc, H, KV, D, bs, scale,
-                                     Sight{window, keep, cap, sink, wide}, part_size, P, stream);
+                                     Sight{window, keep, chunk, cap, sink, sinks, wide}, part_size, P, stream);
   return AS_BAD_DTYPE;
 }
 
@@ -1454,6 +1469,6 @@ extern "C" int as_attn_single_query_static(const void* q, const void* k_pages, c
     part_l = part_m + rows;
   }
   return as_attn_single_query(q, k_pages, v_pages, dtype, items, num_items, positions, tok_row, block_tables,
-                              table_width, out, part_m, part_l, part_acc, H, KV, D, bs, scale, window, 0, 0.f, 0, 0,
+                              table_width, out, part_m, part_l, part_acc, H, KV, D, bs, scale, window, 0, 0, 0.f, 0, nullptr, 0,
                               part_size, P, stream);
 }

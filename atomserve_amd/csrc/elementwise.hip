@@ -712,10 +712,11 @@ __global__ __launch_bounds__(256) void whole_norm_store_kernel(
       const float v = to_f32(row[q_off + c]) + (q_bias ? q_bias[c] : 0.f);
       sq = fmaf(v, v, sq);
     }
-    for (int c = threadIdx.x; c < nk; c += blockDim.x) {
-      const float v = to_f32(row[k_off + c]) + (k_bias ? k_bias[c] : 0.f);
-      sk = fmaf(v, v, sk);
-    }
+    if (kw)
+      for (int c = threadIdx.x; c < nk; c += blockDim.x) {
+        const float v = to_f32(row[k_off + c]) + (k_bias ? k_bias[c] : 0.f);
+        sk = fmaf(v, v, sk);
+      }
     inv_q = 1.0f / sqrtf(block_sum(sq, red) / (float)nq + eps);
     inv_k = 1.0f / sqrtf(block_sum(sk, red) / (float)nk + eps);
   }
@@ -762,13 +763,40 @@ __global__ __launch_bounds__(256) void whole_norm_store_kernel(
   }
 }
 
-// The same for bfloat16 without a norm over the projection and without mixed values, where every width and offset is a
-// multiple of eight: 16 bytes of a head a thread (its bias, its partner if it turns), and for values of a prompt the
-// eight tokens that fill eight slots in a row together, each an eighth of the coordinates (see
-// qk_norm_rope_store_bf16x8_kernel).
+// The inverse root mean squares that `whole_store_bf16x8_kernel` norms with: inv[t] = (of q, of k), columns q_off .. q_off +
+// nq and k_off .. k_off + nk of proj, offsets, widths and ld multiples of eight.  A wave per token.
+__global__ __launch_bounds__(256) void whole_rms_bf16x8_kernel(const bf16* __restrict__ proj, int ld, int q_off, int k_off, int nq,
+                                                               int nk, const float* __restrict__ q_bias,
+                                                               const float* __restrict__ k_bias, float eps,
+                                                               float2* __restrict__ inv, int num_tokens) {
+  typedef __bf16 bf16x8 __attribute__((ext_vector_type(8)));
+  const int t = blockIdx.x * 4 + threadIdx.x / WAVE, lane = threadIdx.x & (WAVE - 1);
+  if (t >= num_tokens) return;
+  auto squares = [&](int off, int count, const float* bias) {
+    const bf16* row = proj + (size_t)t * ld + off;
+    float ss = 0.f;
+    for (int c = lane * 8; c < count; c += WAVE * 8) {
+      const bf16x8 r = *reinterpret_cast<const bf16x8*>(row + c);
+#pragma unroll
+      for (int j = 0; j < 8; ++j) {
+        const float v = (float)r[j] + (bias ? bias[c + j] : 0.f);
+        ss = fmaf(v, v, ss);
+      }
+    }
+    return wave_sum(ss);
+  };
+  const float sq = squares(q_off, nq, q_bias), sk = nk ? squares(k_off, nk, k_bias) : 0.f;
+  if (lane == 0) inv[t] = make_float2(1.0f / sqrtf(sq / (float)nq + eps), nk ? 1.0f / sqrtf(sk / (float)nk + eps) : 0.f);
+}
+
+// The same as whole_norm_store_kernel for bfloat16 without mixed values, where every width and offset is a
+// multiple of eight: 16 bytes of a head a thread (its bias, its norm by what whole_rms_bf16x8_kernel left, its partner if it
+// turns), and for values of a prompt the eight tokens that fill eight slots in a row together, each an eighth of the
+// coordinates (see qk_norm_rope_store_bf16x8_kernel).
 __global__ __launch_bounds__(256) void whole_store_bf16x8_kernel(
     const bf16* __restrict__ proj, int ld, int q_off, int k_off, int v_off, int H, int KV, int dim, int vdim, int Dp,
     const float* __restrict__ q_bias, const float* __restrict__ k_bias, const float* __restrict__ v_bias,
+    const float* __restrict__ qw, const float* __restrict__ kw, const float2* __restrict__ inv,
     const float2* __restrict__ cs, int half, const int* __restrict__ slots, bf16* __restrict__ q_out,
     bf16* __restrict__ k_pages, bf16* __restrict__ v_pages, int bs, int store, int maps, int num_tokens, size_t units) {
   typedef __bf16 bf16x8 __attribute__((ext_vector_type(8)));
@@ -796,6 +824,12 @@ __global__ __launch_bounds__(256) void whole_store_bf16x8_kernel(
         Gain8<float>::load(bias + c, b);
 #pragma unroll
         for (int j = 0; j < 8; ++j) x[j] += b[j];
+      }
+      if (inv) {
+        const float by = is_k ? inv[t].y : inv[t].x;
+        Gain8<float>::load((is_k ? kw : qw) + c, b);
+#pragma unroll
+        for (int j = 0; j < 8; ++j) x[j] = x[j] * by * b[j];
       }
     };
     if (d >= at && d < at + wide) piece(d, v);
@@ -847,23 +881,29 @@ __global__ __launch_bounds__(256) void whole_store_bf16x8_kernel(
 
 extern "C" int as_whole_norm_store(const void* proj, int dtype, int ld, int q_off, int k_off, int v_off, int H, int KV,
                                    int dim, int vdim, int Dp, const float* q_bias, const float* k_bias,
-                                   const float* v_bias, const float* qw, const float* kw, float eps, const float* cs,
-                                   int R, float* v_keep, int v_mode, float lam, const int* slots, void* q_out,
+                                   const float* v_bias, const float* qw, const float* kw, float eps, float* inverse,
+                                   const float* cs, int R, float* v_keep, int v_mode, float lam, const int* slots, void* q_out,
                                    void* k_pages, void* v_pages, int bs, int store, int maps, int num_tokens,
                                    hipStream_t stream) {
   if (num_tokens <= 0) return AS_OK;
   if (cs && (R <= 0 || (R & 1) || R > dim)) return AS_BAD_SHAPE;
-  if (H <= 0 || KV <= 0 || dim <= 0 || vdim <= 0 || Dp < dim || Dp < vdim || bs <= 0 || ld <= 0 || (!qw) != (!kw))
+  if (H <= 0 || KV <= 0 || dim <= 0 || vdim <= 0 || Dp < dim || Dp < vdim || bs <= 0 || ld <= 0 || (!qw && kw) || (qw && !kw && store))
     return AS_BAD_SHAPE;
   if (v_mode < 0 || v_mode > 2 || (v_mode && !v_keep)) return AS_BAD_SHAPE;
   if (maps < 1 || (maps > 1 && (cs || qw || dim % maps || H % maps))) return AS_BAD_SHAPE;
   const int eights = ld | q_off | k_off | v_off | dim | dim / maps | vdim | Dp | (cs ? R / 2 : 0) | (store ? bs : 0);
-  if (dtype == DT_BF16 && !qw && v_mode == 0 && (eights & 7) == 0) {
+  if (dtype == DT_BF16 && (!qw || inverse) && v_mode == 0 && (eights & 7) == 0) {
+    if (qw) {
+      whole_rms_bf16x8_kernel<<<(num_tokens + 3) / 4, 256, 0, stream>>>((const bf16*)proj, ld, q_off, k_off, H * dim, kw ? KV * dim : 0,
+                                                                       q_bias, k_bias, eps, (float2*)inverse, num_tokens);
+      if (hipGetLastError() != hipSuccess) return AS_LAUNCH_FAILED;
+    }
     const size_t units = (size_t)num_tokens * (store ? H + 2 * KV : H) * (Dp / 8);
     const size_t blocks = (units + 255) / 256;
     if (blocks > 0x7fffffffUL) return AS_BAD_SHAPE;
     whole_store_bf16x8_kernel<<<(int)blocks, 256, 0, stream>>>((const bf16*)proj, ld, q_off, k_off, v_off, H, KV, dim, vdim, Dp,
-                                                               q_bias, k_bias, v_bias, (const float2*)cs, cs ? R / 2 : 0, slots,
+                                                               q_bias, k_bias, v_bias, qw, kw, qw ? (const float2*)inverse : nullptr,
+                                                               (const float2*)cs, cs ? R / 2 : 0, slots,
                                                                (bf16*)q_out, (bf16*)k_pages, (bf16*)v_pages, bs, store, maps,
                                                                num_tokens, units);
     return launch_status();
@@ -886,10 +926,11 @@ extern "C" int as_whole_norm_store(const void* proj, int dtype, int ld, int q_of
 
 // ---- an output gate on attention heads --------------------------------------------------------
 // out[t, out_off + h * vdim + j] = scale * sigmoid(gate[t, gate_off + h * vdim + j]) * heads[t, h, j]
-// for j < vdim of the Dp coordinates a head is laid out with; gate [T, ld_gate], out [T, ld_out].
+// for j < vdim of the Dp coordinates a head is laid out with; gate [T, ld_gate], out [T, ld_out].  per_head: one number a
+// head, gate[t, gate_off + h].
 template <typename T>
 __global__ void sigmoid_gate_heads_kernel(const T* __restrict__ heads, int H, int vdim, int Dp,
-                                          const T* __restrict__ gate, int ld_gate, int gate_off, float scale,
+                                          const T* __restrict__ gate, int ld_gate, int gate_off, int per_head, float scale,
                                           T* __restrict__ out, int ld_out, int out_off, size_t total) {
   const size_t stride = (size_t)gridDim.x * blockDim.x;
   const int per = H * vdim;
@@ -898,24 +939,58 @@ __global__ void sigmoid_gate_heads_kernel(const T* __restrict__ heads, int H, in
     const int c = (int)(idx % per), h = c / vdim, j = c % vdim;
     const float v = to_f32(heads[(t * H + h) * Dp + j]);
     // no gate: the heads, scaled
-    out[t * ld_out + out_off + c] = from_f32<T>(gate ? scale * v / (1.0f + expf(-to_f32(gate[t * ld_gate + gate_off + c]))) : scale * v);
+    out[t * ld_out + out_off + c] = from_f32<T>(gate ? scale * v / (1.0f + expf(-to_f32(gate[t * ld_gate + gate_off + (per_head ? h : c)]))) : scale * v);
   }
 }
 
+// The same for bfloat16, 16 bytes a thread: vdim, Dp, ld_out, out_off and, without per_head, ld_gate and gate_off are
+// multiples of eight.
+__global__ __launch_bounds__(256) void sigmoid_gate_heads_bf16x8_kernel(const bf16* __restrict__ heads, int H, int vdim, int Dp,
+                                                                        const bf16* __restrict__ gate, int ld_gate, int gate_off,
+                                                                        int per_head, float scale, bf16* __restrict__ out,
+                                                                        int ld_out, int out_off, int units) {
+  typedef __bf16 bf16x8 __attribute__((ext_vector_type(8)));
+  const int unit = blockIdx.x * 256 + threadIdx.x;
+  if (unit >= units) return;
+  const int pieces = vdim / 8, th = unit / pieces, j = (unit - th * pieces) * 8, t = th / H, h = th - t * H;
+  const bf16x8 v = *reinterpret_cast<const bf16x8*>(heads + (size_t)th * Dp + j);
+  bf16x8 o;
+  if (!gate) {
+#pragma unroll
+    for (int i = 0; i < 8; ++i) o[i] = (bf16)(scale * (float)v[i]);
+  } else if (per_head) {
+    const float f = scale / (1.0f + expf(-(float)gate[(size_t)t * ld_gate + gate_off + h]));
+#pragma unroll
+    for (int i = 0; i < 8; ++i) o[i] = (bf16)(f * (float)v[i]);
+  } else {
+    const bf16x8 g = *reinterpret_cast<const bf16x8*>(gate + (size_t)t * ld_gate + gate_off + h * vdim + j);
+#pragma unroll
+    for (int i = 0; i < 8; ++i) o[i] = (bf16)(scale * (float)v[i] / (1.0f + __expf(-(float)g[i])));
+  }
+  *reinterpret_cast<bf16x8*>(out + (size_t)t * ld_out + out_off + h * vdim + j) = o;
+}
+
 extern "C" int as_sigmoid_gate_heads(const void* heads, int dtype, int H, int vdim, int Dp, const void* gate,
-                                     int ld_gate, int gate_off, float scale, void* out, int ld_out, int out_off,
-                                     int num_tokens, hipStream_t stream) {
+                                     int ld_gate, int gate_off, int per_head, float scale, void* out, int ld_out,
+                                     int out_off, int num_tokens, hipStream_t stream) {
   if (num_tokens <= 0) return AS_OK;
   if (H <= 0 || vdim <= 0 || Dp < vdim) return AS_BAD_SHAPE;
   const size_t total = (size_t)num_tokens * H * vdim;
+  const int eights = vdim | Dp | ld_out | out_off | (gate && !per_head ? ld_gate | gate_off : 0);
+  if (dtype == DT_BF16 && (eights & 7) == 0 && total / 8 < 0x7fffff00UL) {
+    const int units = (int)(total / 8);
+    sigmoid_gate_heads_bf16x8_kernel<<<(units + 255) / 256, 256, 0, stream>>>((const bf16*)heads, H, vdim, Dp, (const bf16*)gate, ld_gate,
+                                                                             gate_off, per_head, scale, (bf16*)out, ld_out, out_off, units);
+    return launch_status();
+  }
   const size_t want = (total + 255) / 256;
   const int blocks = (int)(want > 8192 ? 8192 : want);
   if (dtype == DT_F32)
     sigmoid_gate_heads_kernel<float><<<blocks, 256, 0, stream>>>((const float*)heads, H, vdim, Dp, (const float*)gate,
-                                                                 ld_gate, gate_off, scale, (float*)out, ld_out, out_off, total);
+                                                                 ld_gate, gate_off, per_head, scale, (float*)out, ld_out, out_off, total);
   else if (dtype == DT_BF16)
     sigmoid_gate_heads_kernel<bf16><<<blocks, 256, 0, stream>>>((const bf16*)heads, H, vdim, Dp, (const bf16*)gate,
-                                                                ld_gate, gate_off, scale, (bf16*)out, ld_out, out_off, total);
+                                                                ld_gate, gate_off, per_head, scale, (bf16*)out, ld_out, out_off, total);
   else return AS_BAD_DTYPE;
   return launch_status();
 }

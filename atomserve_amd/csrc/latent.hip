@@ -289,8 +289,9 @@ extern "C" int as_latent_v_expand(const void* heads, const void* uv_t, const voi
 // ---- attention over kv heads of any width ------------------------------------------------------------------
 // For pages whose heads are wider than the paged attention kernels take.  q, out [T, H, width]; k_pages
 // [pages, KV, bs, width], v_pages [pages, KV, width, bs]; a token at position p of row r sees keys 0 .. p of the row's
-// block table, or with a window > 0 the keys p - window + 1 .. p and those of the first `keep` positions; cap > 0: a
-// score s counts as cap tanh(s / cap); sink: one more score of 0 in the denominator.  grid (tokens, heads), 256 threads:
+// block table, or with a window > 0 the keys p - window + 1 .. p and those of the first `keep` positions, or with
+// chunk > 0 those of the chunk of that many positions it lies in; cap > 0: a score s counts as cap tanh(s / cap); sink: one
+// more score in the denominator, sinks[h] or 0.  grid (tokens, heads), 256 threads:
 // the visible keys come 256 at a time in order (a thread a key, its score one chain of multiply-adds), the softmax's
 // maximum and sum move on from block to block, and a thread owns every 256th coordinate of the output.  All sums are fp32 and taken in an order that only positions decide.
 #define WIDE_MAX_COLS 8  // coordinates of the output a thread owns: widths up to 2,048
@@ -302,15 +303,16 @@ __global__ __launch_bounds__(256) void wide_attend_kernel(const T* __restrict__ 
                                                           const int* __restrict__ tok_row,
                                                           const int* __restrict__ block_tables, int table_width,
                                                           T* __restrict__ out, int H, int KV, int width, int bs,
-                                                          float scale, int window, int keep, float cap, int sink,
-                                                          int wide) {
+                                                          float scale, int window, int keep, int chunk, float cap, int sink,
+                                                          const float* __restrict__ sinks, int wide) {
   extern __shared__ float lds[];  // [width] the query, [256] the block's weights
   __shared__ float red[17];
   float* qs = lds;
   float* ps = lds + width;
   const int t = blockIdx.x, h = blockIdx.y, tid = threadIdx.x;
   const int ctx = positions[t] + 1, kvh = h / (H / KV);
-  const int lo = window > 0 ? max(0, ctx - window) : 0, kept = min(keep, lo), seen = kept + ctx - lo;
+  const int lo = chunk > 0 ? (ctx - 1) / chunk * chunk : window > 0 ? max(0, ctx - window) : 0;
+  const int kept = min(keep, lo), seen = kept + ctx - lo;
   auto key_at = [&](int place) { return place < kept ? place : place - kept + lo; };
   const int* table = block_tables + (size_t)(tok_row ? tok_row[t] : t) * table_width;
   for (int i = tid; i < width; i += 256) qs[i] = to_f32(q[((size_t)t * H + h) * width + i]) * scale;
@@ -357,9 +359,9 @@ __global__ __launch_bounds__(256) void wide_attend_kernel(const T* __restrict__ 
   }
   float shrink = 1.f;
   if (sink) {
-    const float top = fmaxf(m, 0.f);
+    const float sk = sinks ? sinks[h] : 0.f, top = fmaxf(m, sk);
     shrink = expf(m - top);
-    l = l * shrink + expf(-top);
+    l = l * shrink + expf(sk - top);
   }
 #pragma unroll
   for (int c = 0; c < WIDE_MAX_COLS; ++c) {
@@ -373,19 +375,20 @@ __global__ __launch_bounds__(256) void wide_attend_kernel(const T* __restrict__ 
 
 extern "C" int as_wide_attend(const void* q, const void* k_pages, const void* v_pages, int dtype, const int* positions,
                               const int* tok_row, const int* block_tables, int table_width, void* out, int H, int KV,
-                              int width, int bs, float scale, int window, int keep, float cap, int sink, int wide, int num_tokens,
+                              int width, int bs, float scale, int window, int keep, int chunk, float cap, int sink, const float* sinks,
+                              int wide, int num_tokens,
                               hipStream_t stream) {
   if (num_tokens <= 0) return AS_OK;
   if (H <= 0 || H > 65535 || KV <= 0 || H % KV || width <= 0 || width > 256 * WIDE_MAX_COLS || bs <= 0 || table_width <= 0) return AS_BAD_SHAPE;
-  if (window < 0 || keep < 0 || (keep && window == 0) || cap < 0.f) return AS_BAD_SHAPE;
+  if (window < 0 || keep < 0 || (keep && window == 0) || cap < 0.f || chunk < 0 || (chunk && window)) return AS_BAD_SHAPE;
   dim3 grid(num_tokens, H);
   const size_t lds = (size_t)(width + 256) * sizeof(float);
   if (dtype == DT_F32)
     wide_attend_kernel<float><<<grid, 256, lds, stream>>>((const float*)q, (const float*)k_pages, (const float*)v_pages, positions,
-                                                         tok_row, block_tables, table_width, (float*)out, H, KV, width, bs, scale, window, keep, cap, sink, wide);
+                                                         tok_row, block_tables, table_width, (float*)out, H, KV, width, bs, scale, window, keep, chunk, cap, sink, sinks, wide);
   else if (dtype == DT_BF16)
     wide_attend_kernel<bf16><<<grid, 256, lds, stream>>>((const bf16*)q, (const bf16*)k_pages, (const bf16*)v_pages, positions,
-                                                        tok_row, block_tables, table_width, (bf16*)out, H, KV, width, bs, scale, window, keep, cap, sink, wide);
+                                                        tok_row, block_tables, table_width, (bf16*)out, H, KV, width, bs, scale, window, keep, chunk, cap, sink, sinks, wide);
   else return AS_BAD_DTYPE;
   return launch_status();
 }

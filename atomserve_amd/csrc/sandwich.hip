@@ -2,58 +2,16 @@
 //
 //   post_norm_add   x += norm(y) * post; out = norm(x) * gain: the norm after a sublayer, the residual sum and the norm
 //                   before the next sublayer in one pass over the row; y may be the sum of two outputs that are
-//                   normed first, each with gains of its own
+//                   normed first, each with gains of its own; either norm divides by the root mean square or, centred,
+//                   takes the mean off first; out may also be x as it is, rounded
 //   poly_norm       a N(z) + b N(z^2) + c N(z^3) + e over a row z, powers taken element by element and N the division
 //                   by the row's root mean square
+//   token_gate      gelu(z) times a row of a table that the token names
 //   map_difference  two attention maps' heads a1 - lam a2, over its root mean square, times a factor
 //
 // A row stays in registers between its reductions.  Everything between the loads and the last rounding is fp32.
 #include "common.h"
-
-// VEC consecutive values at once (4: the address a multiple of 16 bytes for fp32, of 8 for bfloat16).
-template <int VEC, typename T> __device__ __forceinline__ void load_vec(const T* p, float* v) {
-  if constexpr (VEC == 1) {
-    v[0] = to_f32(p[0]);
-  } else if constexpr (sizeof(T) == 4) {
-    const float4 r = *reinterpret_cast<const float4*>(p);
-    v[0] = r.x; v[1] = r.y; v[2] = r.z; v[3] = r.w;
-  } else {
-    const uint2 r = *reinterpret_cast<const uint2*>(p);
-    v[0] = __uint_as_float(r.x << 16); v[1] = __uint_as_float(r.x & 0xffff0000u);
-    v[2] = __uint_as_float(r.y << 16); v[3] = __uint_as_float(r.y & 0xffff0000u);
-  }
-}
-template <int VEC, typename T> __device__ __forceinline__ void store_vec(T* p, const float* v) {
-  if constexpr (VEC == 1) {
-    p[0] = from_f32<T>(v[0]);
-  } else if constexpr (sizeof(T) == 4) {
-    *reinterpret_cast<float4*>(p) = make_float4(v[0], v[1], v[2], v[3]);
-  } else {
-    bf16 b[4] = {from_f32<bf16>(v[0]), from_f32<bf16>(v[1]), from_f32<bf16>(v[2]), from_f32<bf16>(v[3])};
-    *reinterpret_cast<uint2*>(p) = *reinterpret_cast<const uint2*>(b);
-  }
-}
-
-// N sums over the workgroup at once (up to 16 waves), in a fixed order; `red` is a __shared__ float[N * 16].
-template <int N>
-__device__ __forceinline__ void block_sums(float (&v)[N], float* red) {
-  const int lane = threadIdx.x & (WAVE - 1), wave = threadIdx.x / WAVE, waves = blockDim.x / WAVE;
-#pragma unroll
-  for (int i = 0; i < N; ++i) v[i] = wave_sum(v[i]);
-  if (waves == 1) return;
-  __syncthreads();  // protects `red` against a previous use
-  if (lane == 0) {
-#pragma unroll
-    for (int i = 0; i < N; ++i) red[i * 16 + wave] = v[i];
-  }
-  __syncthreads();
-#pragma unroll
-  for (int i = 0; i < N; ++i) {
-    float s = 0.f;
-    for (int w = 0; w < waves; ++w) s += red[i * 16 + w];
-    v[i] = s;
-  }
-}
+#include "rows.h"
 
 struct PostNorm {
   const float* bias1;  // [n] added to y1, y2 as they are read (null: none)
@@ -65,10 +23,12 @@ struct PostNorm {
   float eps_post;
   const float* gain;   // [n] gains of the norm that follows (null: none is taken)
   float eps;
+  int centre_post;     // CENTRED: the norm after the sublayer takes the mean off first (a layer norm)
+  int centre;          // CENTRED: the norm that follows does
 };
 
 // A workgroup per row; a thread owns CH pieces of VEC neighbouring columns.
-template <typename T, int VEC, int CH, bool PAIR>
+template <typename T, int VEC, int CH, bool PAIR, bool CENTRED>
 __global__ __launch_bounds__(1024) void post_norm_add_kernel(float* __restrict__ x, const T* __restrict__ y1,
                                                              const T* __restrict__ y2, PostNorm p,
                                                              const int* __restrict__ rows, T* __restrict__ out, int n,
@@ -102,12 +62,28 @@ __global__ __launch_bounds__(1024) void post_norm_add_kernel(float* __restrict__
     }
 #pragma unroll
     for (int k = 0; k < VEC; ++k) {
-      sums[0] = fmaf(d[c][k], d[c][k], sums[0]);
+      if (CENTRED && !PAIR) sums[0] += p.centre_post ? d[c][k] : d[c][k] * d[c][k];
+      else sums[0] = fmaf(d[c][k], d[c][k], sums[0]);
       if (PAIR) sums[PAIR ? 1 : 0] = fmaf(v[c][k], v[c][k], sums[PAIR ? 1 : 0]);
     }
   }
   block_sums(sums, red);
   float one[1];
+  // a row's mean comes off: what `one` holds is the row's sum, and then the sum of the squared deviations
+  auto centre = [&](float(&r)[CH][VEC]) {
+    const float mean = one[0] / (float)n;
+    one[0] = 0.f;
+#pragma unroll
+    for (int c = 0; c < CH; ++c) {
+      if ((int)(c * blockDim.x + threadIdx.x) * VEC >= n) continue;
+#pragma unroll
+      for (int k = 0; k < VEC; ++k) {
+        r[c][k] -= mean;
+        one[0] = fmaf(r[c][k], r[c][k], one[0]);
+      }
+    }
+    block_sums(one, red);
+  };
   if (PAIR) {
     const float inv1 = 1.0f / sqrtf(sums[0] / (float)n + p.eps_in), inv2 = 1.0f / sqrtf(sums[PAIR ? 1 : 0] / (float)n + p.eps_in);
     one[0] = 0.f;
@@ -121,13 +97,15 @@ __global__ __launch_bounds__(1024) void post_norm_add_kernel(float* __restrict__
 #pragma unroll
       for (int k = 0; k < VEC; ++k) {
         d[c][k] = d[c][k] * inv1 * g1[k] + v[c][k] * inv2 * g2[k];
-        one[0] = fmaf(d[c][k], d[c][k], one[0]);
+        if (CENTRED) one[0] += p.centre_post ? d[c][k] : d[c][k] * d[c][k];
+        else one[0] = fmaf(d[c][k], d[c][k], one[0]);
       }
     }
     block_sums(one, red);
   } else {
     one[0] = sums[0];
   }
+  if (CENTRED && p.centre_post) centre(d);
   const float inv_post = 1.0f / sqrtf(one[0] / (float)n + p.eps_post);
   one[0] = 0.f;
 #pragma unroll
@@ -140,12 +118,15 @@ __global__ __launch_bounds__(1024) void post_norm_add_kernel(float* __restrict__
 #pragma unroll
     for (int k = 0; k < VEC; ++k) {
       v[c][k] += d[c][k] * inv_post * g[k];
-      one[0] = fmaf(v[c][k], v[c][k], one[0]);
+      if (CENTRED) one[0] += p.centre ? v[c][k] : v[c][k] * v[c][k];
+      else one[0] = fmaf(v[c][k], v[c][k], one[0]);
     }
     if (update_x) store_vec<VEC>(x + s * n + i, v[c]);
+    if (!p.gain && out) store_vec<VEC>(out + (size_t)r * n + i, v[c]);
   }
   if (!p.gain) return;
   block_sums(one, red);
+  if (CENTRED && p.centre) centre(v);
   const float inv = 1.0f / sqrtf(one[0] / (float)n + p.eps);
 #pragma unroll
   for (int c = 0; c < CH; ++c) {
@@ -159,30 +140,19 @@ __global__ __launch_bounds__(1024) void post_norm_add_kernel(float* __restrict__
   }
 }
 
-// How many threads take a row and in how many pieces each: few rows (a decode step) as wide as they come, many rows
-// with more in a thread's registers.  False: the row is longer than the kernels keep.
-static bool row_shape(int rows, int n, int vec, int* threads, int* pieces) {
-  const int want = (n + vec - 1) / vec;
-  int ch = rows >= 512 ? 4 : 1;
-  while (ch > 1 && want <= 64 * ch / 2) ch /= 2;
-  while (ch < (vec == 1 ? 32 : 8) && (want + ch - 1) / ch > 1024) ch *= 2;
-  const int t = ((want + ch - 1) / ch + 63) / 64 * 64;
-  if (t > 1024) return false;
-  *threads = t;
-  *pieces = ch;
-  return true;
-}
-
 template <typename T, int VEC>
 static int launch_post_norm(float* x, const void* y1, const void* y2, const PostNorm& p, const int* rows, void* out, int n_out,
                             int n, int update_x, hipStream_t stream) {
   int threads, ch;
   if (!row_shape(n_out, n, VEC, &threads, &ch)) return AS_BAD_SHAPE;
-#define LAUNCH(CHV)                                                                                                    \
-  if (y2) post_norm_add_kernel<T, VEC, CHV, true><<<n_out, threads, 0, stream>>>(x, (const T*)y1, (const T*)y2, p, rows, \
-                                                                                 (T*)out, n, update_x);                \
-  else post_norm_add_kernel<T, VEC, CHV, false><<<n_out, threads, 0, stream>>>(x, (const T*)y1, nullptr, p, rows, (T*)out, \
-                                                                               n, update_x)
+#define LAUNCH2(CHV, PAIRV, CENTREDV)                                                                                       \
+  post_norm_add_kernel<T, VEC, CHV, PAIRV, CENTREDV><<<n_out, threads, 0, stream>>>(x, (const T*)y1, (const T*)y2, p, rows, \
+                                                                                    (T*)out, n, update_x)
+#define LAUNCH(CHV)                                                                \
+  if (y2 && (p.centre || p.centre_post)) LAUNCH2(CHV, true, true);                 \
+  else if (y2) LAUNCH2(CHV, true, false);                                          \
+  else if (p.centre || p.centre_post) LAUNCH2(CHV, false, true);                   \
+  else LAUNCH2(CHV, false, false)
   switch (ch) {
     case 1: LAUNCH(1); break;
     case 2: LAUNCH(2); break;
@@ -196,17 +166,20 @@ static int launch_post_norm(float* x, const void* y1, const void* y2, const Post
       break;
   }
 #undef LAUNCH
+#undef LAUNCH2
   return launch_status();
 }
 
 // x fp32 [T, n]; y1, y2 [T, n] and out [n_out, n] of `dtype`; row r of out comes from row rows[r] (or r) of the rest.
+// centre_post, centre: the norm after the sublayer, the one that follows, take the row's mean off first.  gain null with
+// out given: out receives the stream itself.
 extern "C" int as_post_norm_add(float* x, const void* y1, const void* y2, int dtype, const float* bias1, const float* bias2,
                                 const float* gain1, const float* gain2, float eps_in, const float* post, float eps_post,
-                                const float* gain, float eps, const int* rows, void* out, int n_out, int n,
-                                int update_x, hipStream_t stream) {
+                                const float* gain, float eps, int centre_post, int centre, const int* rows, void* out,
+                                int n_out, int n, int update_x, hipStream_t stream) {
   if (n_out <= 0) return AS_OK;
   if (n <= 0 || !x || !y1 || !post || (gain && !out) || (y2 && (!gain1 || !gain2)) || (!y2 && bias2)) return AS_BAD_SHAPE;
-  const PostNorm p = {bias1, bias2, gain1, gain2, eps_in, post, eps_post, gain, eps};
+  const PostNorm p = {bias1, bias2, gain1, gain2, eps_in, post, eps_post, gain, eps, centre_post, centre};
   if (dtype == DT_F32)
     return n % 4 ? launch_post_norm<float, 1>(x, y1, y2, p, rows, out, n_out, n, update_x, stream)
                  : launch_post_norm<float, 4>(x, y1, y2, p, rows, out, n_out, n, update_x, stream);
@@ -214,6 +187,120 @@ extern "C" int as_post_norm_add(float* x, const void* y1, const void* y2, int dt
     return n % 4 ? launch_post_norm<bf16, 1>(x, y1, y2, p, rows, out, n_out, n, update_x, stream)
                  : launch_post_norm<bf16, 4>(x, y1, y2, p, rows, out, n_out, n, update_x, stream);
   return AS_BAD_DTYPE;
+}
+
+// ---- a layer norm of the stream, with a plain output still to be added ---------------------------------------------
+// v = x[s] (+ y[s]), s = rows[r] or r; x receives v if update_x; out[r] = (v - mean) / sqrt(mean((v - mean)^2) + eps) * gain.
+template <typename T, int VEC, int CH>
+__global__ __launch_bounds__(1024) void layer_norm_kernel(float* __restrict__ x, const T* __restrict__ y,
+                                                          const float* __restrict__ gain, float eps,
+                                                          const int* __restrict__ rows, T* __restrict__ out, int n, int update_x) {
+  __shared__ float red[16];
+  const int r = blockIdx.x;
+  const size_t s = rows ? (size_t)rows[r] : (size_t)r;
+  float v[CH][VEC], one[1] = {0.f};
+#pragma unroll
+  for (int c = 0; c < CH; ++c) {
+    const int i = (c * blockDim.x + threadIdx.x) * VEC;
+#pragma unroll
+    for (int k = 0; k < VEC; ++k) v[c][k] = 0.f;
+    if (i >= n) continue;
+    load_vec<VEC>(x + s * n + i, v[c]);
+    if (y) {
+      float d[VEC];
+      load_vec<VEC>(y + s * n + i, d);
+#pragma unroll
+      for (int k = 0; k < VEC; ++k) v[c][k] += d[k];
+      if (update_x) store_vec<VEC>(x + s * n + i, v[c]);
+    }
+#pragma unroll
+    for (int k = 0; k < VEC; ++k) one[0] += v[c][k];
+  }
+  block_sums(one, red);
+  const float mean = one[0] / (float)n;
+  one[0] = 0.f;
+#pragma unroll
+  for (int c = 0; c < CH; ++c) {
+    if ((int)(c * blockDim.x + threadIdx.x) * VEC >= n) continue;
+#pragma unroll
+    for (int k = 0; k < VEC; ++k) {
+      v[c][k] -= mean;
+      one[0] = fmaf(v[c][k], v[c][k], one[0]);
+    }
+  }
+  block_sums(one, red);
+  const float inv = 1.0f / sqrtf(one[0] / (float)n + eps);
+#pragma unroll
+  for (int c = 0; c < CH; ++c) {
+    const int i = (c * blockDim.x + threadIdx.x) * VEC;
+    if (i >= n) continue;
+    float g[VEC];
+    load_vec<VEC>(gain + i, g);
+#pragma unroll
+    for (int k = 0; k < VEC; ++k) v[c][k] *= inv * g[k];
+    store_vec<VEC>(out + (size_t)r * n + i, v[c]);
+  }
+}
+
+template <typename T, int VEC>
+static int launch_layer_norm(float* x, const void* y, const float* gain, float eps, const int* rows, void* out, int n_out, int n,
+                             int update_x, hipStream_t stream) {
+  int threads, ch;
+  if (!row_shape(n_out, n, VEC, &threads, &ch)) return AS_BAD_SHAPE;
+#define LAUNCH(CHV) layer_norm_kernel<T, VEC, CHV><<<n_out, threads, 0, stream>>>(x, (const T*)y, gain, eps, rows, (T*)out, n, update_x)
+  switch (ch) {
+    case 1: LAUNCH(1); break;
+    case 2: LAUNCH(2); break;
+    case 4: LAUNCH(4); break;
+    case 8: LAUNCH(8); break;
+    default:
+      if constexpr (VEC == 1) {
+        if (ch == 16) { LAUNCH(16); }
+        else { LAUNCH(32); }
+      }
+      break;
+  }
+#undef LAUNCH
+  return launch_status();
+}
+
+extern "C" int as_layer_norm(float* x, const void* y, const float* gain, float eps, const int* rows, void* out, int dtype,
+                             int n_out, int n, int update_x, hipStream_t stream) {
+  if (n_out <= 0) return AS_OK;
+  if (n <= 0 || !x || !gain || !out) return AS_BAD_SHAPE;
+  if (dtype == DT_F32)
+    return n % 4 ? launch_layer_norm<float, 1>(x, y, gain, eps, rows, out, n_out, n, update_x, stream)
+                 : launch_layer_norm<float, 4>(x, y, gain, eps, rows, out, n_out, n, update_x, stream);
+  if (dtype == DT_BF16)
+    return n % 4 ? launch_layer_norm<bf16, 1>(x, y, gain, eps, rows, out, n_out, n, update_x, stream)
+                 : launch_layer_norm<bf16, 4>(x, y, gain, eps, rows, out, n_out, n, update_x, stream);
+  return AS_BAD_DTYPE;
+}
+
+// ---- the token's own input, gated ------------------------------------------------------------------------------------
+// out[t, i] = gelu_tanh(z[t, i]) * table[ids[t], i], i < dim; z, table and out of one type, everything between fp32.
+template <typename T>
+__global__ __launch_bounds__(256) void token_gate_kernel(const T* __restrict__ z, const T* __restrict__ table,
+                                                         const int* __restrict__ ids, T* __restrict__ out, int dim, int total) {
+  const int at = blockIdx.x * 256 + threadIdx.x;
+  if (at >= total) return;
+  const int t = at / dim, i = at - t * dim;
+  const float v = to_f32(z[at]);
+  const float g = 0.5f * v * (1.0f + tanhf(0.7978845608028654f * (v + 0.044715f * v * v * v)));
+  out[at] = from_f32<T>(g * to_f32(table[(size_t)ids[t] * dim + i]));
+}
+
+extern "C" int as_token_gate(const void* z, const void* table, const int* ids, int dtype, void* out, int dim, int num_tokens,
+                             hipStream_t stream) {
+  if (num_tokens <= 0) return AS_OK;
+  if (dim <= 0 || (long)num_tokens * dim > 0x7fffff00L) return AS_BAD_SHAPE;
+  const int total = num_tokens * dim, blocks = (total + 255) / 256;
+  if (dtype == DT_F32)
+    token_gate_kernel<float><<<blocks, 256, 0, stream>>>((const float*)z, (const float*)table, ids, (float*)out, dim, total);
+  else if (dtype == DT_BF16)
+    token_gate_kernel<bf16><<<blocks, 256, 0, stream>>>((const bf16*)z, (const bf16*)table, ids, (bf16*)out, dim, total);
+  else return AS_BAD_DTYPE;
+  return launch_status();
 }
 
 // ---- a polynomial of normed powers ------------------------------------------------------------------------------

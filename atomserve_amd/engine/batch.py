@@ -88,7 +88,8 @@ class StepBatch:
     all_tokens [T]: every token (in a decode step those with the longest contexts first);
     split((short, tile)): the rows sorted as a mixer asks (`RowSplit`), one for every distinct answer of
     the model's mixers (`row_splits`), so that mixers with different kernels share a step;
-    row_first, row_len, row_start, row_slots [R] int32 (for mixers with per-request state)
+    row_first, row_len, row_start, row_slots [R] int32 (for mixers with per-request state); longest_row: the
+    most tokens that a row brings (known on the host)
     """
 
     def __init__(self, rows, block_size: int, num_paged_groups: int, vocab_size: int, device, pools=None,
@@ -274,6 +275,7 @@ class StepBatch:
         self._staging, self._widths, self._vocab = staging, widths, vocab_size
 
         self.num_tokens, self.num_rows = T, R
+        self.longest_row = max(len(row.tokens) for row in rows)
         self.decode_only = all(len(row.tokens) == 1 for row in rows)  # token t is row t
         self.token_ids, self.positions, self.tok_row = parts["token_ids"], parts["positions"], parts["tok_row"]
         self.logits_rows, self.num_logits = parts["logits_rows"], len(want)

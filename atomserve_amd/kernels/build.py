@@ -20,9 +20,9 @@ ARCH = "gfx950"
 # Packed fp32 instructions are switched off for every kernel of this package.
 FLAGS = ["-O3", "-std=c++17", "-shared", "-fPIC", f"--offload-arch={ARCH}",
          "-Xclang", "-target-feature", "-Xclang", "-packed-fp32-ops", "-Wno-unused-command-line-argument"]  # fmt: skip
-HEADERS = ["common.h", "no_alloc.h"]
+HEADERS = ["common.h", "no_alloc.h", "rows.h"]
 LIBRARIES = ("elementwise", "attention", "attention_mix", "gemm", "sampling", "blas", "recurrent", "moe", "layer_ops",
-             "linear_attention", "latent", "streams", "sandwich")
+             "linear_attention", "latent", "streams", "sandwich", "state_space")
 LINK = {"blas": ["-lhipblaslt"]}  # what a library links beside the HIP runtime
 
 

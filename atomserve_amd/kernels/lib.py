@@ -29,12 +29,14 @@ SIGNATURES = {
     "as_head_norm_store": ("elementwise", [P, I, I, I, I, I, I, I, I, I, I, P, P, I, F, P, P, P, P, I, I, I, P, I, P]),
     "as_gated_add_norm": ("elementwise", [P, P, P, I, I, I, P, F, P, P, I, F, P, I, I, I, I, P, P, P]),
     "as_relu2": ("elementwise", [P, I, I, I, P, I, I, P]),
-    "as_whole_norm_store": ("elementwise", [P, I, I, I, I, I, I, I, I, I, I, P, P, P, P, P, F, P, I, P, I, F, P, P, P, P, I, I, I, I, P]),
-    "as_post_norm_add": ("sandwich", [P, P, P, I, P, P, P, P, F, P, F, P, F, P, P, I, I, I, P]),
+    "as_whole_norm_store": ("elementwise", [P, I, I, I, I, I, I, I, I, I, I, P, P, P, P, P, F, P, P, I, P, I, F, P, P, P, P, I, I, I, I, P]),
+    "as_post_norm_add": ("sandwich", [P, P, P, I, P, P, P, P, F, P, F, P, F, I, I, P, P, I, I, I, P]),
+    "as_layer_norm": ("sandwich", [P, P, P, F, P, P, I, I, I, I, P]),
+    "as_token_gate": ("sandwich", [P, P, P, I, P, I, I, P]),
     "as_poly_norm": ("sandwich", [P, I, P, F, P, I, I, P]),
     "as_map_difference": ("sandwich", [P, I, I, I, I, F, F, F, P, I, I, I, I, P]),
     "as_streams_step": ("streams", [P, P, I, I, P, I, P, P, F, P, P, F, P, P, I, P]),
-    "as_sigmoid_gate_heads": ("elementwise", [P, I, I, I, I, P, I, I, F, P, I, I, I, P]),
+    "as_sigmoid_gate_heads": ("elementwise", [P, I, I, I, I, P, I, I, I, F, P, I, I, I, P]),
     "as_short_conv": ("recurrent", [P, I, I, I, I, P, P, P, I, I, I, P, P, P, P, P, P, P, I, I, I, P]),
     "as_delta_prepare": ("recurrent", [P, I, I, I, I, P, I, I, I, I, P, P, I, P, P, I, P]),
     "as_delta_scan": ("recurrent", [P, I, I, I, I, I, P, P, P, P, P, P, P, I, P, I, I, P]),
@@ -61,18 +63,20 @@ SIGNATURES = {
     "as_channel_chunks": ("linear_attention", [P, I, I, I, I, I, I, I, I, F, P, P, P, P, P, P, I, P, I, P]),
     "as_channel_decays": ("linear_attention", [P, I, I, I, I, P, P, F, P, I, I, P]),
     "as_decay_finish": ("linear_attention", [P, I, I, F, P, P, I, I, I, I, P, I, P]),
+    "as_state_space": ("state_space", [P, I, I, I, I, I, P, I, I, I, P, P, P, P, P, P, P, P, I, P, I, I, I, I, P, P, P]),
+    "as_gated_group_norm": ("state_space", [P, P, I, I, I, P, F, I, I, P, I, P]),
     "as_rows_rms_norm": ("latent", [P, I, I, I, I, P, F, P, I, P]),
     "as_latent_kv_store": ("latent", [P, I, I, I, I, I, P, F, P, P, P, P, I, I, I, P]),
     "as_latent_q_absorb": ("latent", [P, I, I, P, P, I, I, I, I, I, P, P, I, I, P]),
     "as_latent_v_expand": ("latent", [P, P, P, I, I, I, I, I, P, I, I, P, I, P]),
-    "as_wide_attend": ("latent", [P, P, P, I, P, P, P, I, P, I, I, I, I, F, I, I, F, I, I, I, P]),
+    "as_wide_attend": ("latent", [P, P, P, I, P, P, P, I, P, I, I, I, I, F, I, I, I, F, I, P, I, I, P]),
     "as_attn_headmix_mfma": ("attention_mix", [P, P, P, P, I, I, I, P, P, P, I, P, P, I, I, I, I, I, F, I, I, I, P, P, P]),
     "as_attn_headmix": ("attention_mix", [P, P, P, I, P, I, I, P, P, P, I, P, P, I, I, I, I, I, F, I, I, P]),
-    "as_attn_single_query": ("attention", [P, P, P, I, P, I, P, P, P, I, P, P, P, P, I, I, I, I, F, I, I, F, I, I, I, I, P]),
-    "as_attn_decode_mfma": ("attention", [P, P, P, P, I, P, P, P, I, P, P, P, P, I, I, I, I, F, I, I, F, I, I, I, I, P]),
-    "as_attn_decode_mfma_shared": ("attention", [P, P, P, P, I, P, P, P, I, P, P, P, P, I, I, I, I, F, I, I, F, I, I, I, I, I, P]),
+    "as_attn_single_query": ("attention", [P, P, P, I, P, I, P, P, P, I, P, P, P, P, I, I, I, I, F, I, I, I, F, I, P, I, I, I, P]),
+    "as_attn_decode_mfma": ("attention", [P, P, P, P, I, P, P, P, I, P, P, P, P, I, I, I, I, F, I, I, I, F, I, P, I, I, I, P]),
+    "as_attn_decode_mfma_shared": ("attention", [P, P, P, P, I, P, P, P, I, P, P, P, P, I, I, I, I, F, I, I, I, F, I, P, I, I, I, I, P]),
     "as_attn_decode_fresh": ("attention", [P, P, P, I, P, P, F, I, P, P, P, I, P, P, I, P, P, P, P, I, I, I, I, F, I, I, I, P]),
-    "as_attn_prefill_mfma": ("attention", [P, P, P, P, I, P, I, P, I, I, I, I, F, I, I, F, I, I, I, I, I, P, P, P, P]),
+    "as_attn_prefill_mfma": ("attention", [P, P, P, P, I, P, I, P, I, I, I, I, F, I, I, I, F, I, P, I, I, I, I, P, P, P, P]),
     "as_gemm_f32": ("gemm", [P, P, P, I, I, I, P]),
     "as_gemm_bf16_skinny": ("gemm", [P, P, P, P, I, I, I, I, I, P]),
     "as_gemm_bf16_gated": ("gemm", [P, P, P, P, I, I, I, P]),

@@ -208,17 +208,23 @@ def silu_mul(gate_up, out) -> None:
 SINGLE_QUERY_MAX_HEAD_DIM = 256
 
 
-def _sight(window, keep_first, softcap, sink, q, out) -> tuple:
-    """(window, keep, cap, sink, wide) as the attention kernels take them: what a query sees, how scores become weights and
-    whether bfloat16 heads' results are written in fp32."""
+def _sight(window, keep_first, chunk, softcap, sink, q, out) -> tuple:
+    """(window, keep, chunk, cap, sink, sinks, wide) as the attention kernels take them: what a query sees, how scores become
+    weights and whether bfloat16 heads' results are written in fp32."""
     _check(out, "out", (q.dtype, F32), tuple(q.shape))
-    if window < 0 or keep_first < 0 or softcap < 0:
-        raise KernelError("attention: a window, a number of kept tokens and a cap of the scores are not negative")
-    return int(window), int(keep_first) if window > 0 else 0, float(softcap), int(bool(sink)), int(out.dtype != q.dtype)
+    if window < 0 or keep_first < 0 or softcap < 0 or chunk < 0 or (chunk and window):
+        raise KernelError("attention: a window, a number of kept tokens, a cap of the scores and a chunk are not negative; "
+                          "a sequence is cut into chunks or seen through a window")  # fmt: skip
+    sinks = 0
+    if isinstance(sink, torch.Tensor):
+        _check(sink, "sinks", F32, (q.shape[1],))
+        sinks = _ptr(sink)
+    has_sink = 1 if sinks else int(bool(sink))
+    return int(window), int(keep_first) if window > 0 else 0, int(chunk), float(softcap), has_sink, sinks, int(out.dtype != q.dtype)
 
 
 def attn_single_query(q, k_pages, v_pages, items, positions, tok_row, block_tables, out, scale, window,
-                      max_context, part_size=None, force_generic=False, keep_first=0, softcap=0.0, sink=False) -> None:  # fmt: skip
+                      max_context, part_size=None, force_generic=False, keep_first=0, softcap=0.0, sink=False, chunk=0) -> None:  # fmt: skip
     """Attention of single query tokens over the paged cache.  bfloat16 with head widths in steps
     of 32 and pages of a multiple of 16 tokens runs on the matrix cores (a group of more than 16 query
     heads, or of wide heads that overfill a workgroup's LDS, as several equal groups that read the same kv
@@ -228,10 +234,12 @@ def attn_single_query(q, k_pages, v_pages, items, positions, tok_row, block_tabl
     order; positions, tok_row [T] int32 (tok_row None: token t belongs to row t, a decode step);
     block_tables [R, W] int32; max_context: host bound on positions[items] + 1.
     window > 0: a query at p sees the keys p - window + 1 .. p and those of the first `keep_first` positions.
-    softcap > 0: a score s counts as softcap tanh(s / softcap).  sink: the softmax's denominator has one more score of 0."""
+    chunk > 0 (without a window): a query sees the keys of its own chunk, chunks of that many positions counted from 0.
+    softcap > 0: a score s counts as softcap tanh(s / softcap).  sink: the softmax's denominator has one more score, of 0
+    (True) or per query head (a tensor fp32 [H])."""
     _check(q, "q", (F32, BF16), (None, None, None))
     T, H, D = q.shape
-    sight = _sight(window, keep_first, softcap, sink, q, out)
+    sight = _sight(window, keep_first, chunk, softcap, sink, q, out)
     _check(k_pages, "k_pages", q.dtype, (None, None, None, D))
     _, KV, bs, _ = k_pages.shape
     _check(v_pages, "v_pages", q.dtype, (k_pages.shape[0], KV, D, bs))
@@ -246,10 +254,10 @@ def attn_single_query(q, k_pages, v_pages, items, positions, tok_row, block_tabl
     N = T if items is None else items.shape[0]
     if N == 0:
         return
-    chunk = 4 if q.dtype == F32 else 8
-    if H % KV or D % chunk or D > SINGLE_QUERY_MAX_HEAD_DIM:
+    piece = 4 if q.dtype == F32 else 8
+    if H % KV or D % piece or D > SINGLE_QUERY_MAX_HEAD_DIM:
         raise KernelError(f"attention: unsupported heads {H}/{KV} or head width {D} "
-                          f"(needs a multiple of {chunk}, at most {SINGLE_QUERY_MAX_HEAD_DIM})")  # fmt: skip
+                          f"(needs a multiple of {piece}, at most {SINGLE_QUERY_MAX_HEAD_DIM})")  # fmt: skip
     if max_context > block_tables.shape[1] * bs:
         raise KernelError("attention: block tables are shorter than the longest context")
     G = H // KV
@@ -257,12 +265,12 @@ def attn_single_query(q, k_pages, v_pages, items, positions, tok_row, block_tabl
     share = next((G // g for g in range(min(G, 16), 0, -1) if G % g == 0 and _decode_mfma_fits(D, g)), 0)
     mfma = q.dtype == BF16 and D % 32 == 0 and bs % 16 == 0 and share > 0 and not force_generic
     if mfma and share > 1:
-        part_size, P, part_m, part_l, part_acc = _partitions(N, H, KV * share, D, max_context, window, True, part_size, q.device, sight[1])
+        part_size, P, part_m, part_l, part_acc = _partitions(N, H, KV * share, D, max_context, window or chunk, True, part_size, q.device, sight[1])
         call("as_attn_decode_mfma_shared", _ptr(q), _ptr(k_pages), _ptr(v_pages), _ptr(items), N, _ptr(positions),
              _ptr(tok_row), _ptr(block_tables), block_tables.shape[1], _ptr(out), _ptr(part_m), _ptr(part_l),
              _ptr(part_acc), H, KV * share, D, bs, float(scale), *sight, part_size, P, share, _stream())  # fmt: skip
         return
-    part_size, P, part_m, part_l, part_acc = _partitions(N, H, KV, D, max_context, window, mfma, part_size, q.device, sight[1])
+    part_size, P, part_m, part_l, part_acc = _partitions(N, H, KV, D, max_context, window or chunk, mfma, part_size, q.device, sight[1])
     if mfma:
         call("as_attn_decode_mfma", _ptr(q), _ptr(k_pages), _ptr(v_pages), _ptr(items), N, _ptr(positions),
              _ptr(tok_row), _ptr(block_tables), block_tables.shape[1], _ptr(out), _ptr(part_m), _ptr(part_l),
@@ -508,7 +516,7 @@ def _prefill_plan_of(num_tiles, H, KV, D, max_context, window, query_tiles, tile
 
 
 def attn_prefill(q, k_pages, v_pages, tiles, block_tables, out, scale, window, max_context, query_tiles=None,
-                 tile_keys: int = 0, keep_first=0, softcap=0.0, sink=False) -> None:  # fmt: skip
+                 tile_keys: int = 0, keep_first=0, softcap=0.0, sink=False, chunk=0) -> None:  # fmt: skip
     """Causal attention of prompt portions over the paged cache, bfloat16, on the matrix cores.
 
     tiles [Nt, 4] int32: (first flat token, count <= 64, block-table row, position of the first
@@ -517,10 +525,10 @@ def attn_prefill(q, k_pages, v_pages, tiles, block_tables, out, scale, window, m
     query_tiles: column tiles of 16 queries that a wave owns, 2 or 1; None: chosen here.
     tile_keys: the sum over the tiles of (position of the first token + count), if the caller knows it: how the
     work is cut is chosen better with it (speed only).
-    window, keep_first, softcap, sink: as for `attn_single_query`."""
+    window, keep_first, softcap, sink, chunk: as for `attn_single_query`."""
     _check(q, "q", BF16, (None, None, None))
     T, H, D = q.shape
-    sight = _sight(window, keep_first, softcap, sink, q, out)
+    sight = _sight(window, keep_first, chunk, softcap, sink, q, out)
     _check(k_pages, "k_pages", BF16, (None, None, None, D))
     _, KV, bs, _ = k_pages.shape
     _check(v_pages, "v_pages", BF16, (k_pages.shape[0], KV, D, bs))
@@ -532,7 +540,7 @@ def attn_prefill(q, k_pages, v_pages, tiles, block_tables, out, scale, window, m
         raise KernelError(f"prefill attention: unsupported heads {H}/{KV}, head width {D} or page size {bs}")
     if max_context > block_tables.shape[1] * bs:
         raise KernelError("attention: block tables are shorter than the longest context")
-    query_tiles, pieces, piece_rounds = _prefill_plan(tiles.shape[0], H, KV, D, max_context, window, query_tiles, tile_keys, sight[1])
+    query_tiles, pieces, piece_rounds = _prefill_plan(tiles.shape[0], H, KV, D, max_context, window or chunk, query_tiles, tile_keys, sight[1])
     cut = part_ml = part_acc = None
     if pieces > 1:
         cut = torch.empty(tiles.shape[0] * KV * _prefill_units(query_tiles, H // KV), dtype=I32, device=q.device)
@@ -1042,9 +1050,10 @@ def topk(logits, k, values, indices) -> None:
 
 
 def post_norm_add(x, y, post, eps_post, gain=None, eps: float = 0.0, out=None, rows=None, update_x=True, other=None, gains=None,
-                  biases=(None, None), eps_in: float = 0.0) -> None:  # fmt: skip
+                  biases=(None, None), eps_in: float = 0.0, centre_post: bool = False, centre: bool = False) -> None:  # fmt: skip
     """v = x[s] + norm(d[s]) * post with s = rows[r] or r (eps_post inside the root), x fp32 [T, n] receiving v when
-    `update_x`; out[r] = norm(v) * gain (gain None: no norm is taken).  d = y (+ biases[0]); with `other`, d =
+    `update_x`; out[r] = norm(v) * gain (gain None: no norm is taken, and out, if there is one, receives v itself).
+    centre_post, centre: that norm takes the row's mean off first (a layer norm without a bias).  d = y (+ biases[0]); with `other`, d =
     norm(y + biases[0]) * gains[0] + norm(other + biases[1]) * gains[1] (eps_in).  y, other [T, n] and out in the compute
     dtype; post, gain, gains and biases fp32 [n]."""
     _check(x, "x", F32, (None, None))
@@ -1056,8 +1065,8 @@ def post_norm_add(x, y, post, eps_post, gain=None, eps: float = 0.0, out=None, r
         n_out = rows.shape[0]
         if update_x:
             raise KernelError("post_norm_add: the stream is updated whole, not by rows")
-    if (gain is None) != (out is None):
-        raise KernelError("post_norm_add: a norm's gain and its output come together")
+    if gain is not None and out is None:
+        raise KernelError("post_norm_add: a norm's gain comes with its output")
     for name, t in (("post", post), ("gain", gain), ("bias", biases[0]), ("other bias", biases[1])):
         if t is not None or name == "post":
             _check(t, name, F32, (n,))
@@ -1072,8 +1081,37 @@ def post_norm_add(x, y, post, eps_post, gain=None, eps: float = 0.0, out=None, r
     elif biases[1] is not None:
         raise KernelError("post_norm_add: a second bias belongs to a second output")
     call("as_post_norm_add", _ptr(x), _ptr(y), _ptr(other), _DT[y.dtype], _ptr(biases[0]), _ptr(biases[1]), _ptr(g1), _ptr(g2),
-         float(eps_in), _ptr(post), float(eps_post), _ptr(gain), float(eps), _ptr(rows), _ptr(out), n_out, n,
+         float(eps_in), _ptr(post), float(eps_post), _ptr(gain), float(eps), int(bool(centre_post)),
+         int(bool(centre)), _ptr(rows), _ptr(out), n_out, n, int(bool(update_x)), _stream())  # fmt: skip
+
+
+def layer_norm(x, gain, eps, out, delta=None, rows=None, update_x=True) -> None:
+    """v = x[s] (+ delta[s]) with s = rows[r] or r, x fp32 [T, n] receiving v when something was added and `update_x`;
+    out[r] = (v - mean) / sqrt(mean((v - mean)^2) + eps) * gain, gain fp32 [n]; delta [T, n] of out's dtype or None."""
+    _check(x, "x", F32, (None, None))
+    T, n = x.shape
+    _check(gain, "gain", F32, (n,))
+    n_out = T
+    if rows is not None:
+        _check(rows, "rows", I32, (None,))
+        n_out = rows.shape[0]
+        if update_x and delta is not None:
+            raise KernelError("layer_norm: the stream is updated whole, not by rows")
+    _check(out, "out", (F32, BF16), (n_out, n))
+    if delta is not None:
+        _check(delta, "delta", out.dtype, (T, n))
+    call("as_layer_norm", _ptr(x), _ptr(delta), _ptr(gain), float(eps), _ptr(rows), _ptr(out), _DT[out.dtype], n_out, n,
          int(bool(update_x)), _stream())  # fmt: skip
+
+
+def token_gate(z, table, ids, out) -> None:
+    """out[t] = gelu(z[t]) * table[ids[t]] (the tanh form of gelu): z, out [T, dim], table [vocab, dim], ids int32 [T]."""
+    _check(z, "z", (F32, BF16), (None, None))
+    T, dim = z.shape
+    _check(table, "table", z.dtype, (None, dim))
+    _check(ids, "ids", I32, (T,))
+    _check(out, "out", z.dtype, (T, dim))
+    call("as_token_gate", _ptr(z), _ptr(table), _ptr(ids), _DT[z.dtype], _ptr(out), dim, T, _stream())
 
 
 def poly_norm(z, coef, eps, out) -> None:
@@ -1156,13 +1194,16 @@ def head_norm_store(proj, q_off, k_off, v_off, num_heads, num_kv_heads, dim, vdi
          _ptr(cos_sin), R, _stream())  # fmt: skip
 
 
+WHOLE_NORM_MANY = 128  # tokens from which on a norm over whole projections is a pass of its own
+
+
 def whole_norm_store(proj, q_off, k_off, v_off, num_heads, num_kv_heads, dim, vdim, slots, q_out, k_pages, v_pages,
                      store_kv=True, biases=None, gains=None, eps: float = 0.0, cos_sin=None, v_keep=None,
                      v_mode: str = "none", lam: float = 0.0, maps: int = 1) -> None:  # fmt: skip
     """`head_norm_store` for heads that are normed over their whole projection.  biases: (q [H dim], k [KV dim], v [KV
     vdim]) fp32, added to the projection's output first, or None.  gains: (q [H dim], k [KV dim]) fp32: queries and keys
-    are divided by the root mean square over ALL their heads (eps inside the root) and multiplied by the gains; None: no
-    norm.  cos_sin: the rotation (after the norm), as in `head_norm_store`.  v_mode "keep": the values (bias added) are
+    are divided by the root mean square over ALL their heads (eps inside the root) and multiplied by the gains (k None: the
+    queries alone, without keys to store); None: no norm.  cos_sin: the rotation (after the norm), as in `head_norm_store`.  v_mode "keep": the values (bias added) are
     also written to v_keep fp32 [T, KV vdim]; "mix": (1 - lam) v + lam v_keep[t] is stored instead of v.
     maps > 1: every head has that many queries and keys over the same values.  num_heads counts the queries (heads x
     maps, `dim` / maps wide each in proj), dim is all of a head's keys side by side, and a query is laid out at its map's
@@ -1175,10 +1216,10 @@ def whole_norm_store(proj, q_off, k_off, v_off, num_heads, num_kv_heads, dim, vd
     if maps < 1 or dim % maps or H % maps or (maps > 1 and (gains is not None or cos_sin is not None)):
         raise KernelError(f"whole_norm_store: {maps} maps of {dim} coordinates in all, {H} queries, no norm and no rotation")
     if Dp < max(dim, vdim) or q_off < 0 or q_off + H * (dim // maps) > ld or \
-            ((store_kv or gains is not None or v_mode != "none") and
+            ((store_kv or (gains is not None and gains[1] is not None) or v_mode != "none") and
              (min(k_off, v_off) < 0 or k_off + KV * dim > ld or v_off + KV * vdim > ld)):  # fmt: skip
         raise KernelError("whole_norm_store: heads lie outside the projection's columns or the padded head width")
-    qb = kb = vb = qw = kw = None
+    qb = kb = vb = qw = kw = inverse = None
     if biases is not None:
         qb, kb, vb = biases
         for name, t, n in (("q bias", qb, H * (dim // maps)), ("k bias", kb, KV * dim), ("v bias", vb, KV * vdim)):
@@ -1187,7 +1228,10 @@ def whole_norm_store(proj, q_off, k_off, v_off, num_heads, num_kv_heads, dim, vd
     if gains is not None:
         qw, kw = gains
         _check(qw, "q gain", F32, (H * dim,))
-        _check(kw, "k gain", F32, (KV * dim,))
+        if kw is not None or store_kv:
+            _check(kw, "k gain", F32, (KV * dim,))
+        if T >= WHOLE_NORM_MANY:  # many tokens: the root mean squares first, then 16 bytes of a head a thread
+            inverse = torch.empty((T, 2), dtype=F32, device=proj.device)
     bs = 1
     if store_kv:
         _check(slots, "slots", I32, (T,))
@@ -1206,7 +1250,7 @@ def whole_norm_store(proj, q_off, k_off, v_off, num_heads, num_kv_heads, dim, vd
     if modes[v_mode]:
         _check(v_keep, "v_keep", F32, (T, KV * vdim))
     call("as_whole_norm_store", _ptr(proj), _DT[proj.dtype], ld, q_off, k_off, v_off, H, KV, dim, vdim, Dp, _ptr(qb),
-         _ptr(kb), _ptr(vb), _ptr(qw), _ptr(kw), float(eps), _ptr(cos_sin), R, _ptr(v_keep) if modes[v_mode] else 0,
+         _ptr(kb), _ptr(vb), _ptr(qw), _ptr(kw), float(eps), _ptr(inverse), _ptr(cos_sin), R, _ptr(v_keep) if modes[v_mode] else 0,
          modes[v_mode], float(lam), _ptr(slots) if store_kv else 0, _ptr(q_out), _ptr(k_pages) if store_kv else 0,
          _ptr(v_pages) if store_kv else 0, bs, int(bool(store_kv)), int(maps), T, _stream())  # fmt: skip
 
@@ -1445,9 +1489,9 @@ def attn_headmix(q, k_pages, v_pages, items, tile: int, positions, tok_row, bloc
          Dout, bs, float(scale), int(window), int(keep_first), _stream())  # fmt: skip
 
 
-def sigmoid_gate_heads(heads, vdim, gate, gate_off, scale, out, out_off) -> None:
+def sigmoid_gate_heads(heads, vdim, gate, gate_off, scale, out, out_off, per_head: bool = False) -> None:
     """out[t, out_off + h * vdim + j] = scale * sigmoid(gate[t, gate_off + h * vdim + j]) * heads[t, h, j], j < vdim;
-    gate None: scale * heads, laid side by side."""
+    gate None: scale * heads, laid side by side; per_head: one number a head, gate[t, gate_off + h]."""
     _check(heads, "heads", (F32, BF16), (None, None, None))
     T, H, Dp = heads.shape
     _check(out, "out", heads.dtype, (T, None))
@@ -1455,12 +1499,12 @@ def sigmoid_gate_heads(heads, vdim, gate, gate_off, scale, out, out_off) -> None
     if gate is not None:
         _check(gate, "gate", heads.dtype, (T, None))
         ld_gate = gate.shape[1]
-        if gate_off < 0 or gate_off + H * vdim > ld_gate:
+        if gate_off < 0 or gate_off + (H if per_head else H * vdim) > ld_gate:
             raise KernelError("sigmoid_gate_heads: columns outside the gate")
     if vdim > Dp or out_off < 0 or out_off + H * vdim > out.shape[1]:
         raise KernelError("sigmoid_gate_heads: columns outside the output")
     call("as_sigmoid_gate_heads", _ptr(heads), _DT[heads.dtype], H, vdim, Dp, _ptr(gate), ld_gate, gate_off,
-         float(scale), _ptr(out), out.shape[1], out_off, T, _stream())  # fmt: skip
+         int(bool(per_head)), float(scale), _ptr(out), out.shape[1], out_off, T, _stream())  # fmt: skip
 
 
 # ---- mixers with a fixed-size state --------------------------------------------------------------------
@@ -2078,6 +2122,89 @@ def decay_finish(o, groups: int, eps, gain, proj, g_off, gate_activation, out) -
          ACTIVATIONS[gate_activation], _ptr(out), T, _stream())  # fmt: skip
 
 
+# ---- a state space per head -----------------------------------------------------------------------------------------
+
+STATE_SPACE_MAX_STATE, STATE_SPACE_CHUNKS_MAX_STATE = 512, 128  # widest state: token by token; in chunks and in decode steps
+STATE_SPACE_KERNELS = {"scan": 0, "step": 1, "chunks": 2}
+STATE_SPACE_FILL = 3  # workgroups per compute unit up to which long rows are cut into segments
+STATE_SPACE_MIN_SEGMENT = 96  # tokens
+
+
+def _state_space_segments(longest: int, num_rows: int, workgroups: int) -> int:
+    """Tokens of a segment for rows of up to `longest` tokens, a row or segment being `workgroups` workgroups (0: rows stay
+    whole): enough segments that they fill the GPU, since a row alone is a chain of chunks."""
+    want = STATE_SPACE_FILL * compute_units() // max(1, workgroups * num_rows)
+    if want < 2 or longest < 2 * STATE_SPACE_MIN_SEGMENT:
+        return 0
+    return max(STATE_SPACE_MIN_SEGMENT, _up32(-(-longest // want)))
+
+
+def state_space(xbc, num_heads, groups, state_dim, vdim, proj, step_off, dt_bias, a_log, skip, state, step_rows, out, writes=True,
+                longest: int = 0, kernel: str = None, seg_len: int = None) -> None:  # fmt: skip
+    """Per head h and token, in the order of a row's tokens, with dt = softplus(proj[:, step_off + h] + dt_bias[h]):
+    S = exp(-exp(a_log[h]) dt) S + dt B x^T,  out = S^T C + skip[h] x.
+    xbc fp32 [T, heads * vdim + 2 groups * state_dim] laid out [x | B | C], head h reading group h // (heads / groups); proj
+    [T, ld] of either type; dt_bias, a_log, skip fp32 [heads]; state fp32 [slots, heads, state_dim, vdim]; out fp32 [T, heads *
+    vdim].  kernel: "scan" (token by token, states of up to STATE_SPACE_MAX_STATE), "step" (every row ONE token, the state
+    moved in whole lines: values in fours) or "chunks" (32 tokens at a time on the matrix cores in fp32), the last two for
+    states of up to STATE_SPACE_CHUNKS_MAX_STATE; None: by what the step and the sizes allow.  longest: the longest row's
+    tokens, if the caller knows it: long rows are then cut into segments that run at once; seg_len: tokens of a segment (a
+    multiple of 32; 0: rows stay whole), None: chosen here.  Cuts change results by rounding only."""
+    _check(xbc, "xbc", F32, (None, None))
+    T, channels = xbc.shape
+    H, G, N, E = num_heads, groups, state_dim, vdim
+    if min(H, G, N, E) < 1 or H % G or channels != H * E + 2 * G * N:
+        raise KernelError(f"state_space: {channels} channels are not {H} x {E} + 2 x {G} x {N}, or the heads do not divide")
+    _check(proj, "proj", (F32, BF16), (T, None))
+    if kernel is None:
+        if N > STATE_SPACE_CHUNKS_MAX_STATE:
+            kernel = "scan"
+        elif step_rows[0] is None:
+            kernel = "step" if E % 4 == 0 else "scan"
+        else:
+            kernel = "chunks"
+    if kernel not in STATE_SPACE_KERNELS:
+        raise KernelError(f"state_space: kernel {kernel!r} (one of {sorted(STATE_SPACE_KERNELS)})")
+    most = STATE_SPACE_MAX_STATE if kernel == "scan" else STATE_SPACE_CHUNKS_MAX_STATE
+    if N > most or (kernel == "step" and E % 4) or step_off < 0 or step_off + H > proj.shape[1]:
+        raise KernelError(f"state_space ({kernel}): a state of {N} x {E}, steps at column {step_off} of {proj.shape[1]}")
+    for name, t in (("dt_bias", dt_bias), ("a_log", a_log), ("skip", skip)):
+        _check(t, name, F32, (H,))
+    _check(state, "state", F32, (None, H, N, E))
+    _check(out, "out", F32, (T, H * E))
+    R = _check_rows(step_rows, T)
+    _, row_first, row_len, row_start, row_slots = step_rows
+    seg_state = seg_decay = None
+    segments = 0
+    if kernel != "chunks":
+        seg_len = 0
+    elif seg_len is None:
+        seg_len = _state_space_segments(longest, R, G * -(-(H // G) * -(-E // 32) // 4))
+    if seg_len:
+        if seg_len < 0 or seg_len % 32:
+            raise KernelError(f"state_space: segments of {seg_len} tokens (a multiple of 32)")
+        segments = T // seg_len + R
+        seg_state = torch.empty((segments + 1, H, -(-E // 32), -(-N // 32), 1024), dtype=F32, device=xbc.device)
+        seg_decay = torch.empty((segments + 1, H), dtype=F32, device=xbc.device)
+    call("as_state_space", _ptr(xbc), channels, H, G, N, E, _ptr(proj), _DT[proj.dtype], proj.shape[1], step_off, _ptr(dt_bias),
+         _ptr(a_log), _ptr(skip), _ptr(state), _ptr(row_first), _ptr(row_len), _ptr(row_start), _ptr(row_slots), R, _ptr(out),
+         int(bool(writes)), STATE_SPACE_KERNELS[kernel], int(seg_len), segments, _ptr(seg_state), _ptr(seg_decay), _stream())  # fmt: skip
+
+
+def gated_group_norm(y, groups: int, eps, gain, proj, z_off, out) -> None:
+    """v = y * silu(z), y fp32 [T, n], z the columns z_off .. of proj [T, ld]; out = v with every one of `groups` equal parts
+    divided by its own root mean square (eps inside the root), times gain fp32 [n]; out [T, n] of proj's dtype."""
+    _check(y, "y", F32, (None, None))
+    T, n = y.shape
+    _check(proj, "proj", (F32, BF16), (T, None))
+    _check(gain, "gain", F32, (n,))
+    _check(out, "out", proj.dtype, (T, n))
+    if groups < 1 or n % groups or z_off < 0 or z_off + n > proj.shape[1]:
+        raise KernelError(f"gated_group_norm: {groups} groups of {n}, gate at column {z_off} of {proj.shape[1]}")
+    call("as_gated_group_norm", _ptr(y), _ptr(proj), _DT[proj.dtype], proj.shape[1], z_off, _ptr(gain), float(eps), n, groups, _ptr(out),
+         T, _stream())  # fmt: skip
+
+
 # ---- attention through a latent ---------------------------------------------------------------------------------
 
 
@@ -2161,14 +2288,14 @@ WIDE_ATTEND_MAX_WIDTH = 2048
 
 
 def wide_attend(q, k_pages, v_pages, positions, tok_row, block_tables, out, scale, max_context, window=0, keep_first=0,
-                softcap=0.0, sink=False) -> None:  # fmt: skip
+                softcap=0.0, sink=False, chunk=0) -> None:  # fmt: skip
     """Causal attention of every token's heads q [T, H, width] over kv heads of any width up to
     WIDE_ATTEND_MAX_WIDTH (k_pages [pages, KV, bs, width], v_pages [pages, KV, width, bs]): for pages wider than the
     paged attention kernels' heads.  positions, tok_row [T] int32 (tok_row None: token t is row t); out like q.
-    window, keep_first, softcap, sink, and out in fp32 for bfloat16 heads: as for `attn_single_query`."""
+    window, keep_first, softcap, sink, chunk, and out in fp32 for bfloat16 heads: as for `attn_single_query`."""
     _check(q, "q", (F32, BF16), (None, None, None))
     T, H, width = q.shape
-    sight = _sight(window, keep_first, softcap, sink, q, out)
+    sight = _sight(window, keep_first, chunk, softcap, sink, q, out)
     _check(k_pages, "k_pages", q.dtype, (None, None, None, width))
     pages, KV, bs, _ = k_pages.shape
     _check(v_pages, "v_pages", q.dtype, (pages, KV, width, bs))

@@ -134,8 +134,8 @@ class Attention(Mixer):
 def attend(q, out, step, cache, scale: float, window: int, split, wide: bool = False, **sight) -> None:
     """Attention of a step's queries q [T, H, D] over the pages of `cache` (which hold the step's own keys
     already) into out [T, H, D]; `split`: the (short, tile) under which the step sorted its rows for this.
-    wide: the heads exceed the paged kernels' (the plain kernel for any width runs).  sight: keep_first, softcap, sink as
-    `ops.attn_single_query` takes them."""
+    wide: the heads exceed the paged kernels' (the plain kernel for any width runs).  sight: keep_first, softcap, sink,
+    chunk as `ops.attn_single_query` takes them."""
     if wide:
         ops.wide_attend(q, cache.k_pages, cache.v_pages, step.positions, None if step.decode_only else step.tok_row,
                         cache.block_tables, out, scale, step.max_context, window, **sight)  # fmt: skip

@@ -10,6 +10,7 @@ Kinds of parts:
   mixer         forward(h, step, cache) -> [T, hidden]; says which cache (or caches) it
                 wants through `cache_request()`
   feed_forward  forward(h, step) -> [T, hidden]
+  token_input   forward(x, step) -> [T, hidden]: what a layer makes of the tokens' own rows of a table
   arrangement   runs one layer: owns the order of norms, mixer, feed-forward and
                 residual sums
 
@@ -214,7 +215,8 @@ class FeedForward(Part):
 class Norm(Part):
     takes_split_sums = False  # whether `forward` accepts a SplitSums as `delta`
     takes_gated_delta = False  # whether `forward` accepts a GatedDelta as `delta`
-    takes_normed_delta = False  # whether `forward` accepts a NormedDelta as `delta`
+    takes_normed_delta = False  # whether `forward` accepts a NormedDelta as `delta`, and may be a NormedDelta's norm
+    centred = False  # whether a row's mean comes off before it is divided by its root mean square
 
     def forward(self, x, delta=None, rows=None, update_residual=True) -> torch.Tensor:
         raise NotImplementedError
@@ -270,7 +272,7 @@ class Arrangement:
 
 # ---- registries --------------------------------------------------------------------
 
-_REGISTRIES: dict = {"norm": {}, "position": {}, "mixer": {}, "feed_forward": {}, "arrangement": {}}
+_REGISTRIES: dict = {"norm": {}, "position": {}, "mixer": {}, "feed_forward": {}, "token_input": {}, "arrangement": {}}
 
 
 def register(family: str, kind: str, builder: Callable, replace: bool = False) -> None:
@@ -292,5 +294,6 @@ def build(family: str, spec: Any, env: BuildEnv):
 
 def _load_builtin() -> None:
     from atomserve_amd.parts import (  # noqa: F401
-        attention, block, experts, joined, latent_attention, linear_attention, mlp, norm, recurrent, rope,
+        attention, block, experts, joined, latent_attention, linear_attention, mlp, norm, recurrent, rope, state_space,
+        token_input,
     )

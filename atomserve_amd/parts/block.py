@@ -7,7 +7,8 @@
               results of all layers before it
 "streams_prenorm": "prenorm" over several residual streams that a sublayer reads as one weighted sum and writes
               through a mixing matrix
-"sandwich":   x += post1(mixer(norm1(x)));  x += post2(ffn(norm2(x))): a norm before and after every sublayer
+"sandwich":   x += post1(mixer(norm1(x)));  x += post2(ffn(norm2(x))): a norm before and after every sublayer; then, where
+              the layer has one, x += norm(token_input(x))
 
 The residual stream `x` is fp32 in both precisions.  A part's output is not added at
 once: it travels as the pending `delta` to the next norm, whose kernel adds it into
@@ -33,6 +34,7 @@ from atomserve_amd.parts.base import (
     build,
     register,
 )
+from atomserve_amd.parts.norm import settle_normed
 
 
 class PreNormBlock(Arrangement):
@@ -158,7 +160,8 @@ register("arrangement", "gated_prenorm", GatedPreNormBlock)
 class SandwichBlock(Arrangement):
     """x += post1(mixer(norm1(x)));  x += post2(ffn(norm2(x)))  (spec.ffn None: the mixer alone).  A sublayer's output
     travels as a pending `NormedDelta` to the kernel of the next norm, which norms it, adds it into the fp32 stream and
-    norms the sum in one pass over the row."""
+    norms the sum in one pass over the row.  With spec.token_input the layer ends with x += norm(token_input(x)), which reads
+    the stream as it is: the kernel that adds the last sublayer's output leaves it in the compute dtype."""
 
     def __init__(self, spec, env):
         super().__init__(spec, env)
@@ -170,7 +173,11 @@ class SandwichBlock(Arrangement):
             self.ffn_norm = build("norm", spec.ffn_norm, env)
             self.ffn = build("feed_forward", spec.ffn, env)
             self.ffn_post_norm = build("norm", spec.ffn_post_norm, env)
-        for norm in (self.mixer_norm, self.mixer_post_norm, self.ffn_norm, self.ffn_post_norm):
+        self.token_input = self.token_norm = None
+        if spec.token_input is not None:
+            self.token_input = build("token_input", spec.token_input, env)
+            self.token_norm = build("norm", spec.token_input.norm, env)
+        for norm in (self.mixer_norm, self.mixer_post_norm, self.ffn_norm, self.ffn_post_norm, self.token_norm):
             if norm is not None and not norm.takes_normed_delta:
                 raise ValueError(f"a norm of kind {norm.spec.kind!r} does not norm outputs on their way into the stream")
 
@@ -178,6 +185,8 @@ class SandwichBlock(Arrangement):
         parts = {"mixer_norm": self.mixer_norm, "mixer": self.mixer, "mixer_post_norm": self.mixer_post_norm}
         if self.ffn is not None:
             parts.update(ffn_norm=self.ffn_norm, ffn=self.ffn, ffn_post_norm=self.ffn_post_norm)
+        if self.token_input is not None:
+            parts.update(token_input=self.token_input, token_norm=self.token_norm)
         return parts
 
     def first_norm(self):
@@ -188,9 +197,13 @@ class SandwichBlock(Arrangement):
             raise ValueError("a layer of this arrangement takes an output that is still to be normed, or none")
         y = self.mixer.forward(self.mixer_norm.forward(x, delta), step, cache)
         delta = self.pending(y, self.mixer_post_norm)
-        if self.ffn is None:
+        if self.ffn is not None:
+            delta = self.pending(self.ffn.forward(self.ffn_norm.forward(x, delta), step), self.ffn_post_norm)
+        if self.token_input is None:
             return delta
-        return self.pending(self.ffn.forward(self.ffn_norm.forward(x, delta), step), self.ffn_post_norm)
+        stream = torch.empty(x.shape, dtype=self.env.dtype, device=x.device)
+        settle_normed(x, delta, stream)
+        return self.pending(self.token_input.forward(stream, step), self.token_norm)
 
     @staticmethod
     def pending(y, norm) -> NormedDelta:

@@ -8,8 +8,8 @@ or, where every core's output is normed before the sum, an output product a core
 kernel that adds into the stream (`NormedSum`).  A core has no products of its own: it says how many columns of `proj` it reads (`in_rows`) and how many of `act` it
 fills (`out_cols`), declares its small tensors, asks for what it keeps between steps, and computes.  One core alone with
 the scale 1 is an ordinary mixer.  Cores here: a grouped-query softmax attention with the options a design may combine
-(biases, a norm over the whole of q and of k, a rotation, values mixed with an earlier layer's, an output gate, a window
-that may keep the first tokens, capped scores, a sink, two attention maps of which the difference is taken, another
+(biases, a norm over the whole of q and of k, a rotation, values mixed with an earlier layer's, an output gate per
+coordinate or per head, a window that may keep the first tokens, chunks, capped scores, a sink, two attention maps of which the difference is taken, another
 layer's keys and values), a matrix memory with exponential gates, and a linear attention with decays per key channel.
 """
 
@@ -25,8 +25,8 @@ from atomserve_amd.parts.recurrent import _step_rows
 
 class SoftmaxCore:
     """Causal grouped-query softmax attention over a paged cache.  Columns read: q [H maps key_dim], k [G maps key_dim], v [G
-    value_dim] (k and v unless spec.own_kv is off) and, with spec.out_gate, the gate's logits [H value_dim]; columns
-    filled: the heads [H value_dim].
+    value_dim] (k and v unless spec.own_kv is off) and, with spec.out_gate, the gate's logits [H value_dim] (spec.head_gate:
+    [H]); columns filled: the heads [H value_dim].
 
     With two maps a kv head's pages hold both its keys side by side over one value, and every query is as wide as both with
     zeros in the other map's place: the attention kernels read keys and values once for both maps.
@@ -46,10 +46,14 @@ class SoftmaxCore:
             raise ValueError(f"values are mixed as 'none', 'first' or 'later', not {s.value_mix!r}")
         if s.maps not in (1, 2):
             raise ValueError(f"an attention has one map or takes the difference of two, not {s.maps}")
-        if s.maps == 2 and (s.whole_norm_eps > 0 or s.position is not None or s.out_gate or not s.difference_eps > 0):
+        if s.out_gate and s.head_gate:
+            raise ValueError("an attention's output gate has a number per coordinate or one per head, not both")
+        if s.chunk < 0 or (s.chunk and s.window):
+            raise ValueError("a query sees a window or its own chunk, not both")
+        if s.maps == 2 and (s.whole_norm_eps > 0 or s.position is not None or s.out_gate or s.head_gate or not s.difference_eps > 0):
             raise ValueError("two maps go with neither a norm of q and k, a rotation nor an output gate; their difference is normed")
-        if not s.own_kv and (s.whole_norm_eps > 0 or s.value_mix != "none"):
-            raise ValueError("a core that reads another layer's keys and values neither norms nor mixes its own")
+        if not s.own_kv and s.value_mix != "none":
+            raise ValueError("a core that reads another layer's keys and values has none of its own to mix")
         chunk = 4 if env.dtype == torch.float32 else 8
         self.keys = s.maps * s.key_dim  # all of a kv head's keys side by side
         widest = max(self.keys, s.value_dim)
@@ -68,7 +72,7 @@ class SoftmaxCore:
         H, G, D, E = s.num_heads, s.num_kv_heads, self.keys, s.value_dim
         kv = 1 if s.own_kv else 0
         self.q_off, self.k_off, self.v_off, self.gate_off = 0, H * D, H * D + kv * G * D, H * D + kv * (G * D + G * E)
-        self.in_rows = self.gate_off + (H * E if s.out_gate else 0)
+        self.in_rows = self.gate_off + (H * E if s.out_gate else H if s.head_gate else 0)
         self.out_cols = H * E
         self.biases = self.gains = None
         self.lam = self.map_lambda = 0.0
@@ -87,7 +91,9 @@ class SoftmaxCore:
         if s.maps == 2:
             decls.update({name: WeightDecl((s.key_dim,), "vector") for name in ("lq1", "lk1", "lq2", "lk2")})
         if s.whole_norm_eps > 0:
-            decls.update({"q_norm": WeightDecl((H * D,), "vector"), "k_norm": WeightDecl((G * D,), "vector")})
+            decls["q_norm"] = WeightDecl((H * D,), "vector")
+            if s.own_kv:
+                decls["k_norm"] = WeightDecl((G * D,), "vector")
         if s.value_mix == "later":
             decls["value_mix"] = WeightDecl((), "vector")
         return decls
@@ -122,13 +128,14 @@ class SoftmaxCore:
             dots = [float((f32[a].double() * f32[b].double()).sum()) for a, b in (("lq1", "lk1"), ("lq2", "lk2"))]
             self.map_lambda = math.exp(dots[0]) - math.exp(dots[1]) + s.difference
         if s.whole_norm_eps > 0:
-            self.gains = (ordered(f32["q_norm"], 0), ordered(f32["k_norm"], nq))
+            self.gains = (ordered(f32["q_norm"], 0), ordered(f32["k_norm"], nq) if s.own_kv else None)
         if s.value_mix == "later":
             self.lam = float(f32["value_mix"])
 
     def cache_request(self) -> dict:
         s = self.spec
-        window = s.window if s.cache_window is None else s.cache_window
+        window = s.window or s.chunk  # what a chunk shows lies within a window of its length
+        window = window if s.cache_window is None else s.cache_window
         keep = s.keep_first if s.cache_keep_first is None else s.cache_keep_first
         return {"pages": PagedCacheRequest(s.num_kv_heads, self.head_width, window, keep if window > 0 else 0)}
 
@@ -152,8 +159,9 @@ class SoftmaxCore:
                              pages.slots, q, pages.k_pages, pages.v_pages, store_kv=pages.writes and s.own_kv,
                              biases=self.biases, gains=self.gains, eps=s.whole_norm_eps, cos_sin=cos_sin, v_keep=v_keep,
                              v_mode=v_mode, lam=self.lam, maps=s.maps)  # fmt: skip
-        how = dict(wide=self.wide, keep_first=s.keep_first, softcap=s.softcap, sink=s.sink)
-        if s.maps == 1 and not s.out_gate and scale == 1.0 and Dp == s.value_dim and out_off == 0 and act.shape[1] == self.out_cols:
+        how = dict(wide=self.wide, keep_first=s.keep_first, softcap=s.softcap, sink=s.sink, chunk=s.chunk)
+        gated = s.out_gate or s.head_gate
+        if s.maps == 1 and not gated and scale == 1.0 and Dp == s.value_dim and out_off == 0 and act.shape[1] == self.out_cols:
             # the core alone, its heads as wide as they are laid out: the attention writes the output product's input itself
             attend(q, act.view(T, H, Dp), step, pages, s.scale, s.window, (SHORT_ROW, TILE_Q), **how)
             return
@@ -163,7 +171,8 @@ class SoftmaxCore:
         if s.maps == 2:
             ops.map_difference(heads, s.value_dim, self.map_lambda, s.difference_eps, scale * (1.0 - s.difference), act, out_off)
             return
-        ops.sigmoid_gate_heads(heads, s.value_dim, proj if s.out_gate else None, off + self.gate_off, scale, act, out_off)
+        ops.sigmoid_gate_heads(heads, s.value_dim, proj if gated else None, off + self.gate_off, scale, act, out_off,
+                               per_head=s.head_gate)  # fmt: skip
 
 
 class MatrixMemoryCore:

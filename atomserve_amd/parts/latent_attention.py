@@ -3,7 +3,8 @@
     c_q = norm(W_dq h);   q_h = W_uq c_q = [q_h plain (head_dim) | q_h turned (rot_dim)]      (or q_h = W_q h)
     [c raw | k_r raw] = W_dkv h;   c = norm(c raw)  [kv_rank];   k_r turned by the position  [rot_dim], one for all heads
     k_h(j) = U_h c_j,   v_h(j) = V_h c_j;   score_h(i, j) = scale (q_h plain(i) . k_h(j) + q_h turned(i) . k_r(j)),  j <= i
-    out = W_o ([softmax_j(score_h) v_h]_h * sigmoid(W_g h))      (or without the gate; j may be bounded by a window)
+    out = W_o ([softmax_j(score_h) v_h]_h * sigmoid(W_g h))      (or without the gate; j may be bounded by a window, and the
+                                                                  softmax's denominator may hold e^(sink_h) too)
 
 Only c and k_r are cached: a page holds one kv head whose keys are [c | k_r] and whose values are c.  Because
 q_h . (U_h c) = (U_h^T q_h) . c and sum_j p_j V_h c_j = V_h sum_j p_j c_j, the attention itself is the package's paged
@@ -67,12 +68,15 @@ class LatentAttention(Mixer):
             decls["uq.weight"] = WeightDecl((s.num_heads * (s.head_dim + s.rot_dim), s.q_rank))
         if s.own_latent:
             decls["kv_norm.weight"] = WeightDecl((s.kv_rank,), role="vector")
+        if s.head_sinks:
+            decls["sink"] = WeightDecl((s.num_heads,), role="vector")
         return decls
 
     def bind(self, tensors: dict) -> None:
         self.kv_norm_weight = self.q_norm_weight = self.uq_weight = self.uq = None
         super().bind(tensors)
         s = self.spec
+        self.sinks = self.sink.float().contiguous() if s.head_sinks else False  # exact: what a file holds in 16 bits widens
         if self.position is not None and self.position.pairs == "neighbours":
             self.order_turned_rows()
         if self.q_norm_weight is not None:
@@ -130,7 +134,7 @@ class LatentAttention(Mixer):
         qa = torch.empty((T, H, self.width), dtype=env.dtype, device=dev)
         ops.latent_q_absorb(q, self.uk_weight, H, D, R, s.kv_rank, cos_sin, qa, uk_t=self.uk_t)
         heads = torch.empty((T, H, self.width), dtype=env.dtype, device=dev)
-        attend(qa, heads, step, cache, s.scale, s.window, self.row_split(), wide=self.wide, keep_first=s.keep_first)
+        attend(qa, heads, step, cache, s.scale, s.window, self.row_split(), wide=self.wide, keep_first=s.keep_first, sink=self.sinks)
         act = torch.empty((T, H * E), dtype=env.dtype, device=dev)
         ops.latent_v_expand(heads, self.uv_t, s.kv_rank, proj if s.out_gate else None, self.g_off, act, uv=self.uv_weight)
         y = torch.empty((T, s.hidden_size), dtype=env.dtype, device=dev)

@@ -1,4 +1,4 @@
-"""RMSNorm: weight * x / sqrt(mean(x^2) + eps), accumulated in fp32 and rounded once
+"""Norms.  RMSNorm: weight * x / sqrt(mean(x^2) + eps), accumulated in fp32 and rounded once
 (reference atomserve/model.py:125-139).  The residual sum that precedes a norm in a
 pre-norm layer is fused into the same kernel: the fp32 residual stream `x` receives
 `delta` and the normalised result is written in the compute dtype."""
@@ -25,6 +25,16 @@ class PendingRMSNorm(PendingNorm):
             return False
         ops.gemm_scaled(self.scaled, self.ssq, self.norm.spec.eps, w, out, gated=True)
         return True
+
+
+def settle_normed(x, delta: NormedDelta, out, norm=None, rows=None, update_residual=True) -> None:
+    """x += the delta's norm of its output; out = `norm` of x, or without a norm x itself in out's dtype: one kernel.  Both
+    norms are of this package's kinds over a row's root mean square, taken as it is or with the mean off first (`centred`)."""
+    y, post = delta.y, delta.norm
+    pair = dict(other=y.ys[1], gains=y.gains, biases=y.biases, eps_in=y.eps) if isinstance(y, NormedSum) else {}
+    ops.post_norm_add(x, y.ys[0] if pair else y, post.gain_f32, post.spec.eps, None if norm is None else norm.gain_f32,
+                      0.0 if norm is None else norm.spec.eps, out, rows, update_residual, centre_post=post.centred,
+                      centre=norm is not None and norm.centred, **pair)  # fmt: skip
 
 
 class RMSNorm(Norm):
@@ -65,22 +75,12 @@ class RMSNorm(Norm):
         elif isinstance(delta, DeltaSum):
             self.with_sibling(None, x, delta, rows, update_residual, out)
         elif isinstance(delta, NormedDelta):
-            self.after_normed(x, delta, rows, update_residual, out)
+            settle_normed(x, delta, out, self, rows, update_residual)
         elif isinstance(delta, SplitSums):
             ops.rmsnorm(x, self.weight, self.spec.eps, out, rows=rows, update_x=update_residual, split_sums=delta.sums)
         else:
             ops.rmsnorm(x, self.weight, self.spec.eps, out, delta=delta, rows=rows, update_x=update_residual)
         return out
-
-    def after_normed(self, x, delta, rows, update_residual, out) -> None:
-        """x += the delta's norm of its output; out = this norm of x: one kernel."""
-        s = self.spec
-        y, post = delta.y, delta.norm
-        if isinstance(y, NormedSum):
-            ops.post_norm_add(x, y.ys[0], post.gain_f32, post.spec.eps, self.gain_f32, s.eps, out, rows, update_residual,
-                              other=y.ys[1], gains=y.gains, biases=y.biases, eps_in=y.eps)  # fmt: skip
-        else:
-            ops.post_norm_add(x, y, post.gain_f32, post.spec.eps, self.gain_f32, s.eps, out, rows, update_residual)
 
     def stream(self, x) -> torch.Tensor:
         """The norm of the fp32 rows x as a new fp32 tensor: for a norm whose result is itself a residual stream
@@ -109,6 +109,36 @@ class RMSNorm(Norm):
 
 
 register("norm", "rmsnorm", RMSNorm)
+
+
+class LayerNorm(Norm):
+    """(x - mean) / sqrt(mean((x - mean)^2) + eps) * gain: a row's mean comes off before it is divided by what is then its
+    root mean square; no bias.  fp32 until the one rounding at the end."""
+
+    capturable = True
+    takes_normed_delta = True
+    centred = True
+
+    def weight_decls(self) -> dict:
+        return {"weight": WeightDecl((self.spec.size,), role="vector")}
+
+    def bind(self, tensors: dict) -> None:
+        super().bind(tensors)
+        self.gain_f32 = self.weight.float().contiguous()  # exact: what a file holds in 16 bits widens
+
+    def forward(self, x, delta=None, rows=None, update_residual=True) -> torch.Tensor:
+        if delta is not None and not isinstance(delta, (torch.Tensor, NormedDelta)):
+            raise ValueError("a layer norm adds a plain pending output, or one still to be normed, into the stream")
+        n_out = x.shape[0] if rows is None else rows.shape[0]
+        out = torch.empty((n_out, self.spec.size), dtype=self.env.dtype, device=x.device)
+        if isinstance(delta, NormedDelta):
+            settle_normed(x, delta, out, self, rows, update_residual)
+        else:
+            ops.layer_norm(x, self.gain_f32, self.spec.eps, out, delta, rows, update_residual)
+        return out
+
+
+register("norm", "layernorm", LayerNorm)
 
 
 class GroupedRMSNorm(Norm):

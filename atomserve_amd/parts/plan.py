@@ -13,7 +13,8 @@ from typing import Any, Optional
 @dataclass(frozen=True)
 class NormSpec:
     """kind "rmsnorm": x / sqrt(mean(x^2) + eps) * gain.  kind "grouped_rmsnorm": the row is cut into `groups` equal
-    consecutive parts, each divided by its own root mean square, the whole times the gain."""
+    consecutive parts, each divided by its own root mean square, the whole times the gain.  kind "layernorm": (x - mean) /
+    sqrt(mean((x - mean)^2) + eps) * gain, without a bias."""
 
     kind: str
     size: int
@@ -95,7 +96,8 @@ class LatentAttentionSpec:
     per head, `head_dim` coordinates that are not rotated and then `rot_dim` that are.  score = scale (q . k of both
     parts).  The concatenated heads [heads, value_dim], with `out_gate` times sigmoid of a projection of the input, go
     through the output projection.  own_latent False: the layer has no projection to the latent; it reads the pages of
-    the run that its run names as its cache.  window, keep_first: as for `SoftmaxCoreSpec`."""
+    the run that its run names as its cache.  window, keep_first: as for `SoftmaxCoreSpec`.  head_sinks: the softmax's
+    denominator has one more score per head, a number of the layer's own that is not scaled and has no value."""
 
     kind: str  # "latent_attention"
     hidden_size: int
@@ -112,6 +114,7 @@ class LatentAttentionSpec:
     out_gate: bool = True
     window: int = 0
     keep_first: int = 0
+    head_sinks: bool = False
 
 
 @dataclass(frozen=True)
@@ -232,15 +235,17 @@ class SoftmaxCoreSpec:
     whole projection (all heads at once) with gains of that size.  position: a rotation of q and k, or None.
     value_mix "first": the core's values (of the step's tokens) are kept for later layers under `value_mix_key`;
     "later": its values become (1 - lam) v + lam v_first before they are cached, lam a scalar of its own.
-    out_gate: the concatenated heads are multiplied by sigmoid of a projection of the input.
+    out_gate: the concatenated heads are multiplied by sigmoid of a projection of the input; head_gate: every head by one
+    number, sigmoid of a projection with a row per head.
     window > 0: a query at p sees the keys p - window + 1 .. p and those of the sequence's first `keep_first` tokens.
+    chunk > 0 (without a window): it sees those of its own chunk up to p, chunks of `chunk` positions counted from 0.
     softcap > 0: a score s counts as softcap tanh(s / softcap).  sink: one more score of 0 in the softmax's denominator,
     without a value.
     maps 2: differential attention: a head has two queries and two keys of `key_dim` over one value, laid out [map 1, map
     2], and its output is a1 - lambda a2 over its root mean square (difference_eps), times (1 - difference), with lambda =
     exp(lq1 . lk1) - exp(lq2 . lk2) + difference.
     own_kv False: no projections to keys and values; the core reads the pages of the run that its run names as its
-    cache.  cache_window, cache_keep_first: what those pages keep where another run reads them too and sees more than
+    cache (whole_norm_eps then norms its queries alone).  cache_window, cache_keep_first: what those pages keep where another run reads them too and sees more than
     this core (None: what this core sees)."""
 
     kind: str  # "softmax_core"
@@ -265,6 +270,8 @@ class SoftmaxCoreSpec:
     own_kv: bool = True
     cache_window: Optional[int] = None
     cache_keep_first: Optional[int] = None
+    head_gate: bool = False
+    chunk: int = 0
 
 
 @dataclass(frozen=True)
@@ -332,6 +339,36 @@ class ChannelDeltaRuleSpec:
     gate_rank: int
     out_norm_eps: float
     unit_eps: float = 1e-6
+
+
+@dataclass(frozen=True)
+class StateSpaceSpec:
+    """A state space per head (Mamba-2): S = exp(-exp(A_h) dt) S + dt B x^T, y = S^T C + D_h x with dt = softplus(step + bias_h).
+    x [num_heads, value_dim], B and C [groups, state_dim] (head h reads group h // (num_heads / groups)) pass one short
+    convolution with a bias and silu; y times silu(z) is RMS-normed in `norm_groups` equal parts with a gain of its own.  z,
+    x, B, C and the steps are rows of one projection of the input, in this order."""
+
+    kind: str  # "state_space"
+    hidden_size: int
+    num_heads: int
+    value_dim: int
+    state_dim: int
+    groups: int
+    conv: ShortConvSpec
+    norm_groups: int
+    out_norm_eps: float
+
+
+@dataclass(frozen=True)
+class TokenInputSpec:
+    """What a layer adds to the stream x for the tokens themselves: norm(P (gelu(G x) * e)), e [dim] the token's row of a
+    table [vocab_size, dim] of the layer's own, G [dim, hidden], P [hidden, dim], gelu in its tanh form."""
+
+    kind: str  # "gated_table"
+    hidden_size: int
+    dim: int
+    vocab_size: int
+    norm: NormSpec
 
 
 @dataclass(frozen=True)
@@ -425,7 +462,7 @@ class BlockSpec:
     x_s + residual_scale c[t] y with a, M, c of its own; the layer marked streams_last leaves their sum as the
     stream.  streams 0: one stream with a = M = c = 1, that is x += residual_scale y.
     arrangement "sandwich": x += mixer_post_norm(mixer(mixer_norm(x))); x += ffn_post_norm(ffn(ffn_norm(x))) (ffn None:
-    the mixer alone)."""
+    the mixer alone); then, with token_input, x += token_input.norm(...) as `TokenInputSpec` says."""
 
     arrangement: str
     mixer: Any
@@ -441,6 +478,7 @@ class BlockSpec:
     streams_last: bool = False
     mixer_post_norm: Optional[NormSpec] = None
     ffn_post_norm: Optional[NormSpec] = None
+    token_input: Optional[TokenInputSpec] = None
 
 
 @dataclass(frozen=True)

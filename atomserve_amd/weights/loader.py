@@ -1,7 +1,7 @@
 """Weights from safetensors, by tensor name (reference atomserve/loader.py:63-148).
 
 The architecture says how each tensor of the plan is made of checkpoint tensors: a name,
-names stacked along the rows (q, k, v into one projection, gate and up into one), rows cut
+names stacked along the rows (q, k, v into one projection, gate and up into one), rows or columns cut
 out of a fused tensor, a transposed matrix, or matrices stacked along a new axis (`Take`,
 `Stack`); the parts say what shape and role each plan tensor has.  Everything that is wrong with a checkpoint is collected
 and reported in one error: missing tensors, unexpected ones, wrong shapes.
@@ -30,14 +30,21 @@ class Take:
 
     transpose: a matrix stored [in, out] is turned to this package's [out, in] first.
     rows: (start, stop) keeps these rows only (after the transposition), for a checkpoint that
-    stores several plan tensors fused in one."""
+    stores several plan tensors fused in one.
+    cols: (start, stop) keeps these columns only of the stored matrix (before the transposition)."""
 
     name: str
     transpose: bool = False
     rows: Optional[tuple] = None
+    cols: Optional[tuple] = None
 
     def shape_from(self, stored: tuple) -> tuple:
         shape = tuple(stored)
+        if self.cols is not None:
+            start, stop = self.cols
+            if len(shape) != 2 or not 0 <= start < stop <= shape[1]:
+                raise ValueError(f"{self.name}: columns {start}:{stop} lie outside its shape {shape}")
+            shape = (shape[0], stop - start)
         if self.transpose:
             if len(shape) != 2:
                 raise ValueError(f"{self.name}: only a matrix can be transposed, this has shape {shape}")
@@ -49,7 +56,9 @@ class Take:
             shape = (stop - start, *shape[1:])
         return shape
 
-    def apply(self, tensor):
+    def fetch(self, source):
+        """The piece out of a source of tensors; of a matrix of which columns are kept, only those are read."""
+        tensor = source.get(self.name) if self.cols is None else source.get_columns(self.name, *self.cols)
         if self.transpose:
             tensor = tensor.t()
         if self.rows is not None:
@@ -112,6 +121,9 @@ class DictSource:
     def get(self, name):
         return self.tensors[name]
 
+    def get_columns(self, name, start, stop):
+        return self.tensors[name][:, start:stop]
+
 
 def missing_shards(model_dir: str) -> list:
     """The weight files that a folder's index (model.safetensors.index.json, if it has one) names and the
@@ -154,6 +166,9 @@ class SafetensorsSource:
 
     def get(self, name):
         return self.where[name].get_tensor(name)
+
+    def get_columns(self, name, start, stop):
+        return self.where[name].get_slice(name)[:, start:stop]
 
 
 def checkpoint_shapes_of(model_dir: str):
@@ -228,7 +243,7 @@ def bind_checkpoint(model, arch, config, source, where: str = "") -> dict:
         recipe = recipes[target]
         stored = source.dtype(recipe.parts[0].name)
         dtype = _storage_dtype(decl.role, stored, env.dtype)
-        pieces = [t.apply(source.get(t.name)).to(device=env.device, dtype=dtype) for t in recipe.parts]
+        pieces = [t.fetch(source).to(device=env.device, dtype=dtype) for t in recipe.parts]
         if recipe.new_axis:
             made = torch.stack(pieces, dim=0)
         else:
