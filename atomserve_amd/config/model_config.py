@@ -1323,7 +1323,7 @@ class TokuvikConfig:
             hidden_size=int(raw["width"]),
             norm_eps=float(_need(raw["norm"], "eps", "norm.")),
             layers=tuple(layers),
-            side_dim=int(_need(side, "dim", "token_side.")) if side else 0,
+            side_dim=int(_need(side, "dim", "token_side.")) if side is not None else 0,
         )
         cfg.validate()
         return cfg

@@ -286,7 +286,8 @@ __global__ __launch_bounds__(256) void token_gate_kernel(const T* __restrict__ z
   if (at >= total) return;
   const int t = at / dim, i = at - t * dim;
   const float v = to_f32(z[at]);
-  const float g = 0.5f * v * (1.0f + tanhf(0.7978845608028654f * (v + 0.044715f * v * v * v)));
+  // (1 + tanh u) / 2 = 1 / (1 + e^(-2u)): nothing cancels for negative u, whose small gates a norm may enlarge again
+  const float g = v / (1.0f + expf(-2.0f * 0.7978845608028654f * (v + 0.044715f * v * v * v)));
   out[at] = from_f32<T>(g * to_f32(table[(size_t)ids[t] * dim + i]));
 }
 

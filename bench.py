@@ -7,6 +7,7 @@
     python bench.py --design mumizen [--widths 1024,2048,4096]   (Mumizen layers beside Qwen3 layers of equal size)
     python bench.py --design natatar [--widths 1024,2048,4096]   (Natatar layers beside Dozusun and Qwen3 layers of equal size)
     python bench.py --design teberax [--widths 1024,2048,4096]   (Teberax layers beside Mumizen and Qwen3 layers of equal size)
+    python bench.py --design tokuvik [--widths 1024,2048,4096]   (Tokuvik layers beside Teberax and Qwen3 layers of equal size)
 
 A step is one decode step of the engine (scheduler, one pass over the GPU, sampling).
 Prints ONE JSON line: decoded tokens per second at batch 8 with 2,048-token contexts,
@@ -79,7 +80,7 @@ def parse_args():
                         "(half of them share their first 32), chunks of 512, 128 tokens decoded each, through the "
                         "scheduler from submission to the last token")  # fmt: skip
     p.add_argument("--chunk-budget", type=int, default=512, help="token budget of a step in the mixed workload")
-    p.add_argument("--design", choices=["qwen3", "dozusun", "koravik", "mumizen", "natatar", "teberax"], default="qwen3",
+    p.add_argument("--design", choices=["qwen3", "dozusun", "koravik", "mumizen", "natatar", "teberax", "tokuvik"], default="qwen3",
                    help="dozusun: prefill and decode throughput of random-weight Dozusun layers (an attention beside a "
                         "gated linear recurrence, gated delta rules, dense and table-routed feed-forwards) at a few "
                         "widths, beside Qwen3 layers of the same width, heads, depth and vocabulary; koravik: the same "
@@ -87,7 +88,8 @@ def parse_args():
                         "shared one, gated residual sums, a stretch of layers run twice); mumizen: the same for Mumizen "
                         "layers (linear attentions with fixed decays, attention through a cached latent, gated "
                         "feed-forwards with limits, dense and routed, an average over all layers' results); natatar: the same for "
-                        "Natatar layers, Dozusun's beside them; teberax: the same for Teberax layers, Mumizen's beside them")  # fmt: skip
+                        "Natatar layers, Dozusun's beside them; teberax: the same for Teberax layers, Mumizen's beside them; tokuvik: the same for Tokuvik "
+                        "layers, Teberax's beside them")  # fmt: skip
     p.add_argument("--widths", default="1024,2048,4096", help="stream widths of the designs")
     p.add_argument("--profile", action="store_true",
                    help="also split the host's time of a decode step into schedule / pack / launch / sample / wait / "
@@ -299,13 +301,35 @@ def teberax_config(width: int, layers: int, vocab: int):
                                     "logit_softcap": 25.0, "layers": made})  # fmt: skip
 
 
+def tokuvik_config(width: int, layers: int, vocab: int):
+    """Layers as a model of this design of that width would have them: attention with heads of 128, a kv head to four query
+    heads and chunks of 1,024, every second one reading the keys of the one before; attention through a latent of 192 (queries
+    through a latent of half the width, heads of 128); state spaces twice the width in heads of 64 over 128 rows, one group of
+    B and C, four taps and a norm in one group; gated feed-forwards three times the width; token inputs 128 wide; the kinds of
+    layers in turn: attention, state space, latent, state space, and the same with the attention reading the first one's keys."""
+    from atomserve_amd.config.model_config import TokuvikConfig
+
+    heads = width // 128
+    attention = {"heads": heads, "kv_heads": max(1, heads // 4), "dim": 128, "vdim": 128, "scale": 128**-0.5, "mask": {"size": 1024}}
+    latent = {"heads": heads, "dim": 128, "vdim": 128, "q_rank": width // 2, "kv_rank": 192, "scale": 128**-0.5}
+    space = {"heads": width // 32, "vdim": 64, "state": 128, "groups": 1, "conv": 4, "norm_groups": 1}
+    made = []
+    for i in range(layers):
+        kind, mixer = [("attention", attention), ("mamba2", space), ("latent_attention", latent), ("mamba2", space)][i % 4]
+        if kind == "attention" and i % 8 == 4:
+            mixer = dict(attention, kv_from=i - 4)
+        made.append({"type": kind, "mixer": mixer, "mlp": {"kind": "dense", "ff": 3 * width}})
+    return TokuvikConfig.from_dict({"architecture": "Tokuvik", "vocab": vocab, "width": width, "norm": {"eps": 1e-6},
+                                    "token_side": {"dim": 128}, "layers": made})  # fmt: skip
+
+
 def design_comparison(args) -> dict:
     """Prefill of --prefill-tokens tokens and decode at batch 1 and --batch with --context tokens of context, for
     the layers of --design and for Qwen3 layers of equal width, heads, depth and vocabulary; random weights, the
     engine's own entry point (scheduler, captured decode steps, sampling)."""
     design = args.design
     make = {"dozusun": dozusun_config, "koravik": koravik_config, "mumizen": mumizen_config, "natatar": natatar_config,
-            "teberax": teberax_config}[design]  # fmt: skip
+            "teberax": teberax_config, "tokuvik": tokuvik_config}[design]  # fmt: skip
     import torch
 
     from atomserve_amd.config import EngineConfig, Qwen3Config
@@ -376,6 +400,8 @@ def design_comparison(args) -> dict:
             sizes[str(width)]["dozusun"] = measure(dozusun_config(width, layers, vocab))
         if design == "teberax":  # its closest relative: a linear attention with decays, a latent that layers share, dense and routed
             sizes[str(width)]["mumizen"] = measure(mumizen_config(width, layers, vocab))
+        if design == "tokuvik":  # its closest relative: norms around sublayers, a state per head, a latent, another layer's keys
+            sizes[str(width)]["teberax"] = measure(teberax_config(width, layers, vocab))
         print(f"width {width}: {json.dumps(sizes[str(width)])}", file=sys.stderr, flush=True)
     widest = sizes[max(sizes, key=int)]
     return {
