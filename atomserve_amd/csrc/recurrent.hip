@@ -9,6 +9,7 @@
 // again); a portion of a prompt goes on from what the portion before left.  State tables are fp32
 // [slots, ...]; a row's state is written back only when `writes`.
 #include "common.h"
+#include "rows.h"
 
 #define CONV_MAX_TAPS 8
 
@@ -47,6 +48,73 @@ __global__ void short_conv_kernel(const T* __restrict__ in, int ld, int col0, in
   }
   if (bias) acc += to_f32(bias[c]);
   out[(size_t)t * C + c] = act == 1 ? siluf_(acc) : acc;
+}
+
+// The same for many tokens, four neighbouring channels of CONV_TOKENS tokens in a row a thread: every input is read once for all
+// its taps.  fp32 weights; C, col0 and ld multiples of four.
+#define CONV_TOKENS 8
+template <typename T> __device__ __forceinline__ float quick_silu(float z) { return siluf_(z); }
+template <> __device__ __forceinline__ float quick_silu<bf16>(float z) { return z * __builtin_amdgcn_rcpf(1.0f + __expf(-z)); }
+
+template <typename T, int TAPS>
+__global__ __launch_bounds__(256) void short_conv_tile_kernel(const T* __restrict__ in, int ld, int col0, int C,
+                                                              const float* __restrict__ in_bias, const float* __restrict__ w,
+                                                              const float* __restrict__ bias, int act,
+                                                              const float* __restrict__ history, const int* __restrict__ tok_row,
+                                                              const int* __restrict__ row_first, const int* __restrict__ row_start,
+                                                              const int* __restrict__ row_slots, float* __restrict__ out,
+                                                              int num_tokens) {
+  const int c = (blockIdx.y * 256 + threadIdx.x) * 4, t0 = blockIdx.x * CONV_TOKENS;
+  if (c >= C) return;
+  const int here = min(CONV_TOKENS, num_tokens - t0);
+  const T* column = in + col0 + c;
+  float now[CONV_TOKENS][4], wt[TAPS * 4], ib[4] = {0.f, 0.f, 0.f, 0.f}, b[4] = {0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+  for (int i = 0; i < CONV_TOKENS; ++i) load_vec<4>(column + (size_t)(t0 + min(i, here - 1)) * ld, now[i]);
+#pragma unroll
+  for (int i = 0; i < TAPS; ++i) load_vec<4>(w + (size_t)c * TAPS + 4 * i, wt + 4 * i);  // channel c + k, tap i: at k TAPS + i
+  if (in_bias) load_vec<4>(in_bias + c, ib);
+  if (bias) load_vec<4>(bias + c, b);
+  float seen[TAPS][4];  // the last TAPS - 1 inputs, then the token's own
+  int row = -1;
+#pragma unroll
+  for (int i = 0; i < CONV_TOKENS; ++i) {
+    if (i < here) {
+      const int t = t0 + i, r = tok_row[t];
+      if (r != row) {  // a row's first token of this tile: what came before it in the row, or waits in the request's history
+        row = r;
+        const int first = row_first[r], j = t - first;
+        const bool carried = row_start[r] > 0 && row_slots[r] >= 0;
+        const float* old = history + (size_t)(carried ? row_slots[r] : 0) * (TAPS - 1) * C + c;
+#pragma unroll
+        for (int p = 0; p < TAPS - 1; ++p) {
+          const int src = j - (TAPS - 1 - p);
+#pragma unroll
+          for (int k = 0; k < 4; ++k) seen[p][k] = 0.f;
+          if (src >= 0) {
+            load_vec<4>(column + (size_t)(first + src) * ld, seen[p]);
+#pragma unroll
+            for (int k = 0; k < 4; ++k) seen[p][k] += ib[k];
+          } else if (carried) {
+            load_vec<4>(old + (size_t)(TAPS - 1 + src) * C, seen[p]);
+          }
+        }
+      }
+      float v[4];
+#pragma unroll
+      for (int k = 0; k < 4; ++k) {
+        seen[TAPS - 1][k] = now[i][k] + ib[k];
+        float acc = 0.f;
+#pragma unroll
+        for (int p = 0; p < TAPS; ++p) acc = fmaf(wt[k * TAPS + p], seen[p][k], acc);
+        acc += b[k];
+        v[k] = act == 1 ? quick_silu<T>(acc) : acc;
+#pragma unroll
+        for (int p = 0; p < TAPS - 1; ++p) seen[p][k] = seen[p + 1][k];
+      }
+      store_vec<4>(out + (size_t)t * C + c, v);
+    }
+  }
 }
 
 // After the convolution: the history of every row moves on by the row's tokens.
@@ -102,6 +170,12 @@ extern "C" int as_short_conv(const void* in, int dtype, int ld, int col0, int C,
   const int threads = C >= 256 ? 256 : 64;
   dim3 grid(num_tokens, (C + threads - 1) / threads), rows_grid(num_rows, (C + threads - 1) / threads);
   if (grid.y > 65535) return AS_BAD_SHAPE;
+  const bool tiled = tok_row && num_tokens >= 64 && w_dtype == DT_F32 && taps >= 2 && taps <= 4 && ((C | col0 | ld) & 3) == 0;
+  dim3 tiles((num_tokens + CONV_TOKENS - 1) / CONV_TOKENS, (C / 4 + 255) / 256);
+#define TILE(T, TAPSV)                                                                                            \
+  short_conv_tile_kernel<T, TAPSV><<<tiles, 256, 0, stream>>>((const T*)in, ld, col0, C, (const float*)in_bias, (const float*)w, \
+                                                              (const float*)bias, act, history, tok_row, row_first, row_start,   \
+                                                              row_slots, out, num_tokens)
 #define LAUNCH(T, W)                                                                                              \
   do {                                                                                                            \
     if (!tok_row && num_rows == num_tokens) { /* every row one token */                                           \
@@ -110,9 +184,15 @@ extern "C" int as_short_conv(const void* in, int dtype, int ld, int col0, int C,
                                                                  row_start, row_slots, writes, out);             \
       break;                                                                                                      \
     }                                                                                                             \
-    short_conv_kernel<T, W><<<grid, threads, 0, stream>>>((const T*)in, ld, col0, C, (const W*)in_bias,          \
-                                                          (const W*)w, (const W*)bias, taps, act, history,       \
-                                                          tok_row, row_first, row_start, row_slots, out);        \
+    if (tiled) {                                                                                                  \
+      if (taps == 2) TILE(T, 2);                                                                                  \
+      else if (taps == 3) TILE(T, 3);                                                                             \
+      else TILE(T, 4);                                                                                            \
+    } else {                                                                                                      \
+      short_conv_kernel<T, W><<<grid, threads, 0, stream>>>((const T*)in, ld, col0, C, (const W*)in_bias,        \
+                                                            (const W*)w, (const W*)bias, taps, act, history,     \
+                                                            tok_row, row_first, row_start, row_slots, out);      \
+    }                                                                                                             \
     if (writes && taps > 1)                                                                                       \
       conv_history_kernel<T, W><<<rows_grid, threads, 0, stream>>>((const T*)in, ld, col0, C, (const W*)in_bias, \
                                                                    taps, history, row_first, row_len, row_start, \
@@ -122,6 +202,7 @@ extern "C" int as_short_conv(const void* in, int dtype, int ld, int col0, int C,
   else if (dtype == DT_BF16 && w_dtype == DT_BF16) LAUNCH(bf16, bf16);
   else if (dtype == DT_BF16 && w_dtype == DT_F32) LAUNCH(bf16, float);
   else return AS_BAD_DTYPE;
+#undef TILE
 #undef LAUNCH
   return launch_status();
 }

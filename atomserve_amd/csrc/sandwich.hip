@@ -38,6 +38,15 @@ __global__ __launch_bounds__(1024) void post_norm_add_kernel(float* __restrict__
   const size_t s = rows ? (size_t)rows[r] : (size_t)r;
   float d[CH][VEC], v[CH][VEC];
   float sums[PAIR ? 2 : 1] = {};
+  // few rows (one piece a thread): everything the row needs is asked for at once, not a reduction later each
+  constexpr bool EARLY = CH == 1 && !PAIR;
+  [[maybe_unused]] float x_early[VEC], post_early[VEC], gain_early[VEC];
+  if constexpr (EARLY) {
+    const int i = min((int)threadIdx.x * VEC, n - VEC);
+    load_vec<VEC>(x + s * n + i, x_early);
+    load_vec<VEC>(p.post + i, post_early);
+    if (p.gain) load_vec<VEC>(p.gain + i, gain_early);
+  }
 #pragma unroll
   for (int c = 0; c < CH; ++c) {
     const int i = (c * blockDim.x + threadIdx.x) * VEC;
@@ -113,8 +122,13 @@ __global__ __launch_bounds__(1024) void post_norm_add_kernel(float* __restrict__
     const int i = (c * blockDim.x + threadIdx.x) * VEC;
     if (i >= n) continue;
     float g[VEC];
-    load_vec<VEC>(p.post + i, g);
-    load_vec<VEC>(x + s * n + i, v[c]);
+    if constexpr (EARLY) {
+#pragma unroll
+      for (int k = 0; k < VEC; ++k) { g[k] = post_early[k]; v[c][k] = x_early[k]; }
+    } else {
+      load_vec<VEC>(p.post + i, g);
+      load_vec<VEC>(x + s * n + i, v[c]);
+    }
 #pragma unroll
     for (int k = 0; k < VEC; ++k) {
       v[c][k] += d[c][k] * inv_post * g[k];
@@ -133,7 +147,12 @@ __global__ __launch_bounds__(1024) void post_norm_add_kernel(float* __restrict__
     const int i = (c * blockDim.x + threadIdx.x) * VEC;
     if (i >= n) continue;
     float g[VEC];
-    load_vec<VEC>(p.gain + i, g);
+    if constexpr (EARLY) {
+#pragma unroll
+      for (int k = 0; k < VEC; ++k) g[k] = gain_early[k];
+    } else {
+      load_vec<VEC>(p.gain + i, g);
+    }
 #pragma unroll
     for (int k = 0; k < VEC; ++k) v[c][k] *= inv * g[k];
     store_vec<VEC>(out + (size_t)r * n + i, v[c]);
@@ -279,6 +298,11 @@ extern "C" int as_layer_norm(float* x, const void* y, const float* gain, float e
 
 // ---- the token's own input, gated ------------------------------------------------------------------------------------
 // out[t, i] = gelu_tanh(z[t, i]) * table[ids[t], i], i < dim; z, table and out of one type, everything between fp32.
+__device__ __forceinline__ float gelu_tanh(float v) {
+  // (1 + tanh u) / 2 = 1 / (1 + e^(-2u)): nothing cancels for negative u, whose small gates a norm may enlarge again
+  return v / (1.0f + expf(-2.0f * 0.7978845608028654f * (v + 0.044715f * v * v * v)));
+}
+
 template <typename T>
 __global__ __launch_bounds__(256) void token_gate_kernel(const T* __restrict__ z, const T* __restrict__ table,
                                                          const int* __restrict__ ids, T* __restrict__ out, int dim, int total) {
@@ -286,9 +310,7 @@ __global__ __launch_bounds__(256) void token_gate_kernel(const T* __restrict__ z
   if (at >= total) return;
   const int t = at / dim, i = at - t * dim;
   const float v = to_f32(z[at]);
-  // (1 + tanh u) / 2 = 1 / (1 + e^(-2u)): nothing cancels for negative u, whose small gates a norm may enlarge again
-  const float g = v / (1.0f + expf(-2.0f * 0.7978845608028654f * (v + 0.044715f * v * v * v)));
-  out[at] = from_f32<T>(g * to_f32(table[(size_t)ids[t] * dim + i]));
+  out[at] = from_f32<T>(gelu_tanh(v) * to_f32(table[(size_t)ids[t] * dim + i]));
 }
 
 extern "C" int as_token_gate(const void* z, const void* table, const int* ids, int dtype, void* out, int dim, int num_tokens,
@@ -301,6 +323,67 @@ extern "C" int as_token_gate(const void* z, const void* table, const int* ids, i
   else if (dtype == DT_BF16)
     token_gate_kernel<bf16><<<blocks, 256, 0, stream>>>((const bf16*)z, (const bf16*)table, ids, (bf16*)out, dim, total);
   else return AS_BAD_DTYPE;
+  return launch_status();
+}
+
+// The product before it too, for up to 16 rows of bfloat16: out[t, i] = gelu_tanh(x[t] . w[i]) * table[ids[t], i].  A workgroup of
+// four waves per output i: their lanes share K, 16 bytes at a time, and hold a sum for every row; a wave's sums meet by lane swaps,
+// each swap halving the rows that a lane still sums, so that a lane ends with one row's sum, and the four waves' in LDS.
+template <int ROWS>
+__global__ __launch_bounds__(256) void token_product_kernel(const bf16* __restrict__ x, const bf16* __restrict__ w,
+                                                            const bf16* __restrict__ table, const int* __restrict__ ids,
+                                                            bf16* __restrict__ out, int K, int dim, int num_tokens) {
+  typedef __bf16 bf16x8 __attribute__((ext_vector_type(8)));
+  __shared__ float sums[4][ROWS];
+  const int i = blockIdx.x, lane = threadIdx.x & (WAVE - 1), wave = threadIdx.x / WAVE, row = threadIdx.x;
+  // what the gate needs is asked for first
+  const float e = row < num_tokens ? (float)table[(size_t)ids[row] * dim + i] : 0.f;
+  float acc[ROWS];
+#pragma unroll
+  for (int t = 0; t < ROWS; ++t) acc[t] = 0.f;
+#pragma unroll 2
+  for (int k = threadIdx.x * 8; k < K; k += 4 * WAVE * 8) {
+    const bf16x8 wv = *reinterpret_cast<const bf16x8*>(w + (size_t)i * K + k);
+#pragma unroll
+    for (int t = 0; t < ROWS; ++t) {
+      const bf16x8 xv = *reinterpret_cast<const bf16x8*>(x + (size_t)min(t, num_tokens - 1) * K + k);
+#pragma unroll
+      for (int j = 0; j < 8; ++j) acc[t] = fmaf((float)wv[j], (float)xv[j], acc[t]);
+    }
+  }
+#pragma unroll
+  for (int n = ROWS, off = WAVE / 2; n > 1; n /= 2, off /= 2) {
+#pragma unroll
+    for (int t = 0; t < n / 2; ++t) {
+      const float keep = lane & off ? acc[t + n / 2] : acc[t], give = lane & off ? acc[t] : acc[t + n / 2];
+      acc[t] = keep + __shfl_xor(give, off, WAVE);
+    }
+  }
+  constexpr int LANES = WAVE / ROWS;  // lanes that still hold parts of one row's sum: row lane / LANES
+  float z = acc[0];
+#pragma unroll
+  for (int off = LANES / 2; off > 0; off /= 2) z += __shfl_xor(z, off, WAVE);
+  if (lane % LANES == 0) sums[wave][lane / LANES] = z;
+  __syncthreads();
+  if (row < num_tokens) {
+    z = (sums[0][row] + sums[1][row]) + (sums[2][row] + sums[3][row]);
+    out[(size_t)row * dim + i] = (bf16)(gelu_tanh(z) * e);
+  }
+}
+
+extern "C" int as_token_product(const void* x, const void* w, const void* table, const int* ids, void* out, int K, int dim,
+                                int num_tokens, hipStream_t stream) {
+  if (num_tokens <= 0) return AS_OK;
+  if (K <= 0 || K % 8 || dim <= 0 || num_tokens > 16) return AS_BAD_SHAPE;
+#define LAUNCH(R)                                                                                                          \
+  token_product_kernel<R><<<dim, 256, 0, stream>>>((const bf16*)x, (const bf16*)w, (const bf16*)table, ids, (bf16*)out, \
+                                                             K, dim, num_tokens)
+  if (num_tokens == 1) LAUNCH(1);
+  else if (num_tokens == 2) LAUNCH(2);
+  else if (num_tokens <= 4) LAUNCH(4);
+  else if (num_tokens <= 8) LAUNCH(8);
+  else LAUNCH(16);
+#undef LAUNCH
   return launch_status();
 }
 

@@ -192,7 +192,7 @@ __device__ __forceinline__ bool find_segment(const Space& s, int z, int* row, in
 }
 
 template <typename T, int NT, bool STATES>
-__global__ __launch_bounds__(256) void state_space_chunk_kernel(Space s) {
+__global__ __launch_bounds__(256, 2) void state_space_chunk_kernel(Space s) {
   constexpr int NP = 32 * NT, LD = NP + 4, QUADS = NP / 4, EACH = CHUNK * QUADS / 256;
   __shared__ __attribute__((aligned(16))) float Bs[CHUNK][LD];
   __shared__ __attribute__((aligned(16))) float Cs[STATES ? 1 : CHUNK][LD];
@@ -220,60 +220,60 @@ __global__ __launch_bounds__(256) void state_space_chunk_kernel(Space s) {
   };
   floatx16 S[NT];
   const bool resume = !STATES && count == 1 && slot >= 0 && s.row_start[r] > 0;
+  if (!STATES && count > 1 && working) {
 #pragma unroll
-  for (int tile = 0; tile < NT; ++tile)
+    for (int tile = 0; tile < NT; ++tile)
 #pragma unroll
-    for (int i = 0; i < 16; ++i) {
-      const int n = 32 * tile + acc_row(i, half);
-      float v = 0.f;
-      if (!STATES && count > 1) v = working ? s.seg_state[segment_state(blockIdx.z, tile, i)] : 0.f;
-      else if (resume && e_live && n < s.N) v = s.state[state_at(s, slot, h, n, e0 + col)];
-      S[tile][i] = v;
-    }
-  // What a chunk reads is asked for a chunk ahead and waits in registers.
+      for (int i = 0; i < 16; ++i) S[tile][i] = s.seg_state[segment_state(blockIdx.z, tile, i)];
+  } else if (resume) {
+    const float* kept = s.state + state_at(s, slot, h, 0, 0);
+#pragma unroll
+    for (int tile = 0; tile < NT; ++tile)
+#pragma unroll
+      for (int i = 0; i < 16; ++i) {  // a place beyond the state is read as the nearest one within and counts as zero
+        const int n = 32 * tile + acc_row(i, half);
+        const float v = kept[min(n, s.N - 1) * s.E + min(e0 + col, s.E - 1)];
+        S[tile][i] = e_live && n < s.N ? v : 0.f;
+      }
+  } else {
+#pragma unroll
+    for (int tile = 0; tile < NT; ++tile)
+#pragma unroll
+      for (int i = 0; i < 16; ++i) S[tile][i] = 0.f;
+  }
+  // B and C of a chunk are asked for while the chunk before updates the state and wait in registers; x while this chunk's first
+  // products run.
   float4 b_next[EACH], c_next[STATES ? 1 : EACH];
-  float x_next[16], step_next = 0.f;
+  float step_next = 0.f;
   auto fetch = [&](int c0) {
     const int n = min(CHUNK, len - c0);
+    const float* base = s.xbc + (size_t)(first + c0) * s.channels;  // one address for the wave, 32-bit offsets for its lanes
 #pragma unroll
     for (int it = 0; it < EACH; ++it) {
       const int idx = tid + 256 * it, t = idx / QUADS, d = (idx % QUADS) * 4;
-      float4 b = make_float4(0.f, 0.f, 0.f, 0.f), c = b;
-      if (t < n && d < s.N) {
-        const float* row = s.xbc + (size_t)(first + c0 + t) * s.channels;
-        if (whole) {
-          b = *reinterpret_cast<const float4*>(row + b_off + d);
-          if (!STATES) c = *reinterpret_cast<const float4*>(row + c_off + d);
-        } else {
-          b.x = row[b_off + d];
-          if (d + 1 < s.N) b.y = row[b_off + d + 1];
-          if (d + 2 < s.N) b.z = row[b_off + d + 2];
-          if (d + 3 < s.N) b.w = row[b_off + d + 3];
-          if (!STATES) {
-            c.x = row[c_off + d];
-            if (d + 1 < s.N) c.y = row[c_off + d + 1];
-            if (d + 2 < s.N) c.z = row[c_off + d + 2];
-            if (d + 3 < s.N) c.w = row[c_off + d + 3];
-          }
-        }
+      float4 b, c = make_float4(0.f, 0.f, 0.f, 0.f);
+      if (whole) {
+        const int at = min(t, n - 1) * s.channels + min(d, s.N - 4);
+        b = *reinterpret_cast<const float4*>(base + b_off + at);
+        if (!STATES) c = *reinterpret_cast<const float4*>(base + c_off + at);
+      } else {
+        const int at = min(t, n - 1) * s.channels, d1 = min(d, s.N - 1), d2 = min(d + 1, s.N - 1), d3 = min(d + 2, s.N - 1), d4 = min(d + 3, s.N - 1);
+        b = make_float4(base[b_off + at + d1], base[b_off + at + d2], base[b_off + at + d3], base[b_off + at + d4]);
+        if (!STATES) c = make_float4(base[c_off + at + d1], base[c_off + at + d2], base[c_off + at + d3], base[c_off + at + d4]);
+        if (d + 1 >= s.N) b.y = c.y = 0.f;
+        if (d + 2 >= s.N) b.z = c.z = 0.f;
+        if (d + 3 >= s.N) b.w = c.w = 0.f;
       }
+      if (t >= n || d >= s.N) b = c = make_float4(0.f, 0.f, 0.f, 0.f);
       b_next[it] = b;
       if (!STATES) c_next[STATES ? 0 : it] = c;
     }
-#pragma unroll
-    for (int i = 0; i < 16; ++i) {
-      const int j = acc_row(i, half);
-      x_next[i] = j < n && e_live ? s.xbc[(size_t)(first + c0 + j) * s.channels + h * s.E + e0 + col] : 0.f;
-    }
-    step_next = col < n ? to_f32(((const T*)s.proj)[(size_t)(first + c0 + col) * s.ld + s.step_off + h]) : 0.f;
+    step_next = to_f32(((const T*)s.proj)[(size_t)(first + c0 + min(col, n - 1)) * s.ld + s.step_off + h]);
   };
   double decayed = 0.0;  // STATES: the segment's whole log decay
   fetch(0);
   for (int c0 = 0; c0 < len; c0 += CHUNK) {
     const int n = min(CHUNK, len - c0);
-    float x[16];
-#pragma unroll
-    for (int i = 0; i < 16; ++i) x[i] = x_next[i];
     // this head's steps and decays: both halves of the wave do the same
     const float dt = col < n ? softplus(step_next + bias) : 0.f;
     double l = -(double)rate * (double)dt;
@@ -299,7 +299,17 @@ __global__ __launch_bounds__(256) void state_space_chunk_kernel(Space s) {
         grow[w][lane] = quick_exp<T>((float)l);
       }
     }
-    if (c0 + CHUNK < len) fetch(c0 + CHUNK);
+    float x[16];
+    {
+      const float* base = s.xbc + (size_t)(first + c0) * s.channels + h * s.E;
+      const int e = min(e0 + col, s.E - 1);
+#pragma unroll
+      for (int i = 0; i < 16; ++i) {
+        const int j = acc_row(i, half);
+        const float v = base[min(j, n - 1) * s.channels + e];
+        x[i] = j < n && e_live ? v : 0.f;
+      }
+    }
     __syncthreads();
     floatx16 y;
     if (!STATES) {
@@ -321,11 +331,12 @@ __global__ __launch_bounds__(256) void state_space_chunk_kernel(Space s) {
         for (int q = 0; q < 4; ++q)
           *reinterpret_cast<float4*>(part[STATES ? 0 : w][q][lane]) = make_float4(acc[4 * q], acc[4 * q + 1], acc[4 * q + 2], acc[4 * q + 3]);
       }
+      __builtin_amdgcn_sched_barrier(0);  // or the operands of everything that follows are asked for at once
       // meanwhile: y = e^(l_t) S^T C
 #pragma unroll
       for (int i = 0; i < 16; ++i) y[i] = 0.f;
 #pragma unroll
-      for (int tile = 0; tile < NT; ++tile)
+      for (int tile = 0; tile < NT; ++tile) {
 #pragma unroll
         for (int q = 0; q < 4; ++q) {
           const float4 c = *reinterpret_cast<const float4*>(&Cs[STATES ? 0 : col][32 * tile + 8 * q + 4 * half]);
@@ -334,6 +345,8 @@ __global__ __launch_bounds__(256) void state_space_chunk_kernel(Space s) {
           y = __builtin_amdgcn_mfma_f32_32x32x2f32(c.z, S[tile][4 * q + 2], y, 0, 0, 0);
           y = __builtin_amdgcn_mfma_f32_32x32x2f32(c.w, S[tile][4 * q + 3], y, 0, 0, 0);
         }
+        if (tile & 1) __builtin_amdgcn_sched_barrier(0);
+      }
 #pragma unroll
       for (int q = 0; q < 4; ++q) {
         const float4 f = *reinterpret_cast<const float4*>(&grow[w][8 * q + 4 * half]);
@@ -354,11 +367,13 @@ __global__ __launch_bounds__(256) void state_space_chunk_kernel(Space s) {
 #pragma unroll
       for (int i = 0; i < 16; ++i) {
         const int j = acc_row(i, half);
-        float m = j <= col ? quick_exp<T>((float)(mine - log_sum[w][j])) * step[w][j] * pairs[i] : 0.f;
-        if (j == col) m += skip;
+        float m = quick_exp<T>(fminf((float)(mine - log_sum[w][j]), 0.f)) * step[w][j] * pairs[i];
+        m = j < col ? m : j == col ? m + skip : 0.f;
         y = __builtin_amdgcn_mfma_f32_32x32x2f32(m, x[i], y, 0, 0, 0);
       }
     }
+    __builtin_amdgcn_sched_barrier(0);
+    if (c0 + CHUNK < len) fetch(c0 + CHUNK);
     const float shrink = quick_exp<T>((float)last);
 #pragma unroll
     for (int q = 0; q < 4; ++q) {
@@ -372,12 +387,18 @@ __global__ __launch_bounds__(256) void state_space_chunk_kernel(Space s) {
 #pragma unroll
       for (int i = 0; i < 16; ++i)
         S[tile] = __builtin_amdgcn_mfma_f32_32x32x2f32(Bs[acc_row(i, half)][32 * tile + col], x[i], S[tile], 0, 0, 0);
+      if (tile & 1) __builtin_amdgcn_sched_barrier(0);
     }
     if (!STATES && e_live) {
+      float* to = s.out + (size_t)(first + c0) * s.H * s.E + h * s.E + e0 + col;
+      const int ld = s.H * s.E;
+      if (n == CHUNK) {
 #pragma unroll
-      for (int i = 0; i < 16; ++i) {
-        const int t = acc_row(i, half);
-        if (t < n) s.out[(size_t)(first + c0 + t) * s.H * s.E + h * s.E + e0 + col] = y[i];
+        for (int i = 0; i < 16; ++i) to[acc_row(i, half) * ld] = y[i];
+      } else {
+#pragma unroll
+        for (int i = 0; i < 16; ++i)
+          if (acc_row(i, half) < n) to[acc_row(i, half) * ld] = y[i];
       }
     }
   }
@@ -392,12 +413,15 @@ __global__ __launch_bounds__(256) void state_space_chunk_kernel(Space s) {
     return;
   }
   if (slot >= 0 && s.writes && e_live && nth + 1 == count) {
+    float* kept = s.state + state_at(s, slot, h, 0, e0 + col);
+    int hf = half;
+    asm volatile("" : "+v"(hf));  // or the addresses of the state's first read are kept through the loop for this
 #pragma unroll
     for (int tile = 0; tile < NT; ++tile)
 #pragma unroll
       for (int i = 0; i < 16; ++i) {
-        const int n = 32 * tile + acc_row(i, half);
-        if (n < s.N) s.state[state_at(s, slot, h, n, e0 + col)] = S[tile][i];
+        const int n = 32 * tile + acc_row(i, hf);
+        if (n < s.N) kept[n * s.E] = S[tile][i];
       }
   }
 }

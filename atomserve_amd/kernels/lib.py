@@ -32,6 +32,7 @@ SIGNATURES = {
     "as_whole_norm_store": ("elementwise", [P, I, I, I, I, I, I, I, I, I, I, P, P, P, P, P, F, P, P, I, P, I, F, P, P, P, P, I, I, I, I, P]),
     "as_post_norm_add": ("sandwich", [P, P, P, I, P, P, P, P, F, P, F, P, F, I, I, P, P, I, I, I, P]),
     "as_layer_norm": ("sandwich", [P, P, P, F, P, P, I, I, I, I, P]),
+    "as_token_product": ("sandwich", [P, P, P, P, P, I, I, I, P]),
     "as_token_gate": ("sandwich", [P, P, P, I, P, I, I, P]),
     "as_poly_norm": ("sandwich", [P, I, P, F, P, I, I, P]),
     "as_map_difference": ("sandwich", [P, I, I, I, I, F, F, F, P, I, I, I, I, P]),

@@ -1114,6 +1114,28 @@ def token_gate(z, table, ids, out) -> None:
     call("as_token_gate", _ptr(z), _ptr(table), _ptr(ids), _DT[z.dtype], _ptr(out), dim, T, _stream())
 
 
+TOKEN_PRODUCT_MAX_ROWS = 16
+
+
+def gemm_token_gate(x, w, table, ids, out, choices=None) -> None:
+    """out[t] = gelu(x[t] @ w^T) * table[ids[t]]: x [T, K], w [dim, K] (or its `Streamed`), table [vocab, dim], out [T, dim].
+    Few rows in one kernel (every product's sum in fp32 until the gate), more as a product and `token_gate`."""
+    rows = _rows(w)
+    _check(x, "x", (F32, BF16), (None, None))
+    T, K = x.shape
+    dim = rows.shape[0]
+    if x.dtype == BF16 and T <= TOKEN_PRODUCT_MAX_ROWS and K % 8 == 0:
+        _check(rows, "w", BF16, (dim, K))
+        _check(table, "table", BF16, (None, dim))
+        _check(ids, "ids", I32, (T,))
+        _check(out, "out", BF16, (T, dim))
+        call("as_token_product", _ptr(x), _ptr(rows), _ptr(table), _ptr(ids), _ptr(out), K, dim, T, _stream())
+        return
+    z = torch.empty((T, dim), dtype=x.dtype, device=x.device)
+    gemm(x, w, z, choices)
+    token_gate(z, table, ids, out)
+
+
 def poly_norm(z, coef, eps, out) -> None:
     """out = a N(z) + b N(z^2) + c N(z^3) + e per row, N the division by the row's root mean square (eps inside the root);
     coef fp32 [4] = a, b, c, e."""
@@ -1194,9 +1216,6 @@ def head_norm_store(proj, q_off, k_off, v_off, num_heads, num_kv_heads, dim, vdi
          _ptr(cos_sin), R, _stream())  # fmt: skip
 
 
-WHOLE_NORM_MANY = 128  # tokens from which on a norm over whole projections is a pass of its own
-
-
 def whole_norm_store(proj, q_off, k_off, v_off, num_heads, num_kv_heads, dim, vdim, slots, q_out, k_pages, v_pages,
                      store_kv=True, biases=None, gains=None, eps: float = 0.0, cos_sin=None, v_keep=None,
                      v_mode: str = "none", lam: float = 0.0, maps: int = 1) -> None:  # fmt: skip
@@ -1230,7 +1249,8 @@ def whole_norm_store(proj, q_off, k_off, v_off, num_heads, num_kv_heads, dim, vd
         _check(qw, "q gain", F32, (H * dim,))
         if kw is not None or store_kv:
             _check(kw, "k gain", F32, (KV * dim,))
-        if T >= WHOLE_NORM_MANY:  # many tokens: the root mean squares first, then 16 bytes of a head a thread
+        if proj.dtype == BF16 and not (ld | q_off | k_off | v_off | dim | vdim | Dp) & 7:
+            # the root mean squares first, then 16 bytes of a head a thread
             inverse = torch.empty((T, 2), dtype=F32, device=proj.device)
     bs = 1
     if store_kv:
@@ -2126,8 +2146,8 @@ def decay_finish(o, groups: int, eps, gain, proj, g_off, gate_activation, out) -
 
 STATE_SPACE_MAX_STATE, STATE_SPACE_CHUNKS_MAX_STATE = 512, 128  # widest state: token by token; in chunks and in decode steps
 STATE_SPACE_KERNELS = {"scan": 0, "step": 1, "chunks": 2}
-STATE_SPACE_FILL = 3  # workgroups per compute unit up to which long rows are cut into segments
-STATE_SPACE_MIN_SEGMENT = 96  # tokens
+STATE_SPACE_FILL = 2  # workgroups per compute unit up to which long rows are cut into segments
+STATE_SPACE_MIN_SEGMENT = 64  # tokens
 
 
 def _state_space_segments(longest: int, num_rows: int, workgroups: int) -> int:

@@ -39,10 +39,8 @@ class GatedTableInput(Part):
         """x [T, hidden] in the compute dtype -> [T, hidden]."""
         s, env = self.spec, self.env
         T, dev = x.shape[0], x.device
-        z = torch.empty((T, s.dim), dtype=env.dtype, device=dev)
-        ops.gemm(x, self.gate, z, env.products)
-        g = torch.empty_like(z)
-        ops.token_gate(z, self.table, step.token_ids, g)
+        g = torch.empty((T, s.dim), dtype=env.dtype, device=dev)
+        ops.gemm_token_gate(x, self.gate, self.table, step.token_ids, g, env.products)
         y = torch.empty((T, s.hidden_size), dtype=env.dtype, device=dev)
         ops.gemm(g, self.proj, y, env.products)
         return y

@@ -984,7 +984,7 @@ def test_long_items_of_a_prompt_step_are_cut_into_pieces_and_merged(ops, H, KV, 
         part_acc = torch.full((n, H, pieces, D), float("nan"), device=DEV)
         out = torch.zeros(n, H, D, dtype=BF16, device=DEV)
         call("as_attn_prefill_mfma", q.data_ptr(), k_pages.data_ptr(), v_pages.data_ptr(), i32(tiles).data_ptr(), len(tiles),
-             tables.data_ptr(), tables.shape[1], out.data_ptr(), H, KV, D, bs, D**-0.5, window, 0, 0.0, 0, 0, query_tiles, pieces, piece_rounds,
+             tables.data_ptr(), tables.shape[1], out.data_ptr(), H, KV, D, bs, D**-0.5, window, 0, 0, 0.0, 0, 0, 0, query_tiles, pieces, piece_rounds,
              cut.data_ptr(), part_ml.data_ptr(), part_acc.data_ptr(), stream)  # fmt: skip
         said = set(cut.tolist())
         assert said <= set(range(1, pieces + 1)) and pieces in said  # every item said how many pieces it is; the longest all of them

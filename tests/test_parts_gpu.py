@@ -605,7 +605,7 @@ def test_position_part_and_unknown_kinds():
     assert torch.allclose(table[..., 0].cpu().double(), ang.cos(), atol=2e-7) and torch.allclose(table[..., 1].cpu().double(), ang.sin(), atol=2e-7)
     assert rope.prepare(Step) is table  # computed once per step, shared by the layers
     with pytest.raises(ValueError, match="no norm part of kind"):
-        build("norm", NormSpec("layernorm", 8, 1e-5), env(torch.float32))
+        build("norm", NormSpec("no_such_norm", 8, 1e-5), env(torch.float32))
 
 
 @pytest.mark.parametrize("dtype", [torch.float32, torch.bfloat16])

@@ -749,7 +749,7 @@ def test_heads_normed_over_their_whole_projection_and_placed(sizes, dtype):
 
 
 @pytest.mark.parametrize("dtype", ["float32", "bfloat16"])
-@pytest.mark.parametrize("sizes", [(96, 12, 50), (90, 5, 33), (256, 64, 300), (64, 1, 7)])
+@pytest.mark.parametrize("sizes", [(96, 12, 50), (90, 5, 33), (256, 64, 300), (64, 1, 7), (1032, 33, 40)])
 def test_token_inputs_alone(sizes, dtype):
     from types import SimpleNamespace
 
@@ -763,7 +763,7 @@ def test_token_inputs_alone(sizes, dtype):
     table = bf(torch.randn(vocab, dim, generator=gen))
     part = build("token_input", TokenInputSpec("gated_table", hidden, dim, vocab, NormSpec("rmsnorm", hidden, 1e-5)), env_for(dtype))
     give(part, {"table": table, "gate.weight": W["l0.side.gate"], "proj.weight": W["l0.side.proj"]}, dtype)
-    for T in (1, 7, 40, 150):
+    for T in (1, 2, 3, 7, 12, 16, 17, 40, 150):
         x, ids = bf(torch.randn(T, hidden, generator=gen) * 2), torch.randint(0, vocab, (T,), generator=gen)
         got = part.forward(x.to(DEV).to(DTYPES[dtype]), SimpleNamespace(token_ids=ids.to(I32).to(DEV))).float().cpu()
         args = ({k: v.double() for k, v in W.items()}, "l0.", table[ids].double(), 1e-5)
