@@ -2150,13 +2150,13 @@ STATE_SPACE_FILL = 2  # workgroups per compute unit up to which long rows are cu
 STATE_SPACE_MIN_SEGMENT = 64  # tokens
 
 
-def _state_space_segments(longest: int, num_rows: int, workgroups: int) -> int:
-    """Tokens of a segment for rows of up to `longest` tokens, a row or segment being `workgroups` workgroups (0: rows stay
-    whole): enough segments that they fill the GPU, since a row alone is a chain of chunks."""
-    want = STATE_SPACE_FILL * compute_units() // max(1, workgroups * num_rows)
-    if want < 2 or longest < 2 * STATE_SPACE_MIN_SEGMENT:
-        return 0
-    return max(STATE_SPACE_MIN_SEGMENT, _up32(-(-longest // want)))
+def _state_space_segments(longest: int, tokens: int, workgroups: int) -> int:
+    """Tokens of a segment for rows of up to `longest` tokens out of `tokens`, a row or segment being `workgroups` workgroups (0:
+    rows stay whole): segments of all rows together fill the GPU, and short rows beside a long one do not keep it whole (a row
+    alone is a chain of chunks); rows of less than two segments are not worth a second pass."""
+    fair = -(-tokens * workgroups // (STATE_SPACE_FILL * compute_units()))
+    seg = max(STATE_SPACE_MIN_SEGMENT, _up32(fair))
+    return seg if longest >= 2 * seg else 0
 
 
 def state_space(xbc, num_heads, groups, state_dim, vdim, proj, step_off, dt_bias, a_log, skip, state, step_rows, out, writes=True,
@@ -2199,7 +2199,7 @@ def state_space(xbc, num_heads, groups, state_dim, vdim, proj, step_off, dt_bias
     if kernel != "chunks":
         seg_len = 0
     elif seg_len is None:
-        seg_len = _state_space_segments(longest, R, G * -(-(H // G) * -(-E // 32) // 4))
+        seg_len = _state_space_segments(longest, T, G * -(-(H // G) * -(-E // 32) // 4))
     if seg_len:
         if seg_len < 0 or seg_len % 32:
             raise KernelError(f"state_space: segments of {seg_len} tokens (a multiple of 32)")

@@ -80,3 +80,13 @@ def test_how_products_of_17_to_128_rows_are_tiled():
     assert ops.gemm_split_plan(64, 4096, 4000, BF16) is None  # K in chunks of 256
     assert ops.gemm_split_plan(64, 4096, 4096, F32) is None
     assert [ops._gated_tile_strips(*case) for case in ((64, 12288), (64, 3072), (128, 25600))] == [6, 2, 8]
+
+
+def test_how_rows_of_a_state_space_are_cut_into_segments():
+    """One long row fills the GPU in segments, whatever short rows stand beside it; many rows of its length stay whole."""
+    choose = ops._state_space_segments
+    assert choose(2048, 2048, 64) == 256  # 128 heads of 64: 8 segments of 64 workgroups
+    assert choose(2041, 2048, 64) == 256 and choose(1700, 2048, 64) == 256  # beside decoding requests, behind another prompt's end
+    assert choose(512, 2048, 64) == 256 and choose(511, 2048, 64) == 0 and choose(256, 2048, 64) == 0
+    assert choose(2048, 2048, 8) == 64 and choose(200, 200, 1) == 64 and choose(100, 100, 1) == 0 and choose(0, 5, 1) == 0
+    assert choose(8192, 8192, 4096) == 0  # a row's own workgroups fill it
